@@ -10,6 +10,11 @@ each with a per-token shape and dtype of its own), indexed by the group's
 page ids. A request holds one *slot*: its row in every group's block
 table and its row of the state tensor.
 
+A mixer may keep something per block of tokens beside what it keeps per token (a
+CacheNeed's `blocks`, with a `stride`): such pools form groups of their own, in which an
+entry stands for `stride` tokens and a page is taken when the first whole block that lies in it
+is cached.
+
 Pages are given back when a request is released and, in a window group, as
 soon as the window has passed them: with n cached positions, the next query
 is at position >= n and sees keys >= n - window + 1, so every page whose last
@@ -38,12 +43,22 @@ class CacheGroup:
     allocator: PageAllocator
     page_size: int = 0                                    # tokens a page of this group holds
     max_pages: int = 0                                    # pages a request can hold at most
+    stride: int = 1                                       # tokens an entry of a page stands for
     instances: List[int] = field(default_factory=list)   # plan entries with pools in this group
+    pools: List[object] = field(default_factory=list)    # their tensors in this group
     tables: Dict[int, List[int]] = field(default_factory=dict)  # slot -> page of each logical page
     window_freed: int = 0
     # the same tables as rows of one array [slots, pages a request can hold], -1 where no page
     # is held: what a step copies its block table from
     rows: Optional[np.ndarray] = None
+
+    def pages_for(self, n: int) -> int:
+        """Pages (counted from a request's first) that hold what n tokens leave here."""
+        return -(-(n // self.stride) // self.page_size)
+
+    def max_tokens(self) -> int:
+        """Tokens that a block table of `max_pages` pages can stand for."""
+        return self.max_pages * self.page_size * self.stride
 
 
 class CacheManager:
@@ -60,23 +75,37 @@ class CacheManager:
         self.needs = list(needs)
         self.groups: List[CacheGroup] = []
         self.group_of_instance: Dict[int, int] = {}
-        by_kind: Dict[Tuple[Optional[int], int], int] = {}
-        for i, need in enumerate(self.needs):
-            if need is None:
+        self.block_group_of_instance: Dict[int, int] = {}   # ... of what is kept per block
+        by_kind: Dict[Tuple[Optional[int], int, int], int] = {}
+        for i, whole in enumerate(self.needs):
+            if whole is None:
                 continue
-            ps = need.page_size if need.page_size is not None else page_size
-            if ps < 1:
-                raise ValueError(f"a mixer asks for pages of {ps} tokens")
-            if (need.window, ps) not in by_kind:
-                by_kind[(need.window, ps)] = len(self.groups)
-                # `num_pages` counts pages of the engine's size: a group with pages of another
-                # size gets as many as hold the same number of tokens
-                n = num_pages if ps == page_size else max(1, num_pages * page_size // ps)
-                self.groups.append(CacheGroup(need.window, PageAllocator(n), page_size=ps,
-                                              max_pages=-(-max_context // ps)))
-            g = by_kind[(need.window, ps)]
-            self.groups[g].instances.append(i)
-            self.group_of_instance[i] = g
+            for need in whole.all_needs():
+                ps = need.page_size if need.page_size is not None else page_size
+                if ps < 1 or need.stride < 1:
+                    raise ValueError(f"a mixer asks for pages of {ps} entries of {need.stride} tokens")
+                if need is not whole and need.blocks is not None:
+                    raise ValueError("what is kept per block has no blocks of its own")
+                kind = (need.window, ps, need.stride)
+                if kind not in by_kind:
+                    by_kind[kind] = len(self.groups)
+                    most = max(1, -(-(max_context // need.stride) // ps))
+                    # `num_pages` counts pages of the engine's size: a group with pages of
+                    # another size gets as many as hold the same number of tokens
+                    n = num_pages if ps == page_size else max(1, num_pages * page_size // ps)
+                    if need.stride > 1:
+                        # entries of whole blocks: the same number of tokens, and a page that is
+                        # not full for every request
+                        n = min(-(-num_pages * page_size // (need.stride * ps)) + max_seqs,
+                                max_seqs * most)
+                    self.groups.append(CacheGroup(need.window, PageAllocator(n), page_size=ps,
+                                                  max_pages=most, stride=need.stride))
+                g = by_kind[kind]
+                self.groups[g].instances.append(i)
+                if need is whole:
+                    self.group_of_instance[i] = g
+                else:
+                    self.block_group_of_instance[i] = g
         for g in self.groups:
             g.rows = np.full((max_seqs, g.max_pages), -1, dtype=np.int32)
         self._free_slots: List[int] = list(range(max_seqs - 1, -1, -1))
@@ -96,12 +125,14 @@ class CacheManager:
         import torch
         self._ops = ops
         named = {"float32": torch.float32, "bfloat16": torch.bfloat16}
-        for i, need in enumerate(self.needs):
-            if need is None:
-                continue
-            group = self.groups[self.group_of_instance[i]]
+        for g in self.groups:
+            g.pools = []
+        homes = [(i, n, (self.group_of_instance if n is whole else self.block_group_of_instance)[i])
+                 for i, whole in enumerate(self.needs) if whole is not None for n in whole.all_needs()]
+        for i, need, g in homes:
+            group = self.groups[g]
             n = group.allocator.num_pages
-            self.pools[i] = {}
+            self.pools.setdefault(i, {})
             for spec in need.pools:
                 if spec.name in self.pools[i]:
                     raise ValueError(f"a mixer names two pools {spec.name!r}")
@@ -111,12 +142,15 @@ class CacheManager:
                 shape = (n, *spec.outer, group.page_size, *spec.inner)
                 self.pools[i][spec.name] = torch.zeros(
                     shape, dtype=named[spec.dtype] if spec.dtype else dtype, device=device)
+                group.pools.append(self.pools[i][spec.name])
         self.state = torch.zeros((self.max_seqs, max(self.state_floats, 1)),
                                  dtype=torch.float32, device=device)
 
     def drop_pools(self) -> None:
         """Give the device memory of every pool and of the state back (the end of an engine)."""
         self.pools = {}
+        for g in self.groups:
+            g.pools = []
         self.state = None
 
     # ---- slots ---------------------------------------------------------------
@@ -153,20 +187,19 @@ class CacheManager:
         g.allocator.free(pages)
         if self.poison_freed and pages and self.pools:
             import torch
-            for i in g.instances:
-                for pool in self.pools[i].values():
-                    idx = torch.tensor(pages, dtype=torch.int32, device=pool.device)
-                    if getattr(self, "_ops", None) is not None:
-                        self._ops.fill_nan_pages(pool, idx)
-                    else:   # no kernel library (host tests)
-                        pool.index_fill_(0, idx.long(), float("nan"))
+            for pool in g.pools:
+                idx = torch.tensor(pages, dtype=torch.int32, device=pool.device)
+                if getattr(self, "_ops", None) is not None:
+                    self._ops.fill_nan_pages(pool, idx)
+                else:   # no kernel library (host tests)
+                    pool.index_fill_(0, idx.long(), float("nan"))
 
     def length(self, slot: int) -> int:
         return self._length[slot]
 
     # ---- pages ---------------------------------------------------------------
     def pages_needed(self, slot: int, new_len: int) -> List[int]:
-        return [max(0, -(-new_len // g.page_size) - len(g.tables[slot])) for g in self.groups]
+        return [max(0, g.pages_for(new_len) - len(g.tables[slot])) for g in self.groups]
 
     def can_reserve(self, slot: int, new_len: int) -> bool:
         return all(n <= g.allocator.free_pages
@@ -246,10 +279,8 @@ class CacheManager:
 
     def kv_bytes_per_token(self, bytes_per_element: int) -> int:
         """Bytes of paged cache one token takes over all cache instances; pools without a
-        dtype of their own count `bytes_per_element` per number."""
-        own = {"float32": 4, "bfloat16": 2}
-        return sum(p.elements_per_token() * (own[p.dtype] if p.dtype else bytes_per_element)
-                   for n in self.needs if n is not None for p in n.pools)
+        dtype of their own count `bytes_per_element` per number, pools of blocks their share."""
+        return sum(n.bytes_per_token(bytes_per_element) for n in self.needs if n is not None)
 
     def pages_total(self, group: int = 0) -> int:
         return self.groups[group].allocator.num_pages

@@ -39,14 +39,27 @@ struct AttnArgs {
                             // [T, Hq*Dv] (0: the same as D)
   int sink;                 // != 0: the softmax's denominator has one more term, exp(0), that
                             // belongs to no key (a sink with score 0 and no value)
+  // Beside the keys of its window a row may see one key and value per block of `block` tokens
+  // that lies wholly before the window: block b (positions b block .. b block + block - 1) where
+  // b block + block - 1 <= position - window. Keys and blocks share one softmax.
+  const void* kblk;         // [pages, Hkv, blk_page_size, D], or null: no blocks
+  const void* vblk;         // [pages, Hkv, blk_page_size, Dv]
+  const int* blk_table;     // [S, blk_bt_stride]
+  int blk_bt_stride;
+  int blk_page_size;
+  int block;
+  // a gate on the output: out[t, c] times sigmoid(gate[t * gate_stride + c]), c < Hq * Dv
+  const void* gate;         // of the activation dtype, or null
+  int gate_stride;
 };
 
+// How many blocks a row at this position sees (they are the first ones of its request).
+__host__ __device__ inline int attention_blocks_seen(int pos, int window, int block) {
+  return pos >= window ? (pos - window + 1) / block : 0;
+}
+
 int attention_check(const AttnArgs& a);
-int attention_generic(const void* q, int q_stride, const void* kpool, const void* vpool,
-                      const int* block_table, int bt_stride, const int* positions,
-                      const int* row_seq, void* out, int T, int Hq, int Hkv, int D, int page_size,
-                      int window, float scale, const float* slopes, int dtype, int Dv, int sink,
-                      hipStream_t stream);
+int attention_generic(const AttnArgs& a, hipStream_t stream);
 
 int64_t attention_decode_workspace_floats(int T, int Hq, int D, int max_kv_len);
 bool attention_decode_takes(const AttnArgs& a);

@@ -24,6 +24,12 @@ int attention_check(const AttnArgs& args) {
   NINFER_REQUIRE(a->max_qlen >= 1 && a->max_kv_len >= 1, "paged_attention: bad size hints");
   NINFER_REQUIRE(a->single_rows >= 0 && a->single_rows <= a->S && a->single_rows <= a->T,
                  "paged_attention: %d single rows of %d requests", a->single_rows, a->S);
+  NINFER_REQUIRE(!a->kblk || (a->vblk && a->blk_table && a->blk_bt_stride > 0 && a->blk_page_size > 0 &&
+                              a->block > 0 && a->window > 0),
+                 "paged_attention: blocks of %d tokens before a window of %d", a->block, a->window);
+  NINFER_REQUIRE(!a->kblk || !a->slopes, "paged_attention: a position bias beside blocks is not built");
+  NINFER_REQUIRE(!a->gate || a->gate_stride >= a->Hq * (a->Dv > 0 ? a->Dv : a->D),
+                 "paged_attention: the gate's rows of %d are too short", a->gate_stride);
   return 0;
 }
 }  // namespace ninfer
@@ -55,7 +61,7 @@ extern "C" int ninfer_paged_attention(const AttnArgs* a, int force_generic, hipS
     return attention_prefill(p, stream);
   }
   if (!force_generic && attention_prefill_takes(*a)) return attention_prefill(*a, stream);
-  // keys and values of sizes of their own, a sink: row tiles of any such shape on the matrix
+  // keys and values of sizes of their own, a sink, blocks, a gate: row tiles of any such shape on the matrix
   // cores; single rows (which come first) with the heads of a kv head as a tile's rows
   if (!force_generic && attention_tiles_takes(*a)) {
     const int n = a->max_qlen == 1 ? a->S : a->single_rows;
@@ -70,10 +76,7 @@ extern "C" int ninfer_paged_attention(const AttnArgs* a, int force_generic, hipS
     }
     return attention_tiles(*a, 0, stream);
   }
-  return attention_generic(a->q, a->q_stride, a->kpool, a->vpool, a->block_table, a->bt_stride,
-                           a->positions, a->row_seq, a->out, a->T, a->Hq, a->Hkv, a->D,
-                           a->page_size, a->window, a->scale, a->slopes, a->dtype, a->Dv, a->sink,
-                           stream);
+  return attention_generic(*a, stream);
 }
 
 // 32-bit floats of workspace the split-KV decode kernel needs for this shape.

@@ -11,103 +11,104 @@
 // Scores, softmax and the value sum are 32-bit. This is the kernel of the true
 // 32-bit path and of head sizes the MFMA kernels refuse. Values may have another size than
 // keys (Dv), and the softmax may have a sink: one more term exp(0) in its denominator that
-// belongs to no key, so that the weights of a row add up to less than one.
-#include "common.h"
+// belongs to no key, so that the weights of a row add up to less than one. Where the cache keeps
+// one key and value per block of tokens, the blocks a row sees are walked first, in tiles of 64
+// too. The output may be gated, element by element.
+#include "attention.h"
 
 namespace ninfer {
 
 constexpr int kMaxDPerLane = 8;  // head sizes up to 512
 
 template <typename T>
-__global__ __launch_bounds__(64) void paged_attention_generic_kernel(
-    const T* __restrict__ q, int q_stride, const T* __restrict__ kpool,
-    const T* __restrict__ vpool, const int* __restrict__ block_table, int bt_stride,
-    const int* __restrict__ positions, const int* __restrict__ row_seq, T* __restrict__ out,
-    int Hq, int Hkv, int D, int page_size, int window, float scale,
-    const float* __restrict__ slopes, int Dv, int sink) {
+__global__ __launch_bounds__(64) void paged_attention_generic_kernel(AttnArgs a) {
   extern __shared__ float smem[];
+  const int D = a.D, Dv = a.Dv, Hkv = a.Hkv;
   float* q_s = smem;                 // [D]
   float* p_s = smem + D;             // [64]
   int64_t* off_s = (int64_t*)(p_s + 64);  // [64] page's slot (page * Hkv + g) * page_size + slot of each key
 
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
-  const int g = h / (Hq / Hkv);
-  const int pos = positions[t];
-  const int* bt = block_table + (int64_t)row_seq[t] * bt_stride;
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
-  const float slope = slopes ? slopes[h] : 0.f;
+  const int g = h / (a.Hq / Hkv);
+  const int pos = a.positions[t];
+  const float slope = a.slopes ? a.slopes[h] : 0.f;
 
-  const T* qr = q + (int64_t)t * q_stride + h * D;
+  const T* qr = (const T*)a.q + (int64_t)t * a.q_stride + h * D;
   for (int d = lane; d < D; d += 64) q_s[d] = to_f32(qr[d]);
   __syncthreads();
 
   // (a sink is a key with score 0 and no value: the running maximum starts at 0, the sum at 1)
-  float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+  float m = a.sink ? 0.f : -INFINITY, l = a.sink ? 1.f : 0.f;
   float acc[kMaxDPerLane];
 #pragma unroll
   for (int i = 0; i < kMaxDPerLane; ++i) acc[i] = 0.f;
 
-  for (int tile = (lo / 64) * 64; tile <= pos; tile += 64) {
-    int j = tile + lane;
-    bool valid = j >= lo && j <= pos;
-    float s = -INFINITY;
-    int64_t off = 0;
-    if (valid) {
-      int page = bt[j / page_size];
-      off = ((int64_t)page * Hkv + g) * page_size + (j % page_size);
-      const T* kr = kpool + off * D;
-      float dot = 0.f;
-      for (int d = 0; d < D; ++d) dot = fmaf(q_s[d], to_f32(kr[d]), dot);
-      s = fmaf(slope, (float)(j - pos), dot * scale);
-    }
-    float m_new = fmaxf(m, wave_max(s));
-    float p = valid ? expf(s - m_new) : 0.f;
-    float alpha = expf(m - m_new);  // 0 on the first tile (m = -inf)
-    l = l * alpha + wave_sum(p);
-    m = m_new;
-    p_s[lane] = p;
-    off_s[lane] = off;
-    __syncthreads();
-    int n_keys = min(64, pos - tile + 1);
-    int first = max(0, lo - tile);
-#pragma unroll
-    for (int i = 0; i < kMaxDPerLane; ++i) {
-      int d = lane + i * 64;
-      if (d < Dv) {
-        float a = acc[i] * alpha;
-        for (int jj = first; jj < n_keys; ++jj) a = fmaf(p_s[jj], to_f32(vpool[off_s[jj] * Dv + d]), a);
-        acc[i] = a;
+  // entries lo .. last of a pair of pools
+  auto walk = [&](const T* kpool, const T* vpool, const int* bt, int page_size, int lo, int last) {
+    for (int tile = (lo / 64) * 64; tile <= last; tile += 64) {
+      int j = tile + lane;
+      bool valid = j >= lo && j <= last;
+      float s = -INFINITY;
+      int64_t off = 0;
+      if (valid) {
+        int page = bt[j / page_size];
+        off = ((int64_t)page * Hkv + g) * page_size + (j % page_size);
+        const T* kr = kpool + off * D;
+        float dot = 0.f;
+        for (int d = 0; d < D; ++d) dot = fmaf(q_s[d], to_f32(kr[d]), dot);
+        s = fmaf(slope, (float)(j - pos), dot * a.scale);
       }
+      float m_new = fmaxf(m, wave_max(s));
+      float p = valid ? expf(s - m_new) : 0.f;
+      float alpha = expf(m - m_new);  // 0 on the first tile (m = -inf)
+      l = l * alpha + wave_sum(p);
+      m = m_new;
+      p_s[lane] = p;
+      off_s[lane] = off;
+      __syncthreads();
+      int n_keys = min(64, last - tile + 1);
+      int first = max(0, lo - tile);
+#pragma unroll
+      for (int i = 0; i < kMaxDPerLane; ++i) {
+        int d = lane + i * 64;
+        if (d < Dv) {
+          float x = acc[i] * alpha;
+          for (int jj = first; jj < n_keys; ++jj) x = fmaf(p_s[jj], to_f32(vpool[off_s[jj] * Dv + d]), x);
+          acc[i] = x;
+        }
+      }
+      __syncthreads();
     }
-    __syncthreads();
-  }
-  T* orow = out + ((int64_t)t * Hq + h) * Dv;
+  };
+  const int s = a.row_seq[t];
+  if (a.kblk)
+    walk((const T*)a.kblk, (const T*)a.vblk, a.blk_table + (int64_t)s * a.blk_bt_stride, a.blk_page_size, 0,
+         attention_blocks_seen(pos, a.window, a.block) - 1);
+  walk((const T*)a.kpool, (const T*)a.vpool, a.block_table + (int64_t)s * a.bt_stride, a.page_size,
+       a.window > 0 ? max(0, pos - a.window + 1) : 0, pos);
+  const int64_t orow = ((int64_t)t * a.Hq + h) * Dv;
+  const T* gate = a.gate ? (const T*)a.gate + (int64_t)t * a.gate_stride + h * Dv : nullptr;
   float inv = 1.f / l;
 #pragma unroll
   for (int i = 0; i < kMaxDPerLane; ++i) {
     int d = lane + i * 64;
-    if (d < Dv) orow[d] = from_f32<T>(acc[i] * inv);
+    if (d < Dv) {
+      float x = acc[i] * inv;
+      if (gate) x /= 1.f + expf(-to_f32(gate[d]));
+      ((T*)a.out)[orow + d] = from_f32<T>(x);
+    }
   }
 }
 
-int attention_generic(const void* q, int q_stride, const void* kpool, const void* vpool,
-                      const int* block_table, int bt_stride, const int* positions,
-                      const int* row_seq, void* out, int T, int Hq, int Hkv, int D, int page_size,
-                      int window, float scale, const float* slopes, int dtype, int Dv, int sink,
-                      hipStream_t stream) {
-  if (Dv <= 0) Dv = D;
-  NINFER_REQUIRE(D <= 64 * kMaxDPerLane && Dv <= 64 * kMaxDPerLane,
-                 "paged_attention: head sizes %d, %d exceed %d", D, Dv, 64 * kMaxDPerLane);
-  dim3 grid(T, Hq);
-  size_t lds = (D + 64) * sizeof(float) + 64 * sizeof(int64_t);
-  if (dtype == kF32)
-    paged_attention_generic_kernel<float><<<grid, 64, lds, stream>>>(
-        (const float*)q, q_stride, (const float*)kpool, (const float*)vpool, block_table, bt_stride,
-        positions, row_seq, (float*)out, Hq, Hkv, D, page_size, window, scale, slopes, Dv, sink);
-  else
-    paged_attention_generic_kernel<bf16><<<grid, 64, lds, stream>>>(
-        (const bf16*)q, q_stride, (const bf16*)kpool, (const bf16*)vpool, block_table, bt_stride,
-        positions, row_seq, (bf16*)out, Hq, Hkv, D, page_size, window, scale, slopes, Dv, sink);
+int attention_generic(const AttnArgs& args, hipStream_t stream) {
+  AttnArgs a = args;
+  if (a.Dv <= 0) a.Dv = a.D;
+  NINFER_REQUIRE(a.D <= 64 * kMaxDPerLane && a.Dv <= 64 * kMaxDPerLane,
+                 "paged_attention: head sizes %d, %d exceed %d", a.D, a.Dv, 64 * kMaxDPerLane);
+  dim3 grid(a.T, a.Hq);
+  size_t lds = (a.D + 64) * sizeof(float) + 64 * sizeof(int64_t);
+  if (a.dtype == kF32) paged_attention_generic_kernel<float><<<grid, 64, lds, stream>>>(a);
+  else paged_attention_generic_kernel<bf16><<<grid, 64, lds, stream>>>(a);
   NINFER_LAUNCH_CHECK();
   return 0;
 }

@@ -1,6 +1,8 @@
 // Softmax attention over the paged cache on the matrix cores (bf16 rows and cache) for keys of
-// D and values of Dv numbers (any multiples of 8 up to 128 each), with a window or none and with
-// a sink or none. The sizes the 64/128 kernels of attention_prefill.hip do not take run here.
+// D and values of Dv numbers (any multiples of 8 up to 128 each), with a window or none, with
+// a sink or none, with a gate on the output or none, and with or without one more key per block
+// of tokens before the window. What the 64/128 kernels of attention_prefill.hip do not take runs
+// here.
 //
 // Prompt portions: a block of four waves owns one kv head and a tile of rows of one request; a
 // wave owns 32 rows of one query head (HB = 4, 2 or 1 query heads of the kv head side by side,
@@ -25,6 +27,11 @@
 // maximum, sum and output of its own, and the two meet through LDS at the end. When rows and
 // kv heads alone do not fill the GPU, a row's visible keys are cut into chunks of whole tiles
 // over several blocks, whose records a second kernel merges.
+//
+// Where the cache keeps a key and value per block of tokens, a row's tiles are those of the
+// blocks it sees (64 blocks each, from the first), followed by those of its window's keys: the
+// block's index stands in the place of the key's position, and only the pools, the block table
+// and the bounds of what is visible change from one kind of tile to the other.
 //
 // No load stands under a condition: a key that is not there (beyond the last row's position,
 // or before the first key any row of the tile sees, whose page a window may have given back)
@@ -166,6 +173,35 @@ __device__ __forceinline__ void wave_keys(const unsigned short* ks_, const unsig
     }
 }
 
+// Where the tiles of one kind come from.
+struct TileSource {
+  const unsigned short* k;
+  const unsigned short* v;
+  const int* bt;
+  int page_size, ps_shift;
+};
+__device__ __forceinline__ TileSource tile_source(const AttnArgs& a, int seq, bool blocks) {
+  TileSource t;
+  t.k = (const unsigned short*)(blocks ? a.kblk : a.kpool);
+  t.v = (const unsigned short*)(blocks ? a.vblk : a.vpool);
+  t.bt = blocks ? a.blk_table + (int64_t)seq * a.blk_bt_stride : a.block_table + (int64_t)seq * a.bt_stride;
+  t.page_size = blocks ? a.blk_page_size : a.page_size;
+  t.ps_shift = __builtin_ctz(t.page_size);
+  return t;
+}
+
+__device__ __forceinline__ float at_sigmoid(float z) {
+  return 1.f / (1.f + __builtin_amdgcn_exp2f(-z * kAtLog2e));
+}
+// four neighbouring gates as factors
+__device__ __forceinline__ void at_gates(const unsigned short* p, float* f) {
+  const uint2 v = *(const uint2*)p;
+  f[0] = at_sigmoid(__uint_as_float(v.x << 16));
+  f[1] = at_sigmoid(__uint_as_float(v.x & 0xffff0000u));
+  f[2] = at_sigmoid(__uint_as_float(v.y << 16));
+  f[3] = at_sigmoid(__uint_as_float(v.y & 0xffff0000u));
+}
+
 template <int KS, int DB>
 __global__ __launch_bounds__(256, 2) void attention_tiles_kernel(AttnArgs a, int HB, int first_seq) {
   using Mover = TileMover<KS, DB, 256>;
@@ -199,11 +235,10 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_kernel(AttnArgs a, int
   if (seq < 0) return;
   const int pos_first = a.positions[row0], pos_last = pos_first + n_rows - 1;
   const int key_lo = a.window > 0 ? max(0, pos_first - a.window + 1) : 0;   // the first key any row sees
-  const int* bt = a.block_table + (int64_t)seq * a.bt_stride;
-  const int ps_shift = __builtin_ctz(a.page_size), ps_mask = a.page_size - 1;
   const int dim = a.D, vdim = a.Dv;
-  const unsigned short* kpool = (const unsigned short*)a.kpool;
-  const unsigned short* vpool = (const unsigned short*)a.vpool;
+  // blocks that the tile's last row sees, and the tiles of 64 that hold them
+  const int blocks_last = a.kblk ? attention_blocks_seen(pos_last, a.window, a.block) : 0;
+  const int n_bt = (blocks_last + 63) / 64;
 
   // zeros everywhere once: the padding columns stay zero, the rest is overwritten
   for (int i = tid; i < 2 * TILE / 8; i += 256) ((at_u32x4*)lds)[i] = at_u32x4{0u, 0u, 0u, 0u};
@@ -246,31 +281,44 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_kernel(AttnArgs a, int
   const int s16 = lane & 15, q4 = lane >> 4;
   const int v_lane = (4 * hi + s16 / 4) * VROW + 16 * (q4 & 1) + 4 * (s16 & 3);
 
-  const int kt0 = key_lo / 64, n_kt = pos_last / 64 + 1;
-  mv.load(kpool, vpool, bt, ps_shift, ps_mask, a.page_size, a.Hkv, g, dim, vdim, kt0 * 64, key_lo,
-          pos_last);
+  // tiles 0 .. n_bt - 1 hold blocks, those from n_bt on keys
+  const int kt0 = key_lo / 64, n_tiles = n_bt + pos_last / 64 + 1 - kt0;
+  TileSource src = tile_source(a, seq, n_bt > 0);
+  mv.load(src.k, src.v, src.bt, src.ps_shift, src.page_size - 1, src.page_size, a.Hkv, g, dim, vdim,
+          n_bt > 0 ? 0 : kt0 * 64, n_bt > 0 ? 0 : key_lo, n_bt > 0 ? blocks_last - 1 : pos_last);
+  const int row_blocks = a.kblk ? attention_blocks_seen(q_pos, a.window, a.block) : 0;
+  const int wave_blocks_first = a.kblk ? attention_blocks_seen(wave_first, a.window, a.block) : 0;
+  const int wave_blocks_last = a.kblk ? attention_blocks_seen(wave_last, a.window, a.block) : 0;
   __syncthreads();   // the zeros are written
-  for (int kt = kt0; kt < n_kt; ++kt) {
-    const int k0 = kt * 64, buf = (kt - kt0) & 1;
+  for (int it = 0; it < n_tiles; ++it) {
+    const bool is_b = it < n_bt;
+    const int k0 = (is_b ? it : kt0 + it - n_bt) * 64, buf = it & 1;
     mv.store(lds + buf * TILE);
     __syncthreads();
-    if (kt + 1 < n_kt)
-      mv.load(kpool, vpool, bt, ps_shift, ps_mask, a.page_size, a.Hkv, g, dim, vdim, k0 + 64, key_lo,
-              pos_last);
-    if (!wave_live || k0 > wave_last || k0 + 63 < wave_lo) continue;
+    if (it + 1 < n_tiles) {
+      if (it + 1 == n_bt) src = tile_source(a, seq, false);
+      const bool nb = it + 1 < n_bt;
+      mv.load(src.k, src.v, src.bt, src.ps_shift, src.page_size - 1, src.page_size, a.Hkv, g, dim, vdim,
+              (nb ? it + 1 : kt0 + it + 1 - n_bt) * 64, nb ? 0 : key_lo, nb ? blocks_last - 1 : pos_last);
+    }
+    if (!wave_live) continue;
+    if (is_b ? k0 >= wave_blocks_last : k0 > wave_last || k0 + 63 < wave_lo) continue;
     const unsigned short* ks_ = lds + buf * TILE;
     const unsigned short* vs_ = ks_ + 64 * KROW;
-    // some row of the wave does not see every key of the tile
-    const bool masked = k0 + 63 > wave_first || (a.window > 0 && k0 < wave_last - a.window + 1);
+    // some row of the wave does not see every key (or block) of the tile
+    const bool masked = is_b ? k0 + 64 > wave_blocks_first
+                             : k0 + 63 > wave_first || (a.window > 0 && k0 < wave_last - a.window + 1);
+    const int up_to = is_b ? row_blocks - 1 : q_pos, from = is_b ? 0 : lo_pos;
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb)
-      wave_keys<KS, DB>(ks_, vs_, kb, c, hi, v_lane, qf, pre, k0 + 32 * kb, q_pos, lo_pos, masked,
+      wave_keys<KS, DB>(ks_, vs_, kb, c, hi, v_lane, qf, pre, k0 + 32 * kb, up_to, from, masked,
                         m, l, o);
   }
   if (!q_valid) return;
   // lane holds, for row c, value columns 32 db + 8 (v / 4) + 4 hi + v % 4
   const float r = 1.f / l;
   unsigned short* orow = (unsigned short*)a.out + ((int64_t)(row0 + q_local) * a.Hq + h) * vdim;
+  const unsigned short* grow = a.gate ? (const unsigned short*)a.gate + (int64_t)(row0 + q_local) * a.gate_stride + h * vdim : nullptr;
 #pragma unroll
   for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -278,15 +326,21 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_kernel(AttnArgs a, int
       const int col = 32 * db + 8 * v4 + 4 * hi;
       if (col < vdim) {   // value sizes are multiples of 8: four columns are there together
         union { __bf16 b[4]; uint2 u; } w;
+        float f[4] = {r, r, r, r};
+        if (grow) {
+          at_gates(grow + col, f);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) w.b[e] = (__bf16)(o[db][4 * v4 + e] * r);
+          for (int e = 0; e < 4; ++e) f[e] *= r;
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) w.b[e] = (__bf16)(o[db][4 * v4 + e] * f[e]);
         *(uint2*)(orow + col) = w.u;
       }
     }
 }
 
 // `tiles_per_chunk`, `n_chunks`: the visible keys of a row are cut into chunks of so many tiles
-// (counted from the tile that holds the row's first visible key), one block each
+// (counted from the first tile of blocks, or from the one that holds the row's first visible key), one block each
 // (blockIdx.z), when rows and kv heads alone do not fill the GPU; every block then leaves a
 // record {m, l, o[Dv]} per head (m in units of log 2) that the merge kernel puts together.
 template <int KS, int DB>
@@ -305,10 +359,13 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
   const int dim = a.D, vdim = a.Dv;
   const bool q_valid = c < hpg;
   const int h = g * hpg + (q_valid ? c : 0);
-  const int kt0 = first / 64 + ch * tiles_per_chunk;
-  const int n_kt = min(pos / 64 + 1, kt0 + tiles_per_chunk);
+  // tiles 0 .. n_bt - 1 hold blocks, those from n_bt on keys; this chunk's are it0 .. it1 - 1
+  const int n_blocks = a.kblk ? attention_blocks_seen(pos, a.window, a.block) : 0;
+  const int n_bt = (n_blocks + 63) / 64, kt0 = first / 64;
+  const int it0 = ch * tiles_per_chunk;
+  const int it1 = min(n_bt + pos / 64 + 1 - kt0, it0 + tiles_per_chunk);
   float* rec = n_chunks > 1 ? a.workspace + (((int64_t)t * a.Hq + h) * n_chunks + ch) * (2 + vdim) : nullptr;
-  if (kt0 >= n_kt) {   // nothing of this chunk is visible: a record that counts for nothing
+  if (it0 >= it1) {   // nothing of this chunk is visible: a record that counts for nothing
     if (q_valid && kb == 0) {
       if (hi == 0) {
         rec[0] = -1e30f;
@@ -321,10 +378,7 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
     }
     return;
   }
-  const int* bt = a.block_table + (int64_t)a.row_seq[t] * a.bt_stride;
-  const int ps_shift = __builtin_ctz(a.page_size), ps_mask = a.page_size - 1;
-  const unsigned short* kpool = (const unsigned short*)a.kpool;
-  const unsigned short* vpool = (const unsigned short*)a.vpool;
+  const int seq = a.row_seq[t];
 
   for (int i = tid; i < TILE / 8; i += 128) ((at_u32x4*)lds)[i] = at_u32x4{0u, 0u, 0u, 0u};
   Mover mv;
@@ -353,19 +407,25 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
   const int s16 = lane & 15, q4 = lane >> 4;
   const int v_lane = (4 * hi + s16 / 4) * VROW + 16 * (q4 & 1) + 4 * (s16 & 3);
 
-  mv.load(kpool, vpool, bt, ps_shift, ps_mask, a.page_size, a.Hkv, g, dim, vdim, kt0 * 64, first, pos);
+  auto fetch = [&](int it) {
+    const bool is_b = it < n_bt;
+    const TileSource src = tile_source(a, seq, is_b);
+    mv.load(src.k, src.v, src.bt, src.ps_shift, src.page_size - 1, src.page_size, a.Hkv, g, dim, vdim,
+            (is_b ? it : kt0 + it - n_bt) * 64, is_b ? 0 : first, is_b ? n_blocks - 1 : pos);
+  };
+  fetch(it0);
   __syncthreads();
-  for (int kt = kt0; kt < n_kt; ++kt) {
-    const int k0 = kt * 64;
-    if (kt > kt0) __syncthreads();   // everyone has read the tile before: it may be written over
+  for (int it = it0; it < it1; ++it) {
+    const bool is_b = it < n_bt;
+    const int k0 = (is_b ? it : kt0 + it - n_bt) * 64;
+    if (it > it0) __syncthreads();   // everyone has read the tile before: it may be written over
     mv.store(lds);
     __syncthreads();
-    if (kt + 1 < n_kt)
-      mv.load(kpool, vpool, bt, ps_shift, ps_mask, a.page_size, a.Hkv, g, dim, vdim, k0 + 64, first, pos);
-    const int key0 = k0 + 32 * kb;
-    if (key0 > pos || key0 + 31 < first) continue;   // none of this wave's keys is visible
-    const bool masked = key0 + 31 > pos || key0 < first;
-    wave_keys<KS, DB>(lds, lds + 64 * KROW, kb, c, hi, v_lane, qf, pre, key0, pos, first, masked, m, l, o);
+    if (it + 1 < it1) fetch(it + 1);
+    const int key0 = k0 + 32 * kb, up_to = is_b ? n_blocks - 1 : pos, from = is_b ? 0 : first;
+    if (key0 > up_to || key0 + 31 < from) continue;   // none of this wave's keys is visible
+    const bool masked = key0 + 31 > up_to || key0 < from;
+    wave_keys<KS, DB>(lds, lds + 64 * KROW, kb, c, hi, v_lane, qf, pre, key0, up_to, from, masked, m, l, o);
   }
   // the two waves meet: the second leaves its maximum, sum and output in LDS, lane by lane
   // (both hold the same rows and columns in the same places), where the tile was
@@ -405,6 +465,7 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
   }
   const float r = 1.f / (l * f1 + l2 * f2);
   unsigned short* orow = (unsigned short*)a.out + ((int64_t)t * a.Hq + h) * vdim;
+  const unsigned short* grow = a.gate ? (const unsigned short*)a.gate + (int64_t)t * a.gate_stride + h * vdim : nullptr;
 #pragma unroll
   for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -412,9 +473,15 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
       const int col = 32 * db + 8 * v4 + 4 * hi;
       if (col < vdim) {
         union { __bf16 b[4]; uint2 u; } w;
+        float f[4] = {r, r, r, r};
+        if (grow) {
+          at_gates(grow + col, f);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) f[e] *= r;
+        }
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-          w.b[e] = (__bf16)((o[db][4 * v4 + e] * f1 + x_s[(2 + db * 16 + 4 * v4 + e) * 64 + lane] * f2) * r);
+          w.b[e] = (__bf16)((o[db][4 * v4 + e] * f1 + x_s[(2 + db * 16 + 4 * v4 + e) * 64 + lane] * f2) * f[e]);
         *(uint2*)(orow + col) = w.u;
       }
     }
@@ -451,10 +518,15 @@ __global__ __launch_bounds__(64) void attention_tiles_merge_kernel(AttnArgs a, i
   }
   const float inv = 1.f / wave_sum(l);
   __bf16* orow = (__bf16*)a.out + (int64_t)th * vdim;
+  const int t = th / a.Hq, h = th - t * a.Hq;
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
     const int d = lane + 64 * i;
-    if (d < vdim) orow[d] = (__bf16)(acc[i] * inv);
+    if (d < vdim) {
+      float x = acc[i] * inv;
+      if (a.gate) x *= at_sigmoid(to_f32(((const bf16*)a.gate)[(int64_t)t * a.gate_stride + h * vdim + d]));
+      orow[d] = (__bf16)x;
+    }
   }
 }
 
@@ -462,7 +534,8 @@ __global__ __launch_bounds__(64) void attention_tiles_merge_kernel(AttnArgs a, i
 // least two tiles a chunk.
 static void heads_plan(const AttnArgs& a, int* tiles_per_chunk, int* n_chunks) {
   const int span = a.window > 0 && a.window < a.max_kv_len ? a.window : a.max_kv_len;
-  const int tiles = span / 64 + 2;   // a span of keys that starts anywhere in a tile
+  // a span of keys that starts anywhere in a tile, and the blocks before the window
+  const int tiles = span / 64 + 2 + (a.kblk ? attention_blocks_seen(a.max_kv_len, a.window, a.block) / 64 + 1 : 0);
   const int blocks = a.T * a.Hkv;
   const int want = (4 * device_cu_count() + blocks - 1) / blocks;
   int per = (tiles + want - 1) / want;
@@ -482,6 +555,8 @@ bool attention_tiles_takes(const AttnArgs& a) {
   const int dv = a.Dv > 0 ? a.Dv : a.D;
   return a.dtype == kBF16 && a.D % 8 == 0 && dv % 8 == 0 && a.D <= 128 && dv <= 128 &&
          a.q_stride % 8 == 0 && (a.page_size & (a.page_size - 1)) == 0 && !a.slopes &&
+         (!a.kblk || (a.blk_page_size & (a.blk_page_size - 1)) == 0) &&
+         (!a.gate || (a.gate_stride % 4 == 0 && (uintptr_t)a.gate % 8 == 0)) &&
          a.seq_row_start != nullptr;
 }
 

@@ -6,7 +6,17 @@
 //   o_t = S_t^T (q_t q_scale)
 //
 // z comes in 32-bit (the decay's logits after their bias); the decay is formed here as
-// exp(log_sigmoid(z) / tau). The state comes from and returns to the request's slot, so a
+// exp(log_sigmoid(z) / tau).
+//
+// A second form of the same recurrence has a forget gate that also says how much is written, and
+// no keys of its own (`lower` given): from the gate's projected columns w and its bias b,
+//
+//   f_t = l + (1 - l) sigmoid(w_t + b),  S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T,
+//   o_t = S_t^T (silu(q_t) q_scale)
+//
+// with a lower bound l in [0, 1] per head and channel; 1 - f is formed as (1 - l) sigmoid(-w - b).
+//
+// The state comes from and returns to the request's slot, so a
 // request may be cut into steps anywhere and every row sees exactly the sums it would see in
 // one piece.
 //
@@ -41,9 +51,31 @@ struct GlaArgs {
   int stride, q_off, k_off, v_off;
   int H, dim, vdim;
   float inv_tau, q_scale;
+  // the form with a forget gate: its columns' first one, bias and lower bounds [H * dim] (z, k_off
+  // and inv_tau are not used then)
+  int f_off;
+  const float* f_bias;
+  const float* lower;
 };
 
-template <typename T, int DPL>
+// What a token brings to a key channel: how much of the state stays, what is written, and the
+// logarithm of the former.
+struct GlaGate {
+  float keep, write, log_keep;
+};
+// the forget gate's form from its logit (with bias) and lower bound
+__device__ __forceinline__ GlaGate forget_gate(float z, float lower) {
+  const float e = expf(-fabsf(z)), r = 1.f / (1.f + e);
+  const float up = z >= 0.f ? r : e * r, down = z >= 0.f ? e * r : r;   // sigmoid(z), sigmoid(-z)
+  GlaGate g;
+  g.keep = fmaf(1.f - lower, up, lower);
+  g.write = (1.f - lower) * down;
+  g.log_keep = fmaxf(log1pf(-g.write), -80.f);   // (exp(-80) is as good as nothing, and finite)
+  return g;
+}
+__device__ __forceinline__ float silu_f(float x) { return x / (1.f + expf(-x)); }
+
+template <typename T, int DPL, bool FORGET>
 __global__ __launch_bounds__(64 * kGlaWaves) void gla_seq_kernel(GlaArgs a) {
   constexpr int DIM = DPL * kGlaParts;            // channels held (>= dim; the rest stay 0)
   static_assert(DIM <= 64 * kGlaWaves, "a thread stages one channel");
@@ -66,14 +98,20 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_seq_kernel(GlaArgs a) {
   // tid looks after channel tid), and v of its column
   const bool stages = tid < DIM, in_dim = tid < dim;
   float fq[kGlaBatch], fk[kGlaBatch], fz[kGlaBatch], fv[kGlaBatch];
+  const float f_bias = FORGET && in_dim ? a.f_bias[h * dim + tid] : 0.f;
+  const float lower = FORGET && in_dim ? a.lower[h * dim + tid] : 0.f;
   auto fetch = [&](int first) {
 #pragma unroll
     for (int j = 0; j < kGlaBatch; ++j) {
       const int row = r0 + min(first + j, n - 1);   // (rows beyond the last are fetched again, not used)
       const T* r = (const T*)a.qkv + (int64_t)row * a.stride;
       fq[j] = in_dim ? to_f32(r[a.q_off + h * dim + tid]) : 0.f;
-      fk[j] = in_dim ? to_f32(r[a.k_off + h * dim + tid]) : 0.f;
-      fz[j] = in_dim ? a.z[((int64_t)row * a.H + h) * dim + tid] : 0.f;
+      if constexpr (FORGET) {
+        fz[j] = in_dim ? to_f32(r[a.f_off + h * dim + tid]) : 0.f;
+      } else {
+        fk[j] = in_dim ? to_f32(r[a.k_off + h * dim + tid]) : 0.f;
+        fz[j] = in_dim ? a.z[((int64_t)row * a.H + h) * dim + tid] : 0.f;
+      }
       fv[j] = has_col ? to_f32(r[a.v_off + h * vdim + col]) : 0.f;
     }
   };
@@ -82,9 +120,16 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_seq_kernel(GlaArgs a) {
     float cq[kGlaBatch], ck[kGlaBatch], ca[kGlaBatch], cv[kGlaBatch];
 #pragma unroll
     for (int j = 0; j < kGlaBatch; ++j) {
-      cq[j] = fq[j] * a.q_scale;
-      ck[j] = fk[j];
-      ca[j] = in_dim ? expf(log_sigmoid(fz[j]) * a.inv_tau) : 1.f;
+      if constexpr (FORGET) {
+        const GlaGate g = forget_gate(fz[j] + f_bias, lower);
+        cq[j] = silu_f(fq[j]) * a.q_scale;
+        ck[j] = in_dim ? g.write : 0.f;
+        ca[j] = in_dim ? g.keep : 1.f;
+      } else {
+        cq[j] = fq[j] * a.q_scale;
+        ck[j] = fk[j];
+        ca[j] = in_dim ? expf(log_sigmoid(fz[j]) * a.inv_tau) : 1.f;
+      }
       cv[j] = fv[j];
     }
     if (base + kGlaBatch < n) fetch(base + kGlaBatch);
@@ -127,12 +172,14 @@ using namespace ninfer;
 
 // qkv: [T, stride] rows of the activation dtype with the heads' q at column q_off, k at k_off
 // (heads x dim each) and v at v_off (heads x vdim); z: [T, heads * dim] 32-bit; out:
-// [T, heads * vdim] 32-bit.
+// [T, heads * vdim] 32-bit. With `lower` [heads * dim] the form with a forget gate: its columns
+// (heads x dim) at f_off, its bias f_bias [heads * dim]; z, k_off and tau are not read.
 extern "C" int ninfer_gated_linear_attention(const void* qkv, int stride, int q_off, int k_off,
                                              int v_off, const float* z, float tau, float q_scale,
                                              float* state, long long state_stride, float* out,
                                              const int* seq_row_start, const int* seq_slots,
                                              int T, int S, int H, int dim, int vdim, int dtype,
+                                             int f_off, const float* f_bias, const float* lower,
                                              hipStream_t stream) {
   NINFER_REQUIRE(T > 0 && S > 0 && H > 0 && dim > 0 && vdim > 0,
                  "gated_linear_attention: T=%d S=%d heads=%d dim=%d vdim=%d must be positive", T,
@@ -148,12 +195,19 @@ extern "C" int ninfer_gated_linear_attention(const void* qkv, int stride, int q_
   a.seq_row_start = seq_row_start, a.seq_slots = seq_slots, a.state_stride = state_stride;
   a.stride = stride, a.q_off = q_off, a.k_off = k_off, a.v_off = v_off;
   a.H = H, a.dim = dim, a.vdim = vdim, a.inv_tau = 1.f / tau, a.q_scale = q_scale;
+  a.f_off = f_off, a.f_bias = f_bias, a.lower = lower;
+  NINFER_REQUIRE(!lower == !f_bias && (lower || z), "gated_linear_attention: a forget gate without its bias, or no gate");
   const int cols = kGlaCols * kGlaWaves;
   const dim3 grid(S, H, (vdim + cols - 1) / cols);
-#define NINFER_GLA(DPL)                                                             \
-  do {                                                                              \
-    if (dtype == kF32) gla_seq_kernel<float, DPL><<<grid, 64 * kGlaWaves, 0, stream>>>(a);      \
-    else gla_seq_kernel<bf16, DPL><<<grid, 64 * kGlaWaves, 0, stream>>>(a);                     \
+#define NINFER_GLA(DPL)                                                                               \
+  do {                                                                                                \
+    if (lower) {                                                                                      \
+      if (dtype == kF32) gla_seq_kernel<float, DPL, true><<<grid, 64 * kGlaWaves, 0, stream>>>(a);    \
+      else gla_seq_kernel<bf16, DPL, true><<<grid, 64 * kGlaWaves, 0, stream>>>(a);                   \
+    } else {                                                                                          \
+      if (dtype == kF32) gla_seq_kernel<float, DPL, false><<<grid, 64 * kGlaWaves, 0, stream>>>(a);   \
+      else gla_seq_kernel<bf16, DPL, false><<<grid, 64 * kGlaWaves, 0, stream>>>(a);                  \
+    }                                                                                                 \
   } while (0)
   if (dim <= 16) NINFER_GLA(4);
   else if (dim <= 32) NINFER_GLA(8);
@@ -213,7 +267,7 @@ __device__ __forceinline__ bool gla_find_chunk(const int* seq_row_start, int S, 
   return false;
 }
 
-template <typename T>
+template <typename T, bool FORGET>
 __global__ __launch_bounds__(256) void gla_chunk_prepare_kernel(GlaChunkArgs a) {
   __shared__ float q_s[kGlaChunk][kGlaChunkMaxDim], k_s[kGlaChunk][kGlaChunkMaxDim];
   __shared__ float al_s[kGlaChunk][kGlaChunkMaxDim], b_s[kGlaChunk][kGlaChunkMaxDim];
@@ -225,14 +279,22 @@ __global__ __launch_bounds__(256) void gla_chunk_prepare_kernel(GlaChunkArgs a) 
   // 1. the rows' q, k and decays; rows beyond the chunk's last count as absent (k = 0, alpha = 1)
   for (int e = tid; e < kGlaChunk * dim; e += 256) {
     const int t = e / dim, d = e % dim;
-    float qv = 0.f, kv = 0.f, g = 0.f;
+    float qv = 0.f, kv = 0.f, g = 0.f, al = 1.f;
     if (t < L) {
       const T* r = (const T*)a.g.qkv + (int64_t)(base + t) * a.g.stride;
       qv = to_f32(r[a.g.q_off + h * dim + d]) * a.g.q_scale;
-      kv = to_f32(r[a.g.k_off + h * dim + d]);
-      g = log_sigmoid(a.g.z[((int64_t)(base + t) * H + h) * dim + d]) * a.g.inv_tau;
+      if constexpr (FORGET) {
+        const GlaGate f = forget_gate(to_f32(r[a.g.f_off + h * dim + d]) + a.g.f_bias[h * dim + d],
+                                      a.g.lower[h * dim + d]);
+        qv = silu_f(to_f32(r[a.g.q_off + h * dim + d])) * a.g.q_scale;
+        kv = f.write, g = f.log_keep, al = f.keep;
+      } else {
+        kv = to_f32(r[a.g.k_off + h * dim + d]);
+        g = log_sigmoid(a.g.z[((int64_t)(base + t) * H + h) * dim + d]) * a.g.inv_tau;
+        al = expf(g);
+      }
     }
-    q_s[t][d] = qv, k_s[t][d] = kv, al_s[t][d] = expf(g), b_s[t][d] = g;
+    q_s[t][d] = qv, k_s[t][d] = kv, al_s[t][d] = al, b_s[t][d] = g;
   }
   __syncthreads();
   // 2. b: the running sum of the logarithms, a channel per thread
@@ -419,7 +481,8 @@ extern "C" int ninfer_gated_linear_attention_chunks(const void* qkv, int stride,
                                                     long long state_stride, float* out,
                                                     const int* seq_row_start, const int* seq_slots,
                                                     float* work, int T, int S, int H, int dim,
-                                                    int vdim, int dtype, hipStream_t stream) {
+                                                    int vdim, int dtype, int f_off, const float* f_bias,
+                                                    const float* lower, hipStream_t stream) {
   NINFER_REQUIRE(T > 0 && S > 0 && H > 0 && dim > 0 && vdim > 0,
                  "gated_linear_attention: T=%d S=%d heads=%d dim=%d vdim=%d must be positive", T,
                  S, H, dim, vdim);
@@ -427,6 +490,7 @@ extern "C" int ninfer_gated_linear_attention_chunks(const void* qkv, int stride,
   NINFER_REQUIRE(state_stride >= (long long)H * dim * vdim,
                  "gated_linear_attention: a request's state of %lld floats holds no %d x %d x %d",
                  state_stride, H, dim, vdim);
+  NINFER_REQUIRE(!lower == !f_bias && (lower || z), "gated_linear_attention: a forget gate without its bias, or no gate");
   NINFER_REQUIRE(work != nullptr, "gated_linear_attention: the chunks need their workspace");
   if (dtype != kBF16 || dim > kGlaChunkMaxDim || dim % 4 != 0 || (uintptr_t)work % 16 != 0) return 1;
   GlaChunkArgs a;
@@ -437,8 +501,10 @@ extern "C" int ninfer_gated_linear_attention_chunks(const void* qkv, int stride,
   const int64_t thd = (int64_t)T * H * dim;
   a.qe = work, a.ke = work + thd, a.eb = work + 2 * thd, a.A = work + 3 * thd;
   a.T = T, a.S = S;
+  a.g.f_off = f_off, a.g.f_bias = f_bias, a.g.lower = lower;
   const int chunks = T / kGlaChunk + S;   // no step has more: each request adds at most one short chunk
-  gla_chunk_prepare_kernel<bf16><<<dim3(chunks, H), 256, 0, stream>>>(a);
+  if (lower) gla_chunk_prepare_kernel<bf16, true><<<dim3(chunks, H), 256, 0, stream>>>(a);
+  else gla_chunk_prepare_kernel<bf16, false><<<dim3(chunks, H), 256, 0, stream>>>(a);
   const int cols = kGlaCols * kGlaWaves;
   const dim3 grid(S, H, (vdim + cols - 1) / cols);
   if (dim <= 16) gla_chunk_scan_kernel<bf16, 1><<<grid, 64 * kGlaWaves, 0, stream>>>(a);

@@ -8,7 +8,11 @@
 //                  with the row's mean taken off first (a layer norm), and with y a weighted
 //                  sum of rows.
 //   gated_rmsnorm  out = o rsqrt(mean(o^2) + eps) w sigmoid(g) (or w g sigmoid(g)), the norm
-//                  over the whole row or over every group of columns (a head's) by itself.
+//                  over the whole row or over every group of columns (a head's) by itself;
+//                  without a gate the last factor is 1.
+//   post_norm      x <- z rsqrt(mean(z^2) + eps) g with z = alpha x + y, written in 32-bit and
+//                  once more in the activation dtype for whoever reads x next; y a row, a
+//                  weighted sum of rows, or half-and-half of two normed rows.
 //
 // All sums are 32-bit and their order depends on the row alone (taps ascending; the block
 // reduction's order depends on the width), never on how a request was cut or on the batch.
@@ -158,6 +162,144 @@ __global__ void norm_add_kernel(float* __restrict__ x, const T* __restrict__ y,
   }
 }
 
+// x <- norm(alpha x + y), norm(z) = z rsqrt(mean(z^2) + eps) gain; also as T into `out` when that
+// is given. y: a row of `y`; with `w` the weighted sum of k rows (as norm_add has it); with `y2`
+// factor * (rms(y) gain1 + rms(y2) gain2). The pieces of a row stay in registers throughout.
+struct PostNormArgs {
+  float* x;            // [T, H]
+  const void* y;       // [T, H], or [T k, H] with w
+  const void* y2;      // [T, H] or null
+  const float* gain1;  // [H] with y2
+  const float* gain2;
+  const float* w;      // [T, k] or null
+  const float* gain;   // [H]
+  void* out;           // [T, H] or null
+  int T;
+  int H;
+  int k;
+  int dtype;
+  float alpha;
+  float eps;
+  float factor;
+};
+
+// Two sums over a block at once; every thread gets both.
+__device__ __forceinline__ void block_sum2(float& u, float& v, float (*red)[2]) {
+  u = wave_sum(u);
+  v = wave_sum(v);
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, nw = (blockDim.x + 63) >> 6;
+  __syncthreads();
+  if (lane == 0) red[wv][0] = u, red[wv][1] = v;
+  __syncthreads();
+  u = v = 0.f;
+  for (int i = 0; i < nw; ++i) u += red[i][0], v += red[i][1];
+}
+
+template <typename T, int VEC>
+__global__ void post_norm_kernel(PostNormArgs a) {
+  constexpr int G = kNormAddPerThread / VEC;
+  __shared__ float red[16];
+  __shared__ float red2[16][2];
+  const int64_t r = blockIdx.x;
+  const int H = a.H;
+  const T* y = (const T*)a.y;
+  float* xr = a.x + r * H;
+  float z[G][VEC];
+  if (a.y2) {
+    const T* y2 = (const T*)a.y2;
+    float b[G][VEC];
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int c = 0; c < G; ++c) {
+      const int i = VEC * (threadIdx.x + c * blockDim.x);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) z[c][e] = b[c][e] = 0.f;
+      if (i < H) {
+        na_load<VEC>(y + r * H + i, z[c]);
+        na_load<VEC>(y2 + r * H + i, b[c]);
+      }
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) sa = fmaf(z[c][e], z[c][e], sa), sb = fmaf(b[c][e], b[c][e], sb);
+    }
+    block_sum2(sa, sb, red2);
+    const float ia = a.factor / sqrtf(sa / (float)H + a.eps), ib = a.factor / sqrtf(sb / (float)H + a.eps);
+#pragma unroll
+    for (int c = 0; c < G; ++c) {
+      const int i = VEC * (threadIdx.x + c * blockDim.x);
+      if (i < H) {
+        float ga[VEC], gb[VEC];
+        na_load<VEC>(a.gain1 + i, ga);
+        na_load<VEC>(a.gain2 + i, gb);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) z[c][e] = z[c][e] * ia * ga[e] + b[c][e] * ib * gb[e];
+      }
+    }
+  } else {
+#pragma unroll
+    for (int c = 0; c < G; ++c) {
+      const int i = VEC * (threadIdx.x + c * blockDim.x);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) z[c][e] = 0.f;
+      if (i < H) {
+        if (a.w) {
+          for (int j = 0; j < a.k; ++j) {
+            float yv[VEC];
+            na_load<VEC>(y + (r * a.k + j) * H + i, yv);
+            const float wj = a.w[r * a.k + j];
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) z[c][e] = fmaf(wj, yv[e], z[c][e]);
+          }
+        } else {
+          na_load<VEC>(y + r * H + i, z[c]);
+        }
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < G; ++c) {
+    const int i = VEC * (threadIdx.x + c * blockDim.x);
+    if (i < H) {
+      float xv[VEC];
+      na_load<VEC>(xr + i, xv);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        z[c][e] = fmaf(a.alpha, xv[e], z[c][e]);
+        ss = fmaf(z[c][e], z[c][e], ss);
+      }
+    }
+  }
+  ss = block_sum(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)H + a.eps);
+#pragma unroll
+  for (int c = 0; c < G; ++c) {
+    const int i = VEC * (threadIdx.x + c * blockDim.x);
+    if (i < H) {
+      float g[VEC];
+      na_load<VEC>(a.gain + i, g);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) z[c][e] *= inv * g[e];
+      if constexpr (VEC == 4) {
+        *(float4*)(xr + i) = make_float4(z[c][0], z[c][1], z[c][2], z[c][3]);
+      } else {
+        xr[i] = z[c][0];
+      }
+      if (a.out) {
+        T* o = (T*)a.out + r * H + i;
+        if constexpr (VEC == 4 && sizeof(T) == 2) {
+          union { __bf16 b[4]; uint2 u; } p;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) p.b[e] = (__bf16)z[c][e];
+          *(uint2*)o = p.u;
+        } else {
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) o[e] = from_f32<T>(z[c][e]);
+        }
+      }
+    }
+  }
+}
+
 template <typename T>
 __global__ void gated_rmsnorm_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                      int gate_stride, const float* __restrict__ w,
@@ -169,10 +311,10 @@ __global__ void gated_rmsnorm_kernel(const float* __restrict__ o, const T* __res
   for (int i = threadIdx.x; i < N; i += blockDim.x) ss = fmaf(orow[i], orow[i], ss);
   ss = block_sum(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)N + eps);
-  const T* g = gate + r * gate_stride;
+  const T* g = gate ? gate + r * gate_stride : nullptr;
   for (int i = threadIdx.x; i < N; i += blockDim.x) {
-    const float z = to_f32(g[i]);
-    const float sg = (silu ? z : 1.f) / (1.f + expf(-z));
+    const float z = g ? to_f32(g[i]) : 0.f;
+    const float sg = g ? (silu ? z : 1.f) / (1.f + expf(-z)) : 1.f;
     out[r * N + i] = from_f32<T>(orow[i] * inv * w[i] * sg);
   }
 }
@@ -190,10 +332,10 @@ __global__ __launch_bounds__(64) void gated_group_rmsnorm_kernel(
   for (int i = lane; i < group; i += 64) ss = fmaf(orow[i], orow[i], ss);
   ss = wave_sum(ss);
   const float inv = 1.f / sqrtf(ss / (float)group + eps);
-  const T* g = gate + r * gate_stride + g0;
+  const T* g = gate ? gate + r * gate_stride + g0 : nullptr;
   for (int i = lane; i < group; i += 64) {
-    const float z = to_f32(g[i]);
-    const float sg = (silu ? z : 1.f) / (1.f + expf(-z));
+    const float z = g ? to_f32(g[i]) : 0.f;
+    const float sg = g ? (silu ? z : 1.f) / (1.f + expf(-z)) : 1.f;
     out[r * N + g0 + i] = from_f32<T>(orow[i] * inv * w[i] * sg);
   }
 }
@@ -263,13 +405,37 @@ extern "C" int ninfer_norm_add(float* x, const void* y, const float* gain, int g
   return 0;
 }
 
+extern "C" int ninfer_post_norm(const PostNormArgs* args, hipStream_t stream) {
+  const PostNormArgs& a = *args;
+  NINFER_REQUIRE(a.T > 0 && a.H > 0 && a.x && a.y && a.gain, "post_norm: T=%d H=%d must be positive", a.T, a.H);
+  NINFER_REQUIRE(a.dtype == kF32 || a.dtype == kBF16, "post_norm: unknown dtype %d", a.dtype);
+  NINFER_REQUIRE(!a.w || a.k > 0, "post_norm: a weighted sum of %d rows", a.k);
+  NINFER_REQUIRE(!a.y2 || (a.gain1 && a.gain2 && !a.w), "post_norm: two normed rows need their gains and no weights");
+  auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  const bool vec = a.H % 4 == 0 && aligned(a.x) && aligned(a.y) && aligned(a.gain) && aligned(a.y2) &&
+                   aligned(a.gain1) && aligned(a.gain2) && aligned(a.out);
+  const int per_thread = vec ? 4 : 1;
+  int block = ((a.H + per_thread - 1) / per_thread + 63) / 64 * 64;
+  if (block > 1024) block = 1024;
+  NINFER_REQUIRE((int64_t)block * kNormAddPerThread >= a.H, "post_norm: width %d exceeds the kernel's", a.H);
+  if (a.dtype == kF32) {
+    if (vec) post_norm_kernel<float, 4><<<a.T, block, 0, stream>>>(a);
+    else post_norm_kernel<float, 1><<<a.T, block, 0, stream>>>(a);
+  } else {
+    if (vec) post_norm_kernel<bf16, 4><<<a.T, block, 0, stream>>>(a);
+    else post_norm_kernel<bf16, 1><<<a.T, block, 0, stream>>>(a);
+  }
+  NINFER_LAUNCH_CHECK();
+  return 0;
+}
+
 // group 0 (or N): the norm over the whole row with a weight of N numbers; else over every
 // group of `group` columns with a weight of `group` numbers. silu: the gate's factor is
 // g sigmoid(g) instead of sigmoid(g).
 extern "C" int ninfer_gated_rmsnorm(const float* o, const void* gate, int gate_stride,
                                     const float* w, void* out, int T, int N, float eps, int dtype,
                                     int group, int silu, hipStream_t stream) {
-  NINFER_REQUIRE(T > 0 && N > 0 && gate_stride >= N, "gated_rmsnorm: T=%d N=%d gate stride %d", T,
+  NINFER_REQUIRE(T > 0 && N > 0 && (!gate || gate_stride >= N), "gated_rmsnorm: T=%d N=%d gate stride %d", T,
                  N, gate_stride);
   NINFER_REQUIRE(dtype == kF32 || dtype == kBF16, "gated_rmsnorm: unknown dtype %d", dtype);
   NINFER_REQUIRE(group >= 0 && (group == 0 || N % group == 0),

@@ -72,9 +72,8 @@ class ModelRunner:
             n = spec.blocks[call.layer].state_floats()
             self._state_range.append(slice(floats, floats + n) if n else None)
             floats += n
-        own = {"float32": 4, "bfloat16": 2}
-        per_token = sum(p.elements_per_token() * own[p.dtype or options.dtype]
-                        for n in needs if n is not None for p in n.pools)
+        per_token = sum(n.bytes_per_token({"float32": 4, "bfloat16": 2}[options.dtype])
+                        for n in needs if n is not None)
         self.cache = CacheManager(needs, options.page_size, options.pool_pages(per_token),
                                   options.num_sequences, options.max_context, floats)
         for g in self.cache.groups:
@@ -184,7 +183,7 @@ class ModelRunner:
         # a graph is replayed for many steps: fixed table width, context rounded up
         if graph:
             max_kv_len = min(-(-max_kv_len // self.graph_context_step) * self.graph_context_step,
-                             min(g.max_pages * g.page_size for g in cache.groups)
+                             min(g.max_tokens() for g in cache.groups if g.stride == 1)
                              if cache.groups else cache.max_pages_per_request * cache.page_size)
         tables = [cache.block_table(g, slots, cache.groups[g].max_pages if graph else None)
                   for g in range(len(cache.groups))]
@@ -239,7 +238,7 @@ class ModelRunner:
         allocator counts as held; no page stands in two requests' rows. (The reference's
         analogue is the overflow throw of its slab, src/runtime/kv_cache.cpp:35-37.)"""
         for g, table in zip(self.cache.groups, tables):
-            ps = g.page_size
+            ps = g.page_size * g.stride   # tokens that a page stands for
             owner: Dict[int, int] = {}
             for i, (c, p) in enumerate(zip(chunks, pos0)):
                 row = table[i]
@@ -248,6 +247,10 @@ class ModelRunner:
                                        f"[0, {g.allocator.num_pages}): {row.tolist()}")
                 lo = 0 if g.window is None else max(0, p - g.window + 1)
                 last = p + len(c.tokens) - 1
+                if g.stride > 1:   # whole blocks only
+                    last = (last + 1) // g.stride * g.stride - 1
+                    if last < 0:
+                        continue
                 if last // ps >= row.shape[0]:
                     raise RuntimeError(f"slot {c.slot}: position {last} is beyond the block "
                                        f"table's {row.shape[0]} pages")
@@ -339,6 +342,11 @@ class ModelRunner:
                 g = cache.group_of_instance[owner]
                 view = CacheView(cache.pools[owner], d_tables[g], cache.groups[g].page_size,
                                  cache.groups[g].window)
+                b = cache.block_group_of_instance.get(owner)
+                if b is not None:
+                    group = cache.groups[b]
+                    view.blocks = CacheView(cache.pools[owner], d_tables[b], group.page_size,
+                                            group.window, stride=group.stride)
             rng = self._state_range[i]
             state = cache.state[:, rng] if rng is not None else None
             infos.append(CallInfo(cache=view, writes_cache=call.cache_from is None, state=state))

@@ -135,7 +135,7 @@ class Scheduler:
         positions, which lie in at most ceil(that / page) + 1 pages wherever they start."""
         for g in self.cache.groups:
             ps = g.page_size
-            most = -(-total // ps)
+            most = g.pages_for(total)
             if g.window is not None:
                 most = min(most, -(-(g.window + self.max_batch_tokens - 1) // ps) + 1)
             if most > g.allocator.num_pages:

@@ -80,7 +80,36 @@ class _AttnArgs(ctypes.Structure):
                 ("D", ctypes.c_int), ("page_size", ctypes.c_int), ("window", ctypes.c_int),
                 ("scale", ctypes.c_float), ("dtype", ctypes.c_int), ("max_qlen", ctypes.c_int),
                 ("max_kv_len", ctypes.c_int), ("single_rows", ctypes.c_int),
-                ("slopes", ctypes.c_void_p), ("Dv", ctypes.c_int), ("sink", ctypes.c_int)]
+                ("slopes", ctypes.c_void_p), ("Dv", ctypes.c_int), ("sink", ctypes.c_int),
+                ("kblk", ctypes.c_void_p), ("vblk", ctypes.c_void_p), ("blk_table", ctypes.c_void_p),
+                ("blk_bt_stride", ctypes.c_int), ("blk_page_size", ctypes.c_int),
+                ("block", ctypes.c_int), ("gate", ctypes.c_void_p), ("gate_stride", ctypes.c_int)]
+
+
+class _QkvWideArgs(ctypes.Structure):
+    _fields_ = [("u", ctypes.c_void_p), ("q_out", ctypes.c_void_p), ("kpool", ctypes.c_void_p),
+                ("vpool", ctypes.c_void_p), ("block_table", ctypes.c_void_p),
+                ("kblk", ctypes.c_void_p), ("vblk", ctypes.c_void_p), ("blk_table", ctypes.c_void_p),
+                ("positions", ctypes.c_void_p), ("row_seq", ctypes.c_void_p),
+                ("seq_row_start", ctypes.c_void_p), ("seq_pos0", ctypes.c_void_p),
+                ("q_gain", ctypes.c_void_p), ("k_gain", ctypes.c_void_p),
+                ("inv_freq", ctypes.c_void_p), ("head_scale", ctypes.c_void_p),
+                ("stride", ctypes.c_int), ("q_col", ctypes.c_int), ("k_col", ctypes.c_int),
+                ("v_col", ctypes.c_int), ("bt_stride", ctypes.c_int), ("blk_bt_stride", ctypes.c_int),
+                ("T", ctypes.c_int), ("S", ctypes.c_int), ("Hq", ctypes.c_int), ("Hkv", ctypes.c_int),
+                ("dim", ctypes.c_int), ("vdim", ctypes.c_int), ("rot_dim", ctypes.c_int),
+                ("interleaved", ctypes.c_int), ("page_size", ctypes.c_int),
+                ("blk_page_size", ctypes.c_int), ("block", ctypes.c_int), ("dtype", ctypes.c_int),
+                ("eps", ctypes.c_float), ("magnitude", ctypes.c_float), ("all_single", ctypes.c_int),
+                ("force_plain", ctypes.c_int)]
+
+
+class _PostNormArgs(ctypes.Structure):
+    _fields_ = [("x", ctypes.c_void_p), ("y", ctypes.c_void_p), ("y2", ctypes.c_void_p),
+                ("gain1", ctypes.c_void_p), ("gain2", ctypes.c_void_p), ("w", ctypes.c_void_p),
+                ("gain", ctypes.c_void_p), ("out", ctypes.c_void_p), ("T", ctypes.c_int),
+                ("H", ctypes.c_int), ("k", ctypes.c_int), ("dtype", ctypes.c_int),
+                ("alpha", ctypes.c_float), ("eps", ctypes.c_float), ("factor", ctypes.c_float)]
 
 
 class _QkvConvArgs(ctypes.Structure):
@@ -896,14 +925,18 @@ class HipOps:
     # ---- attention ------------------------------------------------------------------
     def paged_attention(self, qkv, k_pool, v_pool, block_table, ctx, n_q, n_kv, head_dim,
                         page_size, window, scale, out, plan_only=False, slopes=None, vdim=None,
-                        sink=False):
+                        sink=False, blocks=None, gate=None):
         """Attention of the rows' query heads (the first n_q * head_dim columns
         of `qkv`) over their requests' cached keys and values. `slopes` [n_q] (32-bit): head
         h's scores get slopes[h] * (key's position - row's position) added before the softmax
         (a distance-based position bias; negative distances, so a positive slope favours near
         keys). `vdim`: numbers of a value head when they differ from a key head's (`v_pool` and
         `out` are that wide). `sink`: the softmax's denominator has one more term, exp(0), that
-        belongs to no key. `plan_only`: launch
+        belongs to no key. `blocks` (a CacheView's `blocks` with pools 'k_block' and 'v_block'
+        [.., n_kv, its page size, head_dim or vdim]): one more key and value for every block of
+        `blocks.stride` tokens that lies wholly before the window, in the same softmax. `gate`
+        ([T, n_q * vdim] columns of a wider row-major tensor, a view): the output is multiplied
+        by sigmoid(gate), element by element. `plan_only`: launch
         nothing and say how a step of single-token rows of this shape would run
         (which split-context kernel, keys per chunk, chunks)."""
         vdim = head_dim if vdim is None else int(vdim)
@@ -946,6 +979,16 @@ class HipOps:
             ws, ws_floats, qkv.shape[1], block_table.shape[1], t, ctx.S, n_q, n_kv, head_dim, page_size,
             int(window or 0), float(scale), _DT[qkv.dtype], ctx.max_qlen, ctx.max_kv_len, single,
             _ptr(slopes), vdim, 1 if sink else 0)
+        if blocks is not None:
+            self._blocks_fit(blocks, qkv.dtype, n_kv, head_dim, vdim, ctx, "paged_attention")
+            args.kblk, args.vblk = blocks["k_block"].data_ptr(), blocks["v_block"].data_ptr()
+            args.blk_table, args.blk_bt_stride = blocks.block_table.data_ptr(), blocks.block_table.shape[1]
+            args.blk_page_size, args.block = blocks.page_size, blocks.stride
+        if gate is not None:
+            _need(gate.is_cuda and gate.dtype == qkv.dtype and gate.shape == out.shape
+                  and gate.stride(1) == 1, "paged_attention: the gate must be [T, n_q * vdim] columns of rows")
+            args.gate = gate.data_ptr()
+            args.gate_stride = gate.stride(0) if t > 1 else max(out.shape[1], gate.stride(0))
         if plan_only:
             kernel, chunk, n_chunks = ctypes.c_int(), ctypes.c_int(), ctypes.c_int()
             self._ok(self.lib.ninfer_attention_decode_plan(
@@ -955,6 +998,69 @@ class HipOps:
                     "chunks": n_chunks.value}
         self._ok(self.lib.ninfer_paged_attention(ctypes.byref(args),
                                                  1 if self.force_generic else 0, self._stream()))
+
+    @staticmethod
+    def _blocks_fit(blocks, dtype, n_kv, dim, vdim, ctx, who):
+        for name, n in (("k_block", dim), ("v_block", vdim)):
+            _dev(blocks[name], name, dtype, 4)
+            _need(blocks[name].shape[1:] == (n_kv, blocks.page_size, n)
+                  and blocks[name].shape[0] == blocks["k_block"].shape[0],
+                  f"{who}: the pools of blocks do not fit the head layout")
+        _dev(blocks.block_table, "blocks.block_table", torch.int32, 2)
+        _need(blocks.block_table.shape[0] == ctx.S and blocks.stride >= 1,
+              f"{who}: block table rows of blocks != requests")
+
+    def qkv_wide(self, u, ctx, q_out, heads, kv_heads, dim, vdim, k_pool, v_pool, block_table,
+                 page_size, v_col=None, q_norm=None, k_norm=None, norm_eps=0.0, inv_freq=None,
+                 rot_dim=0, interleaved=False, magnitude=1.0, head_scale=None, blocks=None):
+        """Projected rows u ([T, C] columns of a wider row-major tensor: heads x dim queries,
+        kv_heads x dim keys, and from column `v_col` on kv_heads x vdim values; None: behind the
+        keys; the keys' own first column: values that are the keys as projected) on their way to
+        attention: queries and keys normed over their whole projections (gains `q_norm`
+        [heads * dim], `k_norm` [kv_heads * dim], None: no norm), turned by their position with
+        cosine and sine times `magnitude`, query heads times `head_scale` [heads] (32-bit);
+        queries to `q_out`, keys and values to the requests' pages. `blocks` (see
+        `paged_attention`): the means of the cached keys and values of every block of tokens
+        that this step completes go to its pools."""
+        _need(u.is_cuda and u.dim() == 2 and u.stride(1) == 1 and u.dtype in _DT,
+              "qkv_wide: u must be columns of rows")
+        _dev(q_out, "q_out", u.dtype, 2)
+        _dev(k_pool, "k_pool", u.dtype, 4)
+        _dev(v_pool, "v_pool", u.dtype, 4)
+        _dev(block_table, "block_table", torch.int32, 2)
+        t, nq, nk, nv = ctx.T, heads * dim, kv_heads * dim, kv_heads * vdim
+        v_col = nq + nk if v_col is None else int(v_col)
+        _need(u.shape[0] == t and u.shape[1] >= max(nq + nk, v_col + nv) and v_col >= 0
+              and q_out.shape == (t, nq), f"qkv_wide: rows of {tuple(u.shape)} do not hold the heads")
+        _need(k_pool.shape[0] == v_pool.shape[0] and k_pool.shape[1:] == (kv_heads, page_size, dim)
+              and v_pool.shape[1:] == (kv_heads, page_size, vdim) and block_table.shape[0] == ctx.S,
+              "qkv_wide: pools or block table do not fit the head layout")
+        for g, n, name in ((q_norm, nq, "q_norm"), (k_norm, nk, "k_norm"), (head_scale, heads, "head_scale"),
+                           (inv_freq if rot_dim else None, rot_dim // 2, "inv_freq")):
+            if g is not None:
+                _dev(g, name, torch.float32, 1)
+                _need(g.shape[0] == n, f"qkv_wide: {name} has {g.shape[0]} numbers, not {n}")
+        _need(rot_dim == 0 or (inv_freq is not None and rot_dim <= dim), "qkv_wide: rotation without a table")
+        a = _QkvWideArgs()
+        a.u, a.q_out, a.kpool, a.vpool = u.data_ptr(), q_out.data_ptr(), k_pool.data_ptr(), v_pool.data_ptr()
+        a.block_table, a.bt_stride = block_table.data_ptr(), block_table.shape[1]
+        if blocks is not None:
+            self._blocks_fit(blocks, u.dtype, kv_heads, dim, vdim, ctx, "qkv_wide")
+            a.kblk, a.vblk = blocks["k_block"].data_ptr(), blocks["v_block"].data_ptr()
+            a.blk_table, a.blk_bt_stride = blocks.block_table.data_ptr(), blocks.block_table.shape[1]
+            a.blk_page_size, a.block = blocks.page_size, blocks.stride
+        a.positions, a.row_seq = ctx.positions.data_ptr(), ctx.row_seq.data_ptr()
+        a.seq_row_start, a.seq_pos0 = ctx.seq_row_start.data_ptr(), ctx.seq_pos0.data_ptr()
+        a.q_gain, a.k_gain, a.head_scale = _ptr(q_norm), _ptr(k_norm), _ptr(head_scale)
+        a.inv_freq = inv_freq.data_ptr() if rot_dim else None
+        a.stride = u.stride(0) if t > 1 else max(u.shape[1], u.stride(0))
+        a.q_col, a.k_col, a.v_col = 0, nq, v_col
+        a.T, a.S, a.Hq, a.Hkv, a.dim, a.vdim = t, ctx.S, heads, kv_heads, dim, vdim
+        a.rot_dim, a.interleaved, a.page_size = rot_dim, 1 if interleaved else 0, page_size
+        a.dtype, a.eps, a.magnitude = _DT[u.dtype], norm_eps, magnitude
+        a.all_single = 1 if ctx.max_qlen == 1 else 0
+        a.force_plain = 1 if self.force_generic else 0
+        self._ok(self.lib.ninfer_qkv_wide(ctypes.byref(a), self._stream()))
 
     def qkv_conv(self, u, w_conv, state, ctx, q_out, heads, kv_heads, dim, vdim, k_pool, v_pool,
                  block_table, page_size, q_norm=None, k_norm=None, norm_eps=0.0, inv_freq=None,
@@ -1075,12 +1181,50 @@ class HipOps:
             ctypes.c_float(eps), _DT[y.dtype], 1 if center else 0,
             ctypes.c_void_p(_ptr(weights)), k, self._stream()))
 
+    def post_norm(self, residual, y, gain, eps, alpha, out=None, weights=None):
+        """residual <- norm(alpha residual + y) in 32-bit, norm(z) = z rsqrt(mean(z^2) + eps)
+        gain, gain [H]; the same into `out` [T, H] (y's dtype) when it is given. y: rows [T, H];
+        with `weights` [T, k] (32-bit) T * k rows that stand for their weighted sums, as in
+        `norm_add`; or a NormedSum (two rows normed by themselves, formed in 32-bit here)."""
+        _dev(residual, "residual", torch.float32, 2)
+        _dev(gain, "gain", torch.float32, 1)
+        t, h = residual.shape
+        _need(gain.shape[0] == h, "post_norm: one gain per column")
+        a = _PostNormArgs()
+        first = y
+        if hasattr(y, "gain_b"):
+            _need(weights is None and y.eps == eps, "post_norm: two normed rows share the norm's eps")
+            for v in (y.a, y.b):
+                _dev(v, "y", y.a.dtype, 2)
+                _need(v.shape == (t, h), "post_norm: y does not fit the residual")
+            for g in (y.gain_a, y.gain_b):
+                _dev(g, "gain", torch.float32, 1)
+                _need(g.shape[0] == h, "post_norm: one gain per column")
+            first = y.a
+            a.y2, a.gain1, a.gain2, a.factor = y.b.data_ptr(), y.gain_a.data_ptr(), y.gain_b.data_ptr(), y.factor
+        else:
+            _dev(y, "y", dims=2)
+            k = 1
+            if weights is not None:
+                _dev(weights, "weights", torch.float32, 2)
+                k = weights.shape[1]
+                _need(weights.shape[0] == t, "post_norm: the weights do not fit the residual")
+                a.w, a.k = weights.data_ptr(), k
+            _need(y.shape == (t * k, h), "post_norm: y does not fit the residual")
+        _need(first.dtype in _DT, "post_norm: y's dtype")
+        if out is not None:
+            _dev(out, "out", first.dtype, 2)
+            _need(out.shape == (t, h), "post_norm: out does not fit the residual")
+        a.x, a.y, a.gain, a.out = residual.data_ptr(), first.data_ptr(), gain.data_ptr(), _ptr(out)
+        a.T, a.H, a.dtype, a.alpha, a.eps = t, h, _DT[first.dtype], float(alpha), float(eps)
+        self._ok(self.lib.ninfer_post_norm(ctypes.byref(a), self._stream()))
+
     def gated_rmsnorm(self, o, gate, weight, eps, out, group=0, gate_act="sigmoid"):
         """out = o rsqrt(mean(o^2) + eps) weight sigmoid(gate), the mean over the whole row, or
         with `group` over every group of so many neighbouring columns by itself (`weight` then
         has `group` numbers, shared by the groups). `gate_act` 'silu': gate sigmoid(gate) in
         place of sigmoid(gate). o: [T, N] 32-bit; gate: [T, N] columns of a wider row-major
-        tensor (a view)."""
+        tensor (a view), or None for no gate (factor 1)."""
         _dev(o, "o", torch.float32, 2)
         _dev(weight, "weight", torch.float32, 1)
         _dev(out, "out", dims=2)
@@ -1089,11 +1233,11 @@ class HipOps:
         _need(group >= 0 and (group == 0 or n % group == 0), "gated_rmsnorm: groups do not fill the rows")
         _need(out.shape == (t, n) and weight.shape[0] == (group or n) and out.dtype in _DT,
               "gated_rmsnorm: shapes")
-        _need(gate.is_cuda and gate.dtype == out.dtype and gate.shape == (t, n)
-              and gate.stride(1) == 1, "gated_rmsnorm: the gate must be [T, N] columns of rows")
+        _need(gate is None or (gate.is_cuda and gate.dtype == out.dtype and gate.shape == (t, n)
+              and gate.stride(1) == 1), "gated_rmsnorm: the gate must be [T, N] columns of rows")
         self._ok(self.lib.ninfer_gated_rmsnorm(
-            ctypes.c_void_p(o.data_ptr()), ctypes.c_void_p(gate.data_ptr()),
-            gate.stride(0) if t > 1 else max(n, gate.stride(0)),
+            ctypes.c_void_p(o.data_ptr()), ctypes.c_void_p(_ptr(gate)),
+            0 if gate is None else gate.stride(0) if t > 1 else max(n, gate.stride(0)),
             ctypes.c_void_p(weight.data_ptr()), ctypes.c_void_p(out.data_ptr()), t, n,
             ctypes.c_float(eps), _DT[out.dtype], int(group), 1 if gate_act == "silu" else 0,
             self._stream()))
@@ -1441,7 +1585,7 @@ class HipOps:
         return 3 * heads * dim + 16 * heads
 
     def gated_linear_attention(self, qkv, q_off, k_off, v_off, z, heads, dim, vdim, tau, q_scale,
-                               state, ctx, out, work=None):
+                               state, ctx, out, work=None, forget=None):
         """Linear attention with a decay per key channel and token over the rows of each
         request: S <- diag(alpha) S + k v^T, out = S^T (q q_scale) with alpha =
         sigmoid(z)^(1 / tau), q, k at the columns q_off, k_off (heads x dim) and v at v_off
@@ -1450,15 +1594,28 @@ class HipOps:
         `work` ([T, gla_work_floats(..)] 32-bit, or None): with it a bfloat16 step that brings
         prompt portions runs in chunks of 16 rows on the matrix cores (the sums of a chunk are
         ordered otherwise than token by token, so the 32-bit path, whose logits do not depend
-        on the cut to the bit, stays on the token-by-token kernel)."""
-        _dev(qkv, "qkv", dims=2)
-        _dev(z, "z", torch.float32, 2)
+        on the cut to the bit, stays on the token-by-token kernel). `forget` (f_off, bias,
+        lower): the form with a forget gate f = lower + (1 - lower) sigmoid(w + bias), w the
+        columns f_off (heads x dim) of `qkv`, bias and lower [heads * dim] (32-bit):
+        S <- diag(f) S + (1 - f) v^T, out = S^T (silu(q) q_scale); z, k_off and tau are not
+        used (None, 0, 1). `qkv` may be columns of a wider row-major tensor."""
+        _need(qkv.is_cuda and qkv.dim() == 2 and qkv.stride(1) == 1, "gated_linear_attention: qkv must be columns of rows")
         _dev(out, "out", torch.float32, 2)
         t = qkv.shape[0]
+        row = qkv.stride(0) if t > 1 else max(qkv.shape[1], qkv.stride(0))
         _need(qkv.dtype in _DT, f"gated_linear_attention: rows of {qkv.dtype}")
-        _need(z.shape == (t, heads * dim) and out.shape == (t, heads * vdim) and ctx.T == t,
-              "gated_linear_attention: shapes")
-        for off, n in ((q_off, heads * dim), (k_off, heads * dim), (v_off, heads * vdim)):
+        _need(out.shape == (t, heads * vdim) and ctx.T == t, "gated_linear_attention: shapes")
+        f_off, f_bias, lower = forget if forget is not None else (0, None, None)
+        if forget is None:
+            _dev(z, "z", torch.float32, 2)
+            _need(z.shape == (t, heads * dim), "gated_linear_attention: shapes")
+        else:
+            for g, name in ((f_bias, "bias"), (lower, "lower")):
+                _dev(g, name, torch.float32, 1)
+                _need(g.shape[0] == heads * dim, f"gated_linear_attention: {name} has one number per channel")
+        gate_args = (int(f_off), ctypes.c_void_p(_ptr(f_bias)), ctypes.c_void_p(_ptr(lower)))
+        for off, n in ((q_off, heads * dim), (k_off if forget is None else f_off, heads * dim),
+                       (v_off, heads * vdim)):
             _need(0 <= off and off + n <= qkv.shape[1], "gated_linear_attention: columns outside the rows")
         _need(state.is_cuda and state.dtype == torch.float32 and state.dim() == 2
               and state.stride(1) == 1 and state.shape[1] >= heads * dim * vdim,
@@ -1469,23 +1626,23 @@ class HipOps:
                   and work.shape[1] >= 3 * heads * dim + 16 * heads,
                   "gated_linear_attention: the workspace is too small")
             rc = self.lib.ninfer_gated_linear_attention_chunks(
-                ctypes.c_void_p(qkv.data_ptr()), qkv.shape[1], q_off, k_off, v_off,
-                ctypes.c_void_p(z.data_ptr()), ctypes.c_float(tau), ctypes.c_float(q_scale),
+                ctypes.c_void_p(qkv.data_ptr()), row, q_off, k_off, v_off,
+                ctypes.c_void_p(_ptr(z)), ctypes.c_float(tau), ctypes.c_float(q_scale),
                 ctypes.c_void_p(state.data_ptr()), ctypes.c_longlong(state.stride(0)),
                 ctypes.c_void_p(out.data_ptr()), ctypes.c_void_p(ctx.seq_row_start.data_ptr()),
                 ctypes.c_void_p(ctx.seq_slots.data_ptr()), ctypes.c_void_p(work.data_ptr()),
-                t, ctx.S, heads, dim, vdim, _DT[qkv.dtype], self._stream())
+                t, ctx.S, heads, dim, vdim, _DT[qkv.dtype], *gate_args, self._stream())
             if rc == 0:
                 return
             if rc < 0:
                 self._ok(rc)
         self._ok(self.lib.ninfer_gated_linear_attention(
-            ctypes.c_void_p(qkv.data_ptr()), qkv.shape[1], q_off, k_off, v_off,
-            ctypes.c_void_p(z.data_ptr()), ctypes.c_float(tau), ctypes.c_float(q_scale),
+            ctypes.c_void_p(qkv.data_ptr()), row, q_off, k_off, v_off,
+            ctypes.c_void_p(_ptr(z)), ctypes.c_float(tau), ctypes.c_float(q_scale),
             ctypes.c_void_p(state.data_ptr()), ctypes.c_longlong(state.stride(0)),
             ctypes.c_void_p(out.data_ptr()), ctypes.c_void_p(ctx.seq_row_start.data_ptr()),
             ctypes.c_void_p(ctx.seq_slots.data_ptr()), t, ctx.S, heads, dim, vdim, _DT[qkv.dtype],
-            self._stream()))
+            *gate_args, self._stream()))
 
     def sigmoid_attention(self, qkv, k_pool, v_pool, block_table, ctx, heads, kv_heads, dim, vdim,
                           page_size, scale, chunk, head_bias, mix, out, write_kv=True):

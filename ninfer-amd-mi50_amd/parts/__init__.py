@@ -1,18 +1,21 @@
 from .attention import Attention
 from .base import (Block, CacheNeed, CacheView, CallInfo, FeedForward, Mixer, Norm, Part,
-                   PendingRows, PoolSpec, PositionEncoding, StepContext, WeightBinder, settle)
-from .block import OutputNormBlock, ParallelBlock, PreNormBlock, SandwichBlock
+                   NormedSum, PendingRows, PoolSpec, PositionEncoding, ReadyRows, StepContext,
+                   WeightBinder, plain_rows, settle)
+from .block import OutputNormBlock, ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock
 from .diff_attention import DifferentialAttention
 from .embedding import LMHead, TokenEmbedding
+from .forget_gate import ForgetGateAttention
 from .gla import GatedLinearAttention
 from .latent_attention import LatentAttention
 from .lightning import LightningAttention
 from .mlp import MLP, SwiGLU
 from .moe import RoutedExperts, Routing, SoftmaxTopKRouter, SparseMoE, TopKRouter
-from .norm import LayerNorm, OutputLayerNorm, OutputRMSNorm, RMSNorm
+from .norm import LayerNorm, OutputLayerNorm, OutputRMSNorm, ResidualRMSNorm, RMSNorm
 from .rotary import NoPosition, Rotary
 from .reentry import StreamReentry
 from .short_conv import ShortConv
+from .side_by_side import SideBySide
 from .sigmoid_attention import SigmoidAttention
 
 __all__ = ["Attention", "Block", "CacheNeed", "CacheView", "CallInfo", "FeedForward", "Mixer",
@@ -21,4 +24,6 @@ __all__ = ["Attention", "Block", "CacheNeed", "CacheView", "CallInfo", "FeedForw
            "SparseMoE", "RMSNorm", "NoPosition", "Rotary", "OutputNormBlock", "OutputRMSNorm",
            "LatentAttention", "LightningAttention", "ShortConv", "ParallelBlock",
            "DifferentialAttention", "MLP", "StreamReentry", "GatedLinearAttention",
-           "SigmoidAttention", "SandwichBlock", "LayerNorm", "OutputLayerNorm"]
+           "SigmoidAttention", "SandwichBlock", "LayerNorm", "OutputLayerNorm", "NormedSum",
+           "ReadyRows", "plain_rows", "PostNormBlock", "ForgetGateAttention", "ResidualRMSNorm",
+           "SideBySide"]

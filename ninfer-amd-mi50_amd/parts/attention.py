@@ -15,6 +15,14 @@ last taps - 1 projected rows of a request being per-request state); a softmax wi
 (`sink`: one more term exp(0) in the denominator, so that a row may attend to nothing); and
 a layer without key and value projections that reads the keys and values another layer's
 run has cached (`own_kv` False), with queries, window and everything else of its own.
+
+A further group of parameters runs on a path of its own (product, `qkv_wide`, attention,
+product): queries and keys normed over their whole projections (`qk_norm="projection"`),
+values that are the keys as projected (`values="keys"`), one more key and value per block of
+tokens before the window, the means of the block's (`pool`), a factor per head on the scores
+(`head_temp`), a position encoding that scales what it turns (its `magnitude`), and an output
+gate computed from the layer's input (`output_gate`). Such a layer reads its input through one
+product (`input_width`), which layers side by side may share.
 """
 from __future__ import annotations
 
@@ -35,7 +43,9 @@ class Attention(Mixer):
                  score_slopes: Optional[Sequence[float]] = None,
                  qk_norm_eps: Optional[float] = None, page_size: Optional[int] = None,
                  vdim: Optional[int] = None, conv_taps: int = 0, sink: bool = False,
-                 own_kv: bool = True, names=None, cache_window="same"):
+                 own_kv: bool = True, names=None, cache_window="same", qk_norm: str = "head",
+                 values: str = "own", pool: Optional[int] = None, head_temp: bool = False,
+                 output_gate: bool = False):
         """`score_slopes` [heads]: a distance-based position bias, slope * (key's position -
         query's position) added to head h's scaled scores before the softmax (None: none).
         It is a parameter of the attention kernels, beside or instead of the rotation that
@@ -50,7 +60,37 @@ class Attention(Mixer):
         follows the prefix in the tensors' names, a dict with any of the keys q, k, v, o,
         q_norm, k_norm, conv (the suffix of a projection's convolution). `cache_window`: the
         span of positions whose keys and values the cache keeps, when it differs from this
-        layer's own window (None: all; other layers with wider windows read this cache)."""
+        layer's own window (None: all; other layers with wider windows read this cache).
+        `qk_norm` 'projection': the norm of `qk_norm_eps` goes over all of a row's query numbers
+        (and over all its key numbers), gains [heads * head_dim] and [kv_heads * head_dim].
+        `values` 'keys': no value projection; a token's value is its key as projected, before
+        norm and rotation. `pool`: beside the keys within its window a row sees, for every block
+        of `pool` tokens that lies wholly before the window, the mean of the block's cached keys
+        and values, in the same softmax. `head_temp`: a factor per head on the scores (tensor
+        `names['temp']` [heads]). `output_gate`: the heads' outputs are multiplied by
+        sigmoid(W_g x), element by element (`names['g']` [heads * vdim, hidden])."""
+        if qk_norm not in ("head", "projection") or values not in ("own", "keys"):
+            raise ValueError(f"qk_norm {qk_norm!r} or values {values!r} is not known")
+        self.qk_norm, self.values, self.pool = qk_norm, values, pool
+        self.head_temp, self.output_gate = bool(head_temp), bool(output_gate)
+        self.wide = qk_norm == "projection" or values == "keys" or pool is not None or head_temp \
+            or output_gate or getattr(position, "magnitude", 1.0) != 1.0
+        if self.wide:
+            if qkv_bias or conv_taps or not own_kv:
+                raise ValueError("biases, a convolution or another layer's cache beside norms over "
+                                 "whole projections, values from keys, blocks, head factors, a scaled "
+                                 "rotation or an output gate are not built")
+            if qk_norm_eps is not None and qk_norm != "projection":
+                raise ValueError("a norm per head beside these is not built")
+            if values == "keys" and vdim not in (None, head_dim):
+                raise ValueError(f"values that are keys have {head_dim} numbers, not {vdim}")
+            if pool is not None and (pool < 1 or window is None):
+                raise ValueError("blocks of at least one token lie before a window")
+        if pool is not None and cache_window == "same":
+            # a block's keys stay cached until its mean is formed
+            cache_window = max(window, pool)
+        self.shares_input = False      # the input product's weights belong to whoever holds this layer
+        self.temp: Optional[torch.Tensor] = None
         self.cache_window = window if cache_window == "same" else cache_window
         self.vdim = head_dim if vdim is None else int(vdim)
         self.conv_taps, self.sink, self.own_kv = int(conv_taps), bool(sink), bool(own_kv)
@@ -58,7 +98,8 @@ class Attention(Mixer):
             raise ValueError(f"conv_taps ({conv_taps}) must be >= 0")
         self.names = dict({"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight",
                            "o": "o_proj.weight", "q_norm": "q_norm.weight",
-                           "k_norm": "k_norm.weight", "conv": ".conv"}, **(names or {}))
+                           "k_norm": "k_norm.weight", "conv": ".conv", "temp": "temp", "g": "g_proj.weight"},
+                          **(names or {}))
         # the fused product + rotation + cache write serves the plain layer; everything else
         # (values of their own size, a convolution, another layer's cache) goes the general way
         self.general = self.vdim != head_dim or self.conv_taps > 0 or not self.own_kv
@@ -93,13 +134,20 @@ class Attention(Mixer):
     @property
     def qkv_width(self) -> int:
         kv = self.kv_heads * (self.head_dim + self.vdim) if self.own_kv else 0
+        if self.values == "keys":
+            kv = self.kv_heads * self.head_dim
         return self.heads * self.head_dim + kv
+
+    def input_width(self) -> Optional[int]:
+        if not self.wide:
+            return None
+        return self.qkv_width + (self.heads * self.vdim if self.output_gate else 0)
 
     def cache_need(self) -> Optional[CacheNeed]:
         if not self.own_kv:
             return None
         return CacheNeed.keys_values(self.kv_heads, self.head_dim, self.cache_window,
-                                     self.page_size, vdim=self.vdim)
+                                     self.page_size, vdim=self.vdim, block=self.pool)
 
     def state_floats(self) -> int:
         """The last conv_taps - 1 projected rows of a request."""
@@ -114,7 +162,12 @@ class Attention(Mixer):
                  p + n["o"]: TensorSpec((self.hidden, self.heads * self.vdim))}
         if self.own_kv:
             specs[p + n["k"]] = TensorSpec((self.kv_heads * d, self.hidden))
-            specs[p + n["v"]] = TensorSpec((self.kv_heads * self.vdim, self.hidden))
+            if self.values == "own":
+                specs[p + n["v"]] = TensorSpec((self.kv_heads * self.vdim, self.hidden))
+        if self.head_temp:
+            specs[p + n["temp"]] = TensorSpec((self.heads,), "gain")
+        if self.output_gate:
+            specs[p + n["g"]] = TensorSpec((self.heads * self.vdim, self.hidden))
         if self.conv_taps:
             for key, width in (("q", self.heads * d), ("k", self.kv_heads * d),
                                ("v", self.kv_heads * self.vdim)):
@@ -125,9 +178,10 @@ class Attention(Mixer):
             specs[p + "k_proj.bias"] = TensorSpec((self.kv_heads * d,), "bias")
             specs[p + "v_proj.bias"] = TensorSpec((self.kv_heads * d,), "bias")
         if self.qk_norm_eps is not None:
-            specs[p + n["q_norm"]] = TensorSpec((d,), "gain")
+            nq, nk = (self.heads, self.kv_heads) if self.qk_norm == "projection" else (1, 1)
+            specs[p + n["q_norm"]] = TensorSpec((nq * d,), "gain")
             if self.own_kv:
-                specs[p + n["k_norm"]] = TensorSpec((d,), "gain")
+                specs[p + n["k_norm"]] = TensorSpec((nk * d,), "gain")
         return specs
 
     def unused_tensor_specs(self) -> Dict[str, TensorSpec]:
@@ -144,6 +198,14 @@ class Attention(Mixer):
         if self.qk_norm_eps is not None:
             self.q_norm = w.float32(p + n["q_norm"])
             self.k_norm = w.float32(p + n["k_norm"]) if self.own_kv else None
+        if self.wide:
+            if self.head_temp:
+                self.temp = w.float32(p + n["temp"])
+            if not self.shares_input:
+                self.w_qkv = torch.empty((self.input_width(), self.hidden), dtype=w.act_dtype, device=w.device)
+                self.bind_input(w, self.w_qkv)
+            self.w_o = w.matrix(p + n["o"])
+            return
         self.w_qkv = torch.empty((self.qkv_width, self.hidden), dtype=w.act_dtype, device=w.device)
         w.matrix_into(p + n["q"], self.w_qkv[:nq])
         if self.own_kv:
@@ -165,6 +227,40 @@ class Attention(Mixer):
             w.hold(p + "k_proj.bias", self.b_qkv[nq:nq + nk])
             w.hold(p + "v_proj.bias", self.b_qkv[nq + nk:])
         self.w_o = w.matrix(p + n["o"])
+
+    def bind_input(self, w: WeightBinder, rows: torch.Tensor) -> None:
+        """The input product's weights into `rows` [input_width, hidden]: q, k, v (where values
+        are projected), the gate's."""
+        p, d, n = self.prefix, self.head_dim, self.names
+        at = 0
+        for key, width in (("q", self.heads * d), ("k", self.kv_heads * d),
+                           ("v", self.kv_heads * self.vdim if self.values == "own" else 0),
+                           ("g", self.heads * self.vdim if self.output_gate else 0)):
+            if width:
+                w.matrix_into(p + n[key], rows[at:at + width])
+                at += width
+
+    def forward_projected(self, ctx: StepContext, u, call: CallInfo):
+        ops, cache, d = ctx.ops, call.cache, self.head_dim
+        if not call.writes_cache:
+            raise ValueError(f"{self.prefix}: this layer writes a cache of its own")
+        nq, nk = self.heads * d, self.kv_heads * d
+        q = ctx.empty((ctx.T, nq))
+        ops.qkv_wide(u, ctx, q, self.heads, self.kv_heads, d, self.vdim, cache["k"], cache["v"],
+                     cache.block_table, cache.page_size, v_col=nq if self.values == "keys" else nq + nk,
+                     q_norm=self.q_norm, k_norm=self.k_norm, norm_eps=self.qk_norm_eps or 0.0,
+                     inv_freq=self.position.table(), rot_dim=self.position.rot_dim,
+                     interleaved=self.position.pairing == "interleaved",
+                     magnitude=getattr(self.position, "magnitude", 1.0), head_scale=self.temp,
+                     blocks=cache.blocks)
+        attn = ctx.empty((ctx.T, self.heads * self.vdim))
+        ops.paged_attention(q, cache["k"], cache["v"], cache.block_table, ctx, self.heads,
+                            self.kv_heads, d, cache.page_size, self.window, self.scale, attn,
+                            slopes=self.slopes, vdim=self.vdim, sink=self.sink, blocks=cache.blocks,
+                            gate=u[:, self.qkv_width:] if self.output_gate else None)
+        out = ctx.empty((ctx.T, self.hidden))
+        ops.linear(attn, self.w_o, out)
+        return out
 
     def _forward_general(self, ctx: StepContext, x, call: CallInfo):
         """Product, then one kernel for convolution, head norms, rotation and the cache write,
@@ -191,6 +287,10 @@ class Attention(Mixer):
         return out
 
     def forward(self, ctx: StepContext, x, residual, call: CallInfo):
+        if self.wide:
+            u = ctx.empty((ctx.T, self.input_width()))
+            ctx.ops.linear(x, self.w_qkv, u)
+            return self.forward_projected(ctx, u, call)
         if self.general:
             return self._forward_general(ctx, x, call)
         ops = ctx.ops

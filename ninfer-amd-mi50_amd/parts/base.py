@@ -44,30 +44,56 @@ class CacheNeed:
     number of named pools, each with a per-token shape and dtype of its own,
     for all positions (window None) or only the last `window` of them, in pages
     of `page_size` tokens (None: the engine's). Mixers with the same window and
-    page size share page numbers and block tables; each has pools of its own."""
+    page size share page numbers and block tables; each has pools of its own.
+
+    `stride` > 1: an entry of the pools belongs to a whole block of `stride` tokens (block b to
+    positions b stride .. (b + 1) stride - 1; it exists once all of them are cached), and a page
+    holds `page_size` such entries. `blocks`: a second need of the same mixer, with names of
+    its own, kept in a group (page numbers, block tables) of its own: what it keeps per block of
+    tokens beside what it keeps per token."""
     pools: Tuple[PoolSpec, ...]
     window: Optional[int] = None
     page_size: Optional[int] = None
+    stride: int = 1
+    blocks: Optional["CacheNeed"] = None
+
+    def all_needs(self) -> Tuple["CacheNeed", ...]:
+        return (self,) if self.blocks is None else (self, self.blocks)
+
+    def bytes_per_token(self, bytes_per_element: int) -> int:
+        """Bytes of the pools per token (those of blocks: their share of one token, rounded
+        up); pools without a dtype of their own count `bytes_per_element` per number."""
+        own = {"float32": 4, "bfloat16": 2}
+        return sum(-(-sum(p.elements_per_token() * (own[p.dtype] if p.dtype else bytes_per_element)
+                          for p in n.pools) // n.stride) for n in self.all_needs())
 
     @staticmethod
     def keys_values(kv_heads: int, head_dim: int, window: Optional[int] = None,
-                    page_size: Optional[int] = None, vdim: Optional[int] = None) -> "CacheNeed":
+                    page_size: Optional[int] = None, vdim: Optional[int] = None,
+                    block: Optional[int] = None) -> "CacheNeed":
         """Keys and values of `kv_heads` heads of `head_dim` (values: `vdim`, when given):
-        pools 'k' [pages, kv_heads, page_size, head_dim] and 'v' [.., vdim]."""
-        return CacheNeed((PoolSpec("k", (kv_heads,), (head_dim,)),
-                          PoolSpec("v", (kv_heads,), (head_dim if vdim is None else vdim,))),
-                         window, page_size)
+        pools 'k' [pages, kv_heads, page_size, head_dim] and 'v' [.., vdim]; with `block` also
+        one key and value for every whole block of so many tokens, of all positions: pools
+        'k_block' and 'v_block' of the same shapes."""
+        def pair(suffix):
+            return (PoolSpec("k" + suffix, (kv_heads,), (head_dim,)),
+                    PoolSpec("v" + suffix, (kv_heads,), (head_dim if vdim is None else vdim,)))
+        blocks = CacheNeed(pair("_block"), None, page_size, stride=block) if block else None
+        return CacheNeed(pair(""), window, page_size, blocks=blocks)
 
 
 @dataclass
 class CacheView:
     """One cache instance as a step sees it: the mixer's pools by name (each
     [pages, *outer, page_size, *inner]) and the block table of the step's
-    requests [S, max_pages] (int32, -1 where a page was given back)."""
+    requests [S, max_pages] (int32, -1 where a page was given back). `blocks`: the same for
+    what the mixer keeps per block of `stride` tokens, when it keeps any."""
     pools: Dict[str, torch.Tensor]
     block_table: torch.Tensor
     page_size: int
     window: Optional[int]
+    stride: int = 1
+    blocks: Optional["CacheView"] = None
 
     def __getitem__(self, name: str) -> torch.Tensor:
         return self.pools[name]
@@ -139,13 +165,48 @@ class PendingRows:
             ctx.ops.moe_combine(residual, self.y, self.weights, self.shared, self.gate)
 
 
+@dataclass
+class NormedSum:
+    """Rows that a mixer leaves to be formed by whoever comes next:
+    factor * (rms(a) gain_a + rms(b) gain_b) with rms(y) = y rsqrt(mean(y^2) + eps), from rows
+    a, b [T, hidden] and gains [hidden] (32-bit)."""
+    a: torch.Tensor
+    gain_a: torch.Tensor
+    b: torch.Tensor
+    gain_b: torch.Tensor
+    eps: float
+    factor: float
+
+    def rows(self, ctx: "StepContext") -> torch.Tensor:
+        """The rows themselves, for parts that take only plain ones."""
+        total = torch.zeros(self.a.shape, dtype=torch.float32, device=self.a.device)
+        ctx.ops.norm_add(total, self.a, self.gain_a * self.factor, self.eps)
+        ctx.ops.norm_add(total, self.b, self.gain_b * self.factor, self.eps)
+        return total.to(ctx.act_dtype)
+
+
+@dataclass
+class ReadyRows:
+    """Nothing is left to be added to the residual; `rows` is the residual in the activation
+    dtype, for a block that reads it as it is."""
+    rows: torch.Tensor
+
+
+def plain_rows(ctx: "StepContext", y):
+    """What a part handed on as something that any part takes: a NormedSum becomes rows, a
+    ReadyRows nothing; everything else is handed back unchanged."""
+    if isinstance(y, NormedSum):
+        return y.rows(ctx)
+    return None if isinstance(y, ReadyRows) else y
+
+
 def settle(ctx: "StepContext", residual: torch.Tensor, pending) -> Optional[torch.Tensor]:
     """For parts that take only plain rows: a PendingRows is added into the
     residual now; a tensor (or None) is handed back unchanged."""
     if isinstance(pending, PendingRows):
         pending.add_to(ctx, residual)
         return None
-    return pending
+    return plain_rows(ctx, pending)
 
 
 class WeightBinder:
@@ -278,6 +339,15 @@ class Mixer(Part):
 
     def state_floats(self) -> int:
         return 0
+
+    def input_width(self) -> Optional[int]:
+        """Columns of the one product through which this mixer reads its input, or None when it
+        reads it in another way. A mixer that gives a width also has `bind_input(w, rows)`
+        (place the product's weights into `rows` [input_width, hidden]) and
+        `forward_projected(ctx, u, call)` (`u`: the product's [T, input_width], columns of a
+        wider row-major tensor), so that mixers which read the same input share one product;
+        its own `bind` then leaves these weights alone once `shares_input` is set."""
+        return None
 
     def forward(self, ctx: StepContext, x: torch.Tensor, residual: torch.Tensor,
                 call: CallInfo) -> Optional[torch.Tensor]:

@@ -14,8 +14,8 @@ from ..registry import register_part
 import torch
 
 from ..weights.source import TensorSpec
-from .base import (Block, CallInfo, FeedForward, Mixer, Norm, Part, PendingRows, StepContext,
-                   WeightBinder, settle)
+from .base import (Block, CallInfo, FeedForward, Mixer, Norm, Part, PendingRows, ReadyRows,
+                   StepContext, WeightBinder, plain_rows, settle)
 
 
 class PreNormBlock(Block):
@@ -132,6 +132,48 @@ class SandwichBlock(Block):
 register_part("block", "sandwich", SandwichBlock)
 
 
+class PostNormBlock(Block):
+    """A block whose norms sit behind the sums: x <- norm1(alpha x + mixer(x)), then
+    x <- norm2(alpha x + feed_forward(x)). The sublayers read the residual itself; the norms
+    (`residual_rmsnorm`, alpha is theirs) write it in 32-bit and hand it on in the activation
+    dtype, to the next sublayer and to the next block. `feed_forward` may be None (a norm given
+    all the same is one whose tensors the checkpoint may carry)."""
+
+    def __init__(self, mixer: Mixer, mixer_norm: Part, feed_forward: Optional[FeedForward] = None,
+                 ff_norm: Optional[Part] = None):
+        if feed_forward is not None and ff_norm is None:
+            raise ValueError("a feed-forward needs the norm behind it")
+        self.mixer, self.mixer_norm = mixer, mixer_norm
+        self.feed_forward = feed_forward
+        self.ff_norm = ff_norm if feed_forward is not None else None
+        self.spare_norm = ff_norm if feed_forward is None else None
+
+    def unused_tensor_specs(self):
+        return self.spare_norm.all_tensor_specs() if self.spare_norm is not None else {}
+
+    def children(self) -> List[Part]:
+        return [p for p in (self.mixer, self.mixer_norm, self.feed_forward, self.ff_norm) if p is not None]
+
+    def forward(self, ctx: StepContext, residual, pending, call: CallInfo):
+        if isinstance(pending, ReadyRows):
+            h = pending.rows
+        else:
+            settled = settle(ctx, residual, pending)
+            if settled is not None:
+                residual.add_(settled)
+            h = residual if residual.dtype == ctx.act_dtype else residual.to(ctx.act_dtype)
+        h = self.mixer_norm.apply(ctx, residual, self.mixer.forward(ctx, h, residual, call))
+        if self.feed_forward is not None:
+            y = self.feed_forward.forward(ctx, h, residual)
+            if y is None:
+                raise ValueError("a feed-forward in front of a norm hands its rows back")
+            h = self.ff_norm.apply(ctx, residual, y)
+        return ReadyRows(h)
+
+
+register_part("block", "post_norm", PostNormBlock)
+
+
 class ParallelBlock(Block):
     """A block whose sublayers run side by side on the same residual: h = norm(x), then
     x += mult (c1 mixer(h) + c2 feed_forward(h2)), where h2 = h, or ff_norm(x) when the block
@@ -213,7 +255,7 @@ class ParallelBlock(Block):
         h2 = h
         if self.ff_norm is not None:
             h2 = self.ff_norm.forward(ctx, residual, None)
-        a = self.mixer.forward(ctx, h, residual, call)
+        a = plain_rows(ctx, self.mixer.forward(ctx, h, residual, call))
         f = self.feed_forward.forward(ctx, h2, residual) if self.feed_forward is not None else None
         if self.mixer_gate is None and self.ff_gate is None and self.mult == 1.0:
             ctx.ops.scaled_sum_add(residual, a, self.mixer_scale, f, self.ff_scale)

@@ -13,7 +13,7 @@ import torch
 
 from ..registry import register_part
 from ..weights.source import TensorSpec
-from .base import Norm, Part, PendingRows, StepContext, WeightBinder
+from .base import Norm, Part, PendingRows, StepContext, WeightBinder, plain_rows
 
 
 class RMSNorm(Norm):
@@ -40,6 +40,7 @@ class RMSNorm(Norm):
 
     def forward(self, ctx: StepContext, residual, pending):
         out = ctx.empty((residual.shape[0], self.size))
+        pending = plain_rows(ctx, pending)
         if isinstance(pending, PendingRows):
             ctx.ops.rmsnorm(residual, self.gain, self.eps, out, rows_sum=pending, center=self.center)
         else:
@@ -48,6 +49,7 @@ class RMSNorm(Norm):
 
     def forward_rows(self, ctx: StepContext, residual, rows, pending=None):
         out = ctx.empty((rows.shape[0], self.size))
+        pending = plain_rows(ctx, pending)
         if isinstance(pending, PendingRows):
             ctx.ops.rmsnorm(residual, self.gain, self.eps, out, rows_sum=pending, rows=rows,
                             center=self.center)
@@ -80,6 +82,7 @@ class OutputRMSNorm(Part):
         self.gain = w.float32(self.tensor).reshape(-1)
 
     def add(self, ctx: StepContext, residual: torch.Tensor, y) -> None:
+        y = plain_rows(ctx, y)
         if isinstance(y, PendingRows):
             if y.shared is not None or y.ids is not None:
                 raise ValueError("a norm on a sparse feed-forward's output takes weighted rows only")
@@ -87,6 +90,33 @@ class OutputRMSNorm(Part):
                              weights=y.weights)
         else:
             ctx.ops.norm_add(residual, y, self.gain, self.eps, center=self.center)
+
+
+class ResidualRMSNorm(Part):
+    """The norm of a block that norms the residual stream itself, behind the sum:
+    residual <- z rsqrt(mean(z^2) + eps) gain with z = alpha residual + y, in 32-bit, y what a
+    sublayer gives back (rows, a sparse feed-forward's PendingRows, a NormedSum). `apply` hands
+    back the new residual in the activation dtype, for the sublayer that reads it next."""
+
+    def __init__(self, tensor: str, size: int, eps: float, alpha: float = 1.0):
+        self.tensor, self.size, self.eps, self.alpha = tensor, size, eps, float(alpha)
+        self.gain: Optional[torch.Tensor] = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return {self.tensor: TensorSpec((self.size,), "gain")}
+
+    def bind(self, w: WeightBinder) -> None:
+        self.gain = w.float32(self.tensor)
+
+    def apply(self, ctx: StepContext, residual: torch.Tensor, y) -> torch.Tensor:
+        out = None if ctx.act_dtype == residual.dtype else ctx.empty(residual.shape)
+        weights = None
+        if isinstance(y, PendingRows):
+            if y.shared is not None or y.ids is not None:
+                raise ValueError("a norm behind the sum takes a sparse feed-forward's weighted rows only")
+            y, weights = y.y, y.weights
+        ctx.ops.post_norm(residual, y, self.gain, self.eps, self.alpha, out=out, weights=weights)
+        return residual if out is None else out
 
 
 class LayerNorm(RMSNorm):
@@ -106,5 +136,6 @@ class OutputLayerNorm(OutputRMSNorm):
 
 register_part("norm", "rmsnorm", RMSNorm)
 register_part("norm", "output_rmsnorm", OutputRMSNorm)
+register_part("norm", "residual_rmsnorm", ResidualRMSNorm)
 register_part("norm", "layernorm", LayerNorm)
 register_part("norm", "output_layernorm", OutputLayerNorm)

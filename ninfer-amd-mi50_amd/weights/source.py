@@ -22,7 +22,8 @@ class TensorSpec:
     """What a part expects of one checkpoint tensor.
 
     role: 'matrix' (kept in the compute dtype), 'gain' (norm weight, read in
-    32-bit, random values 1 + N(0, s)), 'bias' (read in 32-bit). A dimension of -1 is one
+    32-bit, random values 1 + N(0, s)), 'bias' (read in 32-bit), 'unit' (numbers between 0
+    and 1, read in 32-bit, random values 0.5 + N(0, min(s, 0.08)), cut at 6 deviations). A dimension of -1 is one
     that the checkpoint decides (any size fits; random tensors cannot be made for it).
     """
     shape: Tuple[int, ...]
@@ -76,7 +77,7 @@ class RandomSource:
     Every element is a pure function of (seed, tensor name, flat index): a
     counter hash turned into an approximately normal number (the sum of twelve
     uniform ones, see counter_random.py). Matrices and biases: std * z; gains:
-    1 + std * z. A tensor's values do not depend on which other tensors exist,
+    1 + std * z; numbers between 0 and 1: 0.5 + min(std, 0.08) * z (|z| <= 6). A tensor's values do not depend on which other tensors exist,
     on the order they are asked for, or on where they are made: on 'cpu' the
     host computes them, on a GPU device the library's fill kernel does, and
     both give the same bits. That is how models too large to write to disk are
@@ -104,14 +105,15 @@ class RandomSource:
             raise WeightError(f"{name}: a size that only a checkpoint decides (shape "
                               f"{list(spec.shape)}); random weights need it in the configuration")
         key = counter_random.tensor_key(self.seed, name)
-        mean = 1.0 if spec.role == "gain" else 0.0
+        mean = {"gain": 1.0, "unit": 0.5}.get(spec.role, 0.0)
+        std = min(self.std, 0.08) if spec.role == "unit" else self.std
         if torch.device(self.device).type == "cpu":
-            return counter_random.fill(spec.shape, key, self.std, mean).to(self.dtype)
+            return counter_random.fill(spec.shape, key, std, mean).to(self.dtype)
         if self._ops is None:
             from ..kernels import load_ops
             self._ops = load_ops()
         t = torch.empty(spec.shape, dtype=self.dtype, device=self.device)
-        self._ops.fill_random(t, key, self.std, mean)
+        self._ops.fill_random(t, key, std, mean)
         return t
 
     def close(self) -> None:
