@@ -42,6 +42,13 @@ query latent, or windowed attention with a convolution on q, k and v, normed hea
 and layers that read another layer's keys and values; a clamped gated feed-forward, dense or
 as routed experts) beside a Qwen2-MoE model of the same width, depth, heads, window and experts.
 
+    python bench.py --scenario designs --design rudazen [--sizes small,medium] [--only rudazen|dense]
+
+the same for Rudazen (norms behind the sums; windowed attention whose values are its keys, with
+a mean key and value per block of tokens before the window, or gated windowed attention and
+forget-gate linear attention side by side; a dense feed-forward) beside a dense Qwen2-style
+model of the same width, depth, heads, window and feed-forward size.
+
     python bench.py --scenario long [--model 57b-a14b] [--requests 8] [--prompt 32768] [--new 256]
 
 is another measurement with a JSON line of its own: the scheduler serves
@@ -104,7 +111,7 @@ def main() -> int:
     ap.add_argument("--scenario", default="decode", choices=["decode", "long", "designs"])
     ap.add_argument("--sizes", default="small,medium",
                     help="--scenario designs: which of the layer sizes to run (small, medium)")
-    ap.add_argument("--design", default="getodra", choices=["getodra", "sosepel", "fopinex", "tuzapel"],
+    ap.add_argument("--design", default="getodra", choices=["getodra", "sosepel", "fopinex", "tuzapel", "rudazen"],
                     help="--scenario designs: the design to run beside the closest model the engine had")
     ap.add_argument("--only", default="", help="--scenario designs: run this one of the two models only")
     ap.add_argument("--requests", type=int, default=8, help="--scenario long: concurrent requests")
@@ -668,6 +675,42 @@ def sparse_for_tuzapel_config(z: dict) -> dict:
                 sliding_window=z["window"], max_window_layers=0)
 
 
+RUDAZEN_SIZES = {
+    # width, layers (of every four the third has two mixers side by side), query and kv heads,
+    # sizes of a key and a value, window, tokens of a block, the recurrence's heads and sizes
+    "small": dict(width=1024, layers=8, heads=8, kv_heads=2, dim=128, vdim=128, window=1024, pool=16,
+                  gla_heads=8, gla_dim=64, gla_vdim=128, ff=2816, vocab=32000, positions=4096),
+    "medium": dict(width=2048, layers=8, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, pool=16,
+                   gla_heads=16, gla_dim=64, gla_vdim=128, ff=5632, vocab=32000, positions=4096),
+}
+
+
+def rudazen_config(z: dict) -> dict:
+    attention = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"],
+                 "scale": z["dim"] ** -0.5, "rot": {"base": 500000.0, "dims": z["dim"]}}
+    pooled = dict(attention, mask={"size": z["window"], "pool": z["pool"]})
+    left = dict(attention, mask={"size": z["window"]}, rot={
+        "base": 10000.0, "dims": z["dim"] // 2,
+        "scaling": {"factor": 8.0, "original": 2048, "fast": 32.0, "slow": 1.0}})
+    right = {"heads": z["gla_heads"], "dim": z["gla_dim"], "vdim": z["gla_vdim"]}
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    layers = [{"type": "parallel", "mixer": {"left": left, "right": right}, "mlp": mlp} if i % 4 == 2
+              else {"type": "attention", "mixer": pooled, "mlp": mlp} for i in range(z["layers"])]
+    return {"architecture": "Rudazen", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "postln_alpha": 2.0, "embedding": {"scale": z["width"] ** 0.5}, "layers": layers}
+
+
+def dense_for_rudazen_config(z: dict) -> dict:
+    """The closest model the engine had: Qwen2-style dense blocks (rotary attention with as many
+    query and kv heads of the same size behind the same window, a feed-forward of the same
+    size) of the same width and depth."""
+    return dict(CONFIG_C, num_hidden_layers=z["layers"], hidden_size=z["width"],
+                num_attention_heads=z["heads"], num_key_value_heads=z["kv_heads"], head_dim=z["dim"],
+                intermediate_size=z["ff"], mlp_only_layers=list(range(z["layers"])), decoder_sparse_step=1,
+                vocab_size=z["vocab"], hidden_act="silu", use_sliding_window=True,
+                sliding_window=z["window"], max_window_layers=0)
+
+
 def designs_scenario(args) -> int:
     import torch
     from ninfer_amd import Chunk, EngineOptions, random_model
@@ -676,20 +719,23 @@ def designs_scenario(args) -> int:
 
     gen = torch.Generator().manual_seed(11)
     fopinex = args.design == "fopinex"
+    rudazen = args.design == "rudazen"
     out = {"metric": "prefill and decode throughput, " + ("Sosepel beside a Qwen2-MoE model" if sosepel
                      else "Fopinex beside a Qwen2-MoE model" if fopinex
                      else "Tuzapel beside a Qwen2-MoE model" if tuzapel
+                     else "Rudazen beside a dense model" if rudazen
                      else "Getodra beside a dense model") + " of equal size",
            "unit": "tok/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
            "data": "synthetic", "sizes": {}}
     for size in args.sizes.split(","):
         z = (SOSEPEL_SIZES if sosepel else FOPINEX_SIZES if fopinex else TUZAPEL_SIZES if tuzapel
-             else DESIGN_SIZES)[size]
+             else RUDAZEN_SIZES if rudazen else DESIGN_SIZES)[size]
         ctx = z["positions"]
         row = {"shape": z}
         pairs = (("sosepel", sosepel_config(z)), ("sparse", sparse_config(z))) if sosepel else \
             (("fopinex", fopinex_config(z)), ("sparse", sparse_for_fopinex_config(z))) if fopinex else \
             (("tuzapel", tuzapel_config(z)), ("sparse", sparse_for_tuzapel_config(z))) if tuzapel else \
+            (("rudazen", rudazen_config(z)), ("dense", dense_for_rudazen_config(z))) if rudazen else \
             (("getodra", getodra_config(z)), ("dense", dense_config(z)))
         for name, raw in pairs:
             if args.only and name != args.only:

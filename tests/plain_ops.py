@@ -335,7 +335,8 @@ class PlainOps:
         self.moe_align(r.ids, experts, r.offsets, r.order, tiles=r, weightless=weightless)
 
     def paged_attention(self, qkv, k_pool, v_pool, block_table, ctx, n_q, n_kv, head_dim,
-                        page_size, window, scale, out, slopes=None, vdim=None, sink=False):
+                        page_size, window, scale, out, slopes=None, vdim=None, sink=False,
+                        blocks=None, gate=None):
         t = qkv.shape[0]
         vdim = head_dim if vdim is None else vdim
         q = _f(qkv[:, :n_q * head_dim]).view(t, n_q, head_dim)
@@ -349,6 +350,13 @@ class PlainOps:
             assert (pages >= 0).all(), "read of a page that is not held"
             k = _f(k_pool[pages, :, js % page_size, :])  # [n, n_kv, D]
             v = _f(v_pool[pages, :, js % page_size, :])
+            if blocks is not None:   # the means of the blocks that lie wholly before the window
+                n = max(0, (pos[r] - window + 1) // blocks.stride)
+                bs = torch.arange(n)
+                bp = blocks.block_table[seq[r], bs // blocks.page_size].long()
+                assert (bp >= 0).all(), "read of a block's page that is not held"
+                k = torch.cat([_f(blocks["k_block"][bp, :, bs % blocks.page_size, :]), k])
+                v = torch.cat([_f(blocks["v_block"][bp, :, bs % blocks.page_size, :]), v])
             for h in range(n_q):
                 g = h // group
                 s = (k[:, g, :] @ q[r, h]) * scale
@@ -357,7 +365,65 @@ class PlainOps:
                 top = torch.clamp(s.max(), min=0.0) if sink else s.max()
                 p = torch.exp(s - top)
                 p = p / (p.sum() + (torch.exp(-top) if sink else 0.0))
-                out[r, h * vdim:(h + 1) * vdim] = (p @ v[:, g, :]).to(out.dtype)
+                y = p @ v[:, g, :]
+                if gate is not None:
+                    y = y * torch.sigmoid(_f(gate[r, h * vdim:(h + 1) * vdim]))
+                out[r, h * vdim:(h + 1) * vdim] = y.to(out.dtype)
+
+    def qkv_wide(self, u, ctx, q_out, heads, kv_heads, dim, vdim, k_pool, v_pool, block_table,
+                 page_size, v_col=None, q_norm=None, k_norm=None, norm_eps=0.0, inv_freq=None,
+                 rot_dim=0, interleaved=False, magnitude=1.0, head_scale=None, blocks=None):
+        t, nq, nk = ctx.T, heads * dim, kv_heads * dim
+        v_col = nq + nk if v_col is None else v_col
+        x = _f(u)
+
+        def ready(y, gain, n):
+            if gain is not None:
+                y = y * torch.rsqrt((y * y).mean(-1, keepdim=True) + norm_eps) * gain
+            y = y.view(t, n, dim)
+            turned = self._turn(y, ctx.positions, inv_freq, rot_dim, interleaved)
+            if magnitude != 1.0:
+                turned = torch.cat([turned[..., :rot_dim] * magnitude, y[..., rot_dim:]], -1)
+            return turned
+        q = ready(x[:, :nq], q_norm, heads)
+        if head_scale is not None:
+            q = q * head_scale[None, :, None]
+        q_out.copy_(q.reshape(t, nq).to(q_out.dtype))
+        k = ready(x[:, nq:nq + nk], k_norm, kv_heads)
+        v = x[:, v_col:v_col + kv_heads * vdim].reshape(t, kv_heads, vdim)
+        pos = ctx.positions.long()
+        page = block_table[ctx.row_seq.long(), pos // page_size].long()
+        assert (page >= 0).all(), "write into a page that is not held"
+        k_pool[page, :, pos % page_size, :] = k.to(k_pool.dtype)
+        v_pool[page, :, pos % page_size, :] = v.to(v_pool.dtype)
+        if blocks is None:
+            return
+        size, start, first = blocks.stride, ctx.seq_row_start.tolist(), ctx.seq_pos0.tolist()
+        for s in range(ctx.S):
+            end = first[s] + start[s + 1] - start[s]
+            for b in range(first[s] // size, end // size):
+                js = torch.arange(b * size, (b + 1) * size)
+                pages = block_table[s, js // page_size].long()
+                assert (pages >= 0).all(), "read of a page that is not held"
+                to = int(blocks.block_table[s, b // blocks.page_size])
+                assert to >= 0, "write into a block's page that is not held"
+                for src, dst in ((k_pool, blocks["k_block"]), (v_pool, blocks["v_block"])):
+                    dst[to, :, b % blocks.page_size] = _f(src[pages, :, js % page_size, :]).mean(0).to(dst.dtype)
+
+    def post_norm(self, residual, y, gain, eps, alpha, out=None, weights=None):
+        if hasattr(y, "gain_b"):
+            def rms(v):
+                return v * torch.rsqrt((v * v).mean(-1, keepdim=True) + y.eps)
+            add = y.factor * (rms(_f(y.a)) * y.gain_a + rms(_f(y.b)) * y.gain_b)
+        else:
+            add = _f(y)
+            if weights is not None:
+                t, k = weights.shape
+                add = (add.view(t, k, -1) * weights[:, :, None]).sum(1)
+        z = alpha * residual + add
+        residual.copy_(z * torch.rsqrt((z * z).mean(-1, keepdim=True) + eps) * gain)
+        if out is not None:
+            out.copy_(residual.to(out.dtype))
 
     # ---- parallel sublayers, hashed pairs, differential attention ------------------------------
     def embed_pairs(self, ctx, table, out, scale=1.0, pair_table=None, buckets=0, mul_prev=0,
@@ -416,22 +482,32 @@ class PlainOps:
         g = group or n
         x = o.view(t, n // g, g)
         x = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * weight
-        z = _f(gate)
-        f = torch.sigmoid(z) * (z if gate_act == "silu" else 1.0)
+        f = 1.0
+        if gate is not None:
+            z = _f(gate)
+            f = torch.sigmoid(z) * (z if gate_act == "silu" else 1.0)
         out.copy_((x.reshape(t, n) * f).to(out.dtype))
 
     def gla_work_floats(self, qkv_dtype, ctx, heads, dim):
         return 0
 
     def gated_linear_attention(self, qkv, q_off, k_off, v_off, z, heads, dim, vdim, tau, q_scale,
-                               state, ctx, out, work=None):
+                               state, ctx, out, work=None, forget=None):
         starts, slots = ctx.seq_row_start.tolist(), ctx.seq_slots.tolist()
-        alpha = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(-1, heads, dim)
+        n = heads * dim
+        if forget is not None:
+            off, bias, lower = forget
+            alpha = (lower + (1 - lower) * torch.sigmoid(_f(qkv[:, off:off + n]) + bias)).view(-1, heads, dim)
+        else:
+            alpha = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(-1, heads, dim)
         for s, slot in enumerate(slots):
             st = state[slot, :heads * dim * vdim].view(heads, dim, vdim)
             for r in range(starts[s], starts[s + 1]):
                 q = _f(qkv[r, q_off:q_off + heads * dim]).view(heads, dim) * q_scale
-                k = _f(qkv[r, k_off:k_off + heads * dim]).view(heads, dim)
+                if forget is not None:
+                    q, k = torch.nn.functional.silu(q / q_scale) * q_scale, 1 - alpha[r]
+                else:
+                    k = _f(qkv[r, k_off:k_off + heads * dim]).view(heads, dim)
                 v = _f(qkv[r, v_off:v_off + heads * vdim]).view(heads, vdim)
                 st.copy_(alpha[r][:, :, None] * st + k[:, :, None] * v[:, None, :])
                 out[r] = torch.einsum("hd,hdv->hv", q, st).reshape(-1)
