@@ -60,22 +60,34 @@ extern "C" int ninfer_paged_attention(const AttnArgs* a, int force_generic, hipS
     p.T = a->T - n;
     return attention_prefill(p, stream);
   }
-  if (!force_generic && attention_prefill_takes(*a)) return attention_prefill(*a, stream);
-  // keys and values of sizes of their own, a sink, blocks, a gate: row tiles of any such shape on the matrix
-  // cores; single rows (which come first) with the heads of a kv head as a tile's rows
-  if (!force_generic && attention_tiles_takes(*a)) {
-    const int n = a->max_qlen == 1 ? a->S : a->single_rows;
-    if (n > 0 && attention_tiles_heads_takes(*a)) {
-      AttnArgs d = *a;
-      d.T = n;
-      d.S = n;
-      d.max_qlen = 1;
-      if (int rc = attention_tiles_heads(d, stream)) return rc;
-      if (n == a->S) return 0;
-      return attention_tiles(*a, n, stream);
-    }
-    return attention_tiles(*a, 0, stream);
+  // single rows (which come first) of layers with values of another size, a sink, blocks or a
+  // gate: the heads of a kv head as a tile's rows
+  const int n = a->max_qlen == 1 ? a->S : a->single_rows;
+  const bool tiles = !force_generic && attention_tiles_takes(*a);
+  const bool apart = tiles && n > 0 && attention_tiles_heads_takes(*a) &&
+                     (!attention_prefill_takes(*a) || a->kblk || a->gate);
+  if (apart) {
+    AttnArgs d = *a;
+    d.T = n;
+    d.S = n;
+    d.max_qlen = 1;
+    if (int rc = attention_tiles_heads(d, stream)) return rc;
+    if (n == a->S) return 0;
   }
+  if (!force_generic && attention_prefill_takes(*a)) {
+    if (!apart) return attention_prefill(*a, stream);
+    AttnArgs p = *a;
+    p.seq_row_start += n;
+    p.seq_qlen += n;
+    p.seq_pos0 += n;
+    p.block_table += (int64_t)n * a->bt_stride;
+    if (p.kblk) p.blk_table += (int64_t)n * a->blk_bt_stride;
+    p.S = a->S - n;
+    p.T = a->T - n;
+    return attention_prefill(p, stream);
+  }
+  // ... and prompt portions of any such shape on the matrix cores
+  if (tiles) return attention_tiles(*a, apart ? n : 0, stream);
   return attention_generic(*a, stream);
 }
 

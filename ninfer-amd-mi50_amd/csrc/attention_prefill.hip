@@ -29,6 +29,12 @@
 // a window has passed may be gone (block-table entry -1): their keys are never
 // visible, and the last key's row is loaded in their place.
 //
+// Where the cache keeps one more key and value per block of tokens before the window (BLOCKS),
+// the tiles of the blocks that the rows see come in front of the keys' tiles: in the kernel
+// they lie at "keys" before t_first, and a tile there takes its rows from the blocks' pools
+// and pages and its bounds from how many blocks a row sees. The output may be gated, element by
+// element, where it is written.
+//
 // The same kernel serves decoding for models whose kv heads are shared by three
 // or more query heads (HEADS): the 32 "rows" of a block are then the query
 // heads of one kv head for one decoded token, all at one position, and the block
@@ -62,7 +68,8 @@ __device__ __forceinline__ void tr_read2(unsigned addr, short4v& r0, short4v& r1
                : "v"(addr), "n"(OFF0), "n"(OFF1));
 }
 
-template <int D, int NQ, bool HEADS>   // HEADS: rows are the query heads of one token (decode)
+// HEADS: rows are the query heads of one token (decode)
+template <int D, int NQ, bool HEADS, bool BLOCKS>
 __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, int CHUNK,
                                                                    int paired) {
   constexpr int KH = 2;             // waves per group of 32 rows: each meets one half of a tile's keys
@@ -155,8 +162,11 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
     lo_first = a.window > 0 ? max(0, pos_first - a.window + 1) : 0;
   }
   const int* bt = a.block_table + (int64_t)seq * a.bt_stride;
-  const bf16* kpool = (const bf16*)a.kpool;
-  const bf16* vpool = (const bf16*)a.vpool;
+  // the blocks' tiles: n_bt of them, at "keys" t_start .. t_first - 1
+  const int t_first = (lo_first / PK) * PK;
+  const int* bt_b = BLOCKS ? a.blk_table + (int64_t)seq * a.blk_bt_stride : nullptr;
+  const int blocks_last = BLOCKS ? attention_blocks_seen(pos_last, a.window, a.block) : 0;
+  const int t_start = BLOCKS ? t_first - (blocks_last + PK - 1) / PK * PK : t_first;
   // the page size divides the tile of 64 keys: a power of two
   const int ps_shift = __builtin_ctz(a.page_size), ps_mask = a.page_size - 1, Hkv = a.Hkv;
 
@@ -177,6 +187,10 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   const int all_see_last = HEADS ? pos_first : pos_first + qg * 32;
   const int all_see_first =
       HEADS ? lo_first : (a.window > 0 ? max(0, pos_first + qg * 32 + 31 - a.window + 1) : 0);
+  // the same bounds in blocks
+  const int q_blocks = BLOCKS ? attention_blocks_seen(q_pos, a.window, a.block) : 0;
+  const int wave_blocks = BLOCKS ? attention_blocks_seen(wave_pos_last, a.window, a.block) : 0;
+  const int all_see_blocks = BLOCKS ? attention_blocks_seen(all_see_last, a.window, a.block) : 0;
   bf16x8 qf[KS];
   {
     const int ql = q_valid ? q_local : 0;
@@ -227,6 +241,9 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   const int pos_last_u = __builtin_amdgcn_readfirstlane(pos_last);
   const int64_t last_at =
       (int64_t)bt[pos_last >> ps_shift] * page_stride + (((int64_t)g << ps_shift) + (pos_last & ps_mask)) * D;
+  const int64_t last_at_b = !BLOCKS || blocks_last == 0 ? 0
+      : (int64_t)bt_b[(blocks_last - 1) >> ps_shift] * page_stride +
+            (((int64_t)g << ps_shift) + ((blocks_last - 1) & ps_mask)) * D;
   // Page numbers, fetched NST tiles ahead of the keys with scalar loads: the rows of one load
   // lie in one page (a page holds at least RPP rows: see attention_prefill_takes), so its
   // number is the same in every lane, and scalar loads do not count among the vector loads
@@ -241,11 +258,24 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   const unsigned bt_hi = (unsigned)__builtin_amdgcn_readfirstlane((int)(bt_bits >> 32));
   const unsigned bt_lo = (unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)bt_bits);
   const table_ptr bt_c = (table_ptr)(((uintptr_t)bt_hi << 32) | (uintptr_t)bt_lo);
+  const uintptr_t btb_bits = (uintptr_t)bt_b;
+  const unsigned btb_hi = (unsigned)__builtin_amdgcn_readfirstlane((int)(btb_bits >> 32));
+  const unsigned btb_lo = (unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)btb_bits);
+  const table_ptr btb_c = (table_ptr)(((uintptr_t)btb_hi << 32) | (uintptr_t)btb_lo);
+  const int blocks_last_u = __builtin_amdgcn_readfirstlane(blocks_last);
+  const int t_first_u = __builtin_amdgcn_readfirstlane(t_first), t_start_u = __builtin_amdgcn_readfirstlane(t_start);
   int kpage[NST][KPT];
   auto load_pages = [&](int slot, int t0) {
 #pragma unroll
     for (int i = 0; i < KPT; ++i) {
       const int kp = t0 + (i * NW + wave_u) * RPP;   // the load's first row
+      if constexpr (BLOCKS) {
+        const bool is_b = t0 < t_first_u;
+        const table_ptr table = is_b ? btb_c : bt_c;
+        const int at = is_b ? min(kp - t_start_u, blocks_last_u - 1) : min(kp, pos_last_u);
+        kpage[slot][i] = table[__builtin_amdgcn_readfirstlane(at >> ps_shift)];
+        continue;
+      }
       kpage[slot][i] = bt_c[__builtin_amdgcn_readfirstlane(min(kp, pos_last_u) >> ps_shift)];   // always a table entry of the request
     }
   };
@@ -253,11 +283,16 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   auto issue_tile = [&](int buf, int slot, int t0) {
     unsigned char* kb = stages + buf * STAGE_BYTES + wave_u * 1024;
     unsigned char* vb = kb + TILE_BYTES;
+    const bool is_b = BLOCKS && t0 < t_first_u;
+    const bf16* kpool = is_b ? (const bf16*)a.kblk : (const bf16*)a.kpool;
+    const bf16* vpool = is_b ? (const bf16*)a.vblk : (const bf16*)a.vpool;
+    const int shift = is_b ? t_start_u : 0, last = is_b ? blocks_last - 1 : pos_last;
+    const int64_t there = is_b ? last_at_b : last_at;
 #pragma unroll
     for (int i = 0; i < KPT; ++i) {
       const int page = kpage[slot][i];
-      const int kp = t0 + (i * NW + wave_u) * RPP + l_row;
-      const int64_t at = (page >= 0 && kp <= pos_last) ? page * page_stride + in_page[i] : last_at;
+      const int kp = t0 + (i * NW + wave_u) * RPP + l_row - shift;
+      const int64_t at = (page >= 0 && kp <= last) ? page * page_stride + in_page[i] : there;
       // decoding reads every key once a step (marked non-temporal: the last argument); a
       // prompt's keys serve many blocks of rows from L2
       __builtin_amdgcn_global_load_lds((gptr)(kpool + at + k_chunk[i]), (lptr)(kb + i * (NW * 1024)), 16, 0,
@@ -279,9 +314,14 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   }
   // the products of this wave's part of the tile at keys t0.. in LDS buffer buf
   auto multiply = [&](int buf, int t0) {
-    const int k0 = t0 + 32 * NKB * kh;
+    const bool is_b = BLOCKS && t0 < t_first_u;
+    const int k0 = t0 + 32 * NKB * kh - (is_b ? t_start_u : 0);
+    // what the rows see of this tile, in keys or in blocks
+    const int wave_pos_last_ = is_b ? wave_blocks - 1 : wave_pos_last, wave_lo_ = is_b ? 0 : wave_lo;
+    const int see_last = is_b ? all_see_blocks - 1 : all_see_last, see_first = is_b ? 0 : all_see_first;
+    const int up_to = is_b ? q_blocks - 1 : q_pos, from = is_b ? 0 : q_lo;
     // not for tiles beyond the last key, or out of sight of every row of the wave
-    if (!wave_live || k0 > wave_pos_last || k0 + 32 * NKB <= wave_lo) return;
+    if (!wave_live || k0 > wave_pos_last_ || k0 + 32 * NKB <= wave_lo_) return;
     const unsigned char* k_s = stages + buf * STAGE_BYTES;
     // Left alone, the compiler reads each fragment from LDS just before the matrix instruction
     // that needs it (it keeps registers few), and that instruction then waits a whole LDS
@@ -338,7 +378,7 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
         }
     }
     float mx = -1e30f;
-    if (k0 + 32 * NKB - 1 > all_see_last || k0 < all_see_first) {
+    if (k0 + 32 * NKB - 1 > see_last || k0 < see_first) {
 #pragma unroll
       for (int kb = 0; kb < NKB; ++kb)
 #pragma unroll
@@ -346,7 +386,7 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
           int kp = k0 + 32 * kb + 8 * (v >> 2) + 4 * j + (v & 3);
           // minus infinity, so that the probability is exactly 0 whatever the row's maximum
           // (the maximum itself starts at -1e30 and stays finite)
-          float val = (kp <= q_pos && kp >= q_lo) ? s[kb][v] : -__builtin_inff();
+          float val = (kp <= up_to && kp >= from) ? s[kb][v] : -__builtin_inff();
           s[kb][v] = val;
           mx = fmaxf(mx, val);
         }
@@ -413,19 +453,18 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   // LDS (and nothing else that the vector memory counter counts); when tile i is needed, the
   // loads issued after its own are those of the NST - 2 tiles after it.
   constexpr int YOUNGER = (NST - 2) * 2 * KPT;
-  const int t_first = (lo_first / PK) * PK;
 #pragma unroll
-  for (int st = 0; st < NST; ++st) load_pages(st, t_first + st * PK);
+  for (int st = 0; st < NST; ++st) load_pages(st, t_start + st * PK);
 #pragma unroll
   for (int st = 0; st + 1 < NST; ++st) {
-    issue_tile(st, st, t_first + st * PK);
-    load_pages(st, t_first + (NST + st) * PK);
+    issue_tile(st, st, t_start + st * PK);
+    load_pages(st, t_start + (NST + st) * PK);
   }
   // NST tiles per turn, so that the stage and the page slot of each are constants. Nothing
   // in the loop stands under a condition: tiles beyond the last key are loaded (the last
   // key's row, over and over) and skipped by the products, so the wait counts exactly the
   // loads issued after the ones it needs.
-  for (int t0 = t_first; t0 <= pos_last; t0 += NST * PK) {
+  for (int t0 = t_start; t0 <= pos_last; t0 += NST * PK) {
 #pragma unroll
     for (int u = 0; u < NST; ++u) {
       // this wave's part of tile u has landed; after the barrier everybody's has, and the
@@ -490,6 +529,18 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
     // lane holds, of its query's output, dims 32 db + 8 (v / 4) + 4 j + v % 4
     const float inv = 1.f / l;
     bf16* orow = (bf16*)a.out + ((int64_t)(row0 + q_local) * a.Hq + h) * D;
+    if (a.gate) {
+      const bf16* grow = (const bf16*)a.gate + (int64_t)(row0 + q_local) * a.gate_stride + h * D;
+#pragma unroll
+      for (int db = 0; db < DB; ++db)
+#pragma unroll
+        for (int qd = 0; qd < 4; ++qd) {
+          const bf16x4 z = *(const bf16x4*)(grow + db * 32 + 8 * qd + 4 * j);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            o[db][4 * qd + e] /= 1.f + __builtin_amdgcn_exp2f(-1.44269504088896f * (float)z[e]);
+        }
+    }
 #pragma unroll
     for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -517,9 +568,9 @@ static bool prefill_page_ok(const AttnArgs& a) {
   return PK % a.page_size == 0 && a.page_size * 2 * a.D >= 1024;
 }
 
-template <int D, int NQ, bool HEADS>
+template <int D, int NQ, bool HEADS, bool BLOCKS = false>
 static int launch_attn(const AttnArgs& a, dim3 grid, int chunk, int paired, hipStream_t stream) {
-  auto kern = attn_prefill_kernel<D, NQ, HEADS>;
+  auto kern = attn_prefill_kernel<D, NQ, HEADS, BLOCKS>;
   const size_t lds = prefill_lds(D, NQ);
   if (lds > 48 * 1024) {
     hipError_t e = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -551,7 +602,9 @@ int attention_decode_heads(const AttnArgs& a, int chunk, int n_chunks, hipStream
 
 bool attention_prefill_takes(const AttnArgs& a) {
   return a.dtype == kBF16 && (a.D == 64 || a.D == 128) && a.q_stride % 8 == 0 &&
-         prefill_page_ok(a) && a.seq_row_start != nullptr && (a.Dv == 0 || a.Dv == a.D) && !a.sink && !a.kblk && !a.gate;
+         prefill_page_ok(a) && a.seq_row_start != nullptr && (a.Dv == 0 || a.Dv == a.D) && !a.sink &&
+         (!a.kblk || (a.blk_page_size == a.page_size && !a.slopes)) &&
+         (!a.gate || (a.gate_stride % 4 == 0 && (uintptr_t)a.gate % 8 == 0));
 }
 
 // Row tiles of PQ rows that the launch enumerates (one more per request than whole tiles:
@@ -562,6 +615,10 @@ template <int NQ>
 static int launch_prefill(const AttnArgs& a, int paired, hipStream_t stream) {
   constexpr int PQ = NQ * 32;
   dim3 grid(prefill_tiles(a, PQ), a.Hq);
+  if (a.kblk) {
+    if (a.D == 128) return launch_attn<128, NQ, false, true>(a, grid, 0, paired, stream);
+    return launch_attn<64, NQ, false, true>(a, grid, 0, paired, stream);
+  }
   if (a.D == 128) return launch_attn<128, NQ, false>(a, grid, 0, paired, stream);
   return launch_attn<64, NQ, false>(a, grid, 0, paired, stream);
 }

@@ -488,9 +488,13 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
 }
 
 // The records of a row and head put together: out = sum_c o_c 2^(m_c - m) / sum_c l_c 2^(m_c - m).
-// Lane c weighs chunk c (64 chunks at a time); the outputs' loads do not wait for each other.
-__global__ __launch_bounds__(64) void attention_tiles_merge_kernel(AttnArgs a, int n_chunks) {
-  const int th = blockIdx.x, lane = threadIdx.x;
+// Four waves share the records: every wave weighs them all (lane c chunk c, 64 at a time) and
+// adds up the outputs of every fourth, whose loads do not wait for each other; the waves meet
+// in LDS.
+constexpr int kMergeWaves = 4;
+__global__ __launch_bounds__(64 * kMergeWaves) void attention_tiles_merge_kernel(AttnArgs a, int n_chunks) {
+  __shared__ float acc_s[kMergeWaves][128];
+  const int th = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int vdim = a.Dv, stride = 2 + vdim;
   const float* rec = a.workspace + (int64_t)th * n_chunks * stride;
   float mm = -1e30f;
@@ -506,7 +510,7 @@ __global__ __launch_bounds__(64) void attention_tiles_merge_kernel(AttnArgs a, i
     }
     const int cnt = min(64, n_chunks - c0);
 #pragma unroll 4
-    for (int j = 0; j < cnt; ++j) {
+    for (int j = wave; j < cnt; j += kMergeWaves) {
       const float fj = __shfl(f, j, 64);
       const float* r = rec + (c0 + j) * stride + 2;
 #pragma unroll
@@ -516,18 +520,19 @@ __global__ __launch_bounds__(64) void attention_tiles_merge_kernel(AttnArgs a, i
       }
     }
   }
+  acc_s[wave][lane] = acc[0];
+  acc_s[wave][64 + lane] = acc[1];
   const float inv = 1.f / wave_sum(l);
-  __bf16* orow = (__bf16*)a.out + (int64_t)th * vdim;
-  const int t = th / a.Hq, h = th - t * a.Hq;
+  __syncthreads();
+  const int d = threadIdx.x;
+  if (d >= vdim) return;
+  float x = 0.f;
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int d = lane + 64 * i;
-    if (d < vdim) {
-      float x = acc[i] * inv;
-      if (a.gate) x *= at_sigmoid(to_f32(((const bf16*)a.gate)[(int64_t)t * a.gate_stride + h * vdim + d]));
-      orow[d] = (__bf16)x;
-    }
-  }
+  for (int w = 0; w < kMergeWaves; ++w) x += acc_s[w][d];
+  x *= inv;
+  const int t = th / a.Hq, h = th - t * a.Hq;
+  if (a.gate) x *= at_sigmoid(to_f32(((const bf16*)a.gate)[(int64_t)t * a.gate_stride + h * vdim + d]));
+  ((__bf16*)a.out)[(int64_t)th * vdim + d] = (__bf16)x;
 }
 
 // Chunks of the visible keys (whole tiles) so that the launch has about four blocks a CU, at
@@ -601,7 +606,7 @@ static int launch_heads(const AttnArgs& a, hipStream_t stream) {
   kern<<<dim3(a.T, a.Hkv, n), 128, lds, stream>>>(a, per, n);
   NINFER_LAUNCH_CHECK();
   if (n > 1) {
-    attention_tiles_merge_kernel<<<a.T * a.Hq, 64, 0, stream>>>(a, n);
+    attention_tiles_merge_kernel<<<a.T * a.Hq, 64 * kMergeWaves, 0, stream>>>(a, n);
     NINFER_LAUNCH_CHECK();
   }
   return 0;

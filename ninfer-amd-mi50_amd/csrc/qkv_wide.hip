@@ -248,6 +248,141 @@ __global__ __launch_bounds__(kWideThreads) void qkv_wide_kernel(QkvWideArgs a) {
   }
 }
 
+// The same for bfloat16 rows of whole pieces, ROWS rows to a block of as many threads as a row
+// has pieces of queries and keys: a thread keeps its piece's gains and its piece of every row
+// in registers, so that gains are fetched once for ROWS rows and the rows' loads are under way
+// together; only pieces whose partners lie in another thread's (half-split pairs) go through
+// LDS. One barrier.
+constexpr int kWideRowsMaxThreads = 1024;
+template <int ROWS>
+__global__ __launch_bounds__(kWideRowsMaxThreads) void qkv_wide_rows_kernel(QkvWideArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  __shared__ float red[ROWS][kWideRowsMaxThreads / 64][2];
+  const int nq = a.Hq * a.dim, nk = a.Hkv * a.dim, nv = a.Hkv * a.vdim;
+  const int tid = threadIdx.x, nt = blockDim.x, wave = tid >> 6;
+  const int half = a.rot_dim / 2, t0 = blockIdx.x * ROWS;
+  float* trig = smem;                          // [ROWS][rot_dim]: cos, then sin
+  float* x_s = smem + ROWS * a.rot_dim;        // [ROWS][nq + nk], for half-split pairs
+  const int i = 8 * tid;
+  const bool live = i < nq + nk, is_q = i < nq;
+  const int j0 = is_q ? i : i - nq;
+  const int hd = j0 / a.dim, d0 = j0 - hd * a.dim;
+  const bool split = !a.interleaved && d0 < a.rot_dim;   // the partners are another piece
+  const float* gain = is_q ? a.q_gain : a.k_gain;
+  wide_u32x4 raw[ROWS];
+  int pos[ROWS], seq[ROWS];
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    const int t = min(t0 + r, a.T - 1);
+    pos[r] = a.positions[t];
+    seq[r] = a.row_seq[t];
+    const unsigned short* u = (const unsigned short*)a.u + (int64_t)t * a.stride;
+    raw[r] = live ? *(const wide_u32x4*)(u + (is_q ? a.q_col : a.k_col) + j0) : wide_u32x4{0u, 0u, 0u, 0u};
+  }
+  float g[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) g[e] = 1.f;
+  if (gain && live) {
+    const float4 g0 = *(const float4*)(gain + j0), g1 = *(const float4*)(gain + j0 + 4);
+    g[0] = g0.x; g[1] = g0.y; g[2] = g0.z; g[3] = g0.w; g[4] = g1.x; g[5] = g1.y; g[6] = g1.z; g[7] = g1.w;
+  }
+  for (int idx = tid; idx < ROWS * half; idx += nt) {
+    const int r = idx / half, p = idx - r * half;
+    float sn, cs;
+    sincosf((float)a.positions[min(t0 + r, a.T - 1)] * a.inv_freq[p], &sn, &cs);
+    trig[r * a.rot_dim + p] = cs * a.magnitude;
+    trig[r * a.rot_dim + half + p] = sn * a.magnitude;
+  }
+  const bool has_q = wave * 512 < nq, has_k = wave * 512 + 511 >= nq;
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    float f[8], ss = 0.f;
+    wide_load<bf16, 8>((const bf16*)&raw[r], f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = fmaf(f[e], f[e], ss);
+    if (live && split) {
+      float* dst = x_s + r * (nq + nk) + i;
+      *(float4*)dst = make_float4(f[0] * g[0], f[1] * g[1], f[2] * g[2], f[3] * g[3]);
+      *(float4*)(dst + 4) = make_float4(f[4] * g[4], f[5] * g[5], f[6] * g[6], f[7] * g[7]);
+    }
+    const float sq = has_q ? wave_sum(is_q ? ss : 0.f) : 0.f;
+    const float sk = has_k ? wave_sum(is_q ? 0.f : ss) : 0.f;
+    if ((tid & 63) == 0) red[r][wave][0] = sq, red[r][wave][1] = sk;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    const int t = t0 + r;
+    if (t >= a.T) break;
+    float sum = 0.f;
+    for (int w = 0; w < nt / 64; ++w) sum += red[r][w][is_q ? 0 : 1];
+    const float inv = gain ? 1.f / sqrtf(sum / (float)(is_q ? nq : nk) + a.eps) : 1.f;
+    const int* bt = a.block_table + (int64_t)seq[r] * a.bt_stride;
+    const int64_t page = bt[pos[r] / a.page_size];
+    const int slot = pos[r] % a.page_size;
+    const bool means = ROWS == 1 && a.block > 0 && a.all_single && (pos[r] + 1) % a.block == 0;
+    const int b = means ? pos[r] / a.block : 0;
+    const float* tr = trig + r * a.rot_dim;
+    if (live) {
+      float x[8];
+      wide_load<bf16, 8>((const bf16*)&raw[r], x);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] *= inv * g[e];
+      if (split) {
+        const bool first = d0 < half;
+        const float* other = x_s + r * (nq + nk) + i + (first ? half : -half);
+        const int p0 = first ? d0 : d0 - half;
+        const float4 y0 = *(const float4*)other, y1 = *(const float4*)(other + 4);
+        const float y[8] = {y0.x, y0.y, y0.z, y0.w, y1.x, y1.y, y1.z, y1.w};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float cs = tr[p0 + e], sn = tr[half + p0 + e], z = y[e] * inv * sn;
+          x[e] = first ? x[e] * cs - z : x[e] * cs + z;
+        }
+      } else if (d0 < a.rot_dim) {
+#pragma unroll
+        for (int e = 0; e < 8; e += 2) {
+          if (d0 + e < a.rot_dim) {
+            const int p = (d0 + e) >> 1;
+            const float cs = tr[p], sn = tr[half + p], x0 = x[e], x1 = x[e + 1];
+            x[e] = x0 * cs - x1 * sn;
+            x[e + 1] = x1 * cs + x0 * sn;
+          }
+        }
+      }
+      if (is_q) {
+        if (a.head_scale) {
+          const float hs = a.head_scale[hd];
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] *= hs;
+        }
+        wide_store<bf16, 8>((bf16*)a.q_out + (int64_t)t * nq + i, x);
+      } else {
+        const int64_t at = ((page * a.Hkv + hd) * a.page_size + slot) * a.dim + d0;
+        wide_store<bf16, 8>((bf16*)a.kpool + at, x);
+        if (means) {
+          float own[8], m[8];
+#pragma unroll
+          for (int e = 0; e < 8; ++e) own[e] = to_f32(from_f32<bf16>(x[e]));   // as the page holds it
+          wide_block_mean<bf16, 8>(a, bt, false, j0, b * a.block, own, m);
+          wide_store_mean<bf16, 8>(a, seq[r], false, j0, b, m);
+        }
+      }
+    }
+    for (int v = 8 * tid; v < nv; v += 8 * nt) {
+      const wide_u32x4 val = *(const wide_u32x4*)((const unsigned short*)a.u + (int64_t)t * a.stride + a.v_col + v);
+      const int gv = v / a.vdim, dv = v - gv * a.vdim;
+      *(wide_u32x4*)((unsigned short*)a.vpool + ((page * a.Hkv + gv) * a.page_size + slot) * a.vdim + dv) = val;
+      if (means) {
+        float own[8], m[8];
+        wide_load<bf16, 8>((const bf16*)&val, own);
+        wide_block_mean<bf16, 8>(a, bt, true, v, b * a.block, own, m);
+        wide_store_mean<bf16, 8>(a, seq[r], true, v, b, m);
+      }
+    }
+  }
+}
+
 // The means of all blocks that the step's rows complete: a block of threads per token block,
 // counted request after request.
 template <typename T, int VEC>
@@ -286,6 +421,29 @@ static int wide_lds(K kern, size_t lds, bool* raised) {
 }
 
 template <typename T, int VEC>
+static int launch_means(const QkvWideArgs& a, hipStream_t stream) {
+  if (a.block > 0 && !a.all_single) {
+    // no step completes more: every request adds at most one block begun before
+    const int most = a.T / a.block + a.S;
+    block_means_kernel<T, VEC><<<most, kWideThreads, 0, stream>>>(a);
+    NINFER_LAUNCH_CHECK();
+  }
+  return 0;
+}
+
+// Rows of bfloat16 whole pieces: several rows to a block where there are many.
+template <int ROWS>
+static int launch_wide_rows(const QkvWideArgs& a, hipStream_t stream) {
+  const int n = (a.Hq + a.Hkv) * a.dim;
+  const size_t lds = (size_t)ROWS * (a.rot_dim + (a.interleaved ? 0 : n)) * sizeof(float);
+  static bool raised = false;
+  if (int rc = wide_lds(qkv_wide_rows_kernel<ROWS>, lds, &raised)) return rc;
+  qkv_wide_rows_kernel<ROWS><<<(a.T + ROWS - 1) / ROWS, (n / 8 + 63) / 64 * 64, lds, stream>>>(a);
+  NINFER_LAUNCH_CHECK();
+  return launch_means<bf16, 8>(a, stream);
+}
+
+template <typename T, int VEC>
 static int launch_wide(const QkvWideArgs& a, hipStream_t stream) {
   const size_t lds = (size_t)((a.Hq + a.Hkv) * a.dim + a.rot_dim) * sizeof(float);
   NINFER_REQUIRE(lds <= (size_t)kWideMaxLds, "qkv_wide: rows of %d queries' and keys' numbers exceed LDS",
@@ -294,13 +452,7 @@ static int launch_wide(const QkvWideArgs& a, hipStream_t stream) {
   if (int rc = wide_lds(qkv_wide_kernel<T, VEC>, lds, &raised)) return rc;
   qkv_wide_kernel<T, VEC><<<a.T, kWideThreads, lds, stream>>>(a);
   NINFER_LAUNCH_CHECK();
-  if (a.block > 0 && !a.all_single) {
-    // no step completes more: every request adds at most one block begun before
-    const int most = a.T / a.block + a.S;
-    block_means_kernel<T, VEC><<<most, kWideThreads, 0, stream>>>(a);
-    NINFER_LAUNCH_CHECK();
-  }
-  return 0;
+  return launch_means<T, VEC>(a, stream);
 }
 
 }  // namespace ninfer
@@ -329,6 +481,16 @@ extern "C" int ninfer_qkv_wide(const QkvWideArgs* args, hipStream_t stream) {
   const bool pieces = a.dim % 8 == 0 && a.vdim % 8 == 0 && (a.interleaved || a.rot_dim % 16 == 0) &&
                       a.stride % 8 == 0 && a.q_col % 8 == 0 && a.k_col % 8 == 0 && a.v_col % 8 == 0 &&
                       (uintptr_t)a.u % 16 == 0;
-  if (pieces && a.force_plain != 1) return launch_wide<bf16, 8>(a, stream);
+  if (pieces && a.force_plain != 1) {
+    const int n = (a.Hq + a.Hkv) * a.dim;
+    const bool aligned = (uintptr_t)a.q_gain % 16 == 0 && (uintptr_t)a.k_gain % 16 == 0;
+    auto fits = [&](int rows) {
+      return aligned && n <= 8 * kWideRowsMaxThreads &&
+             (size_t)rows * (a.rot_dim + (a.interleaved ? 0 : n)) * sizeof(float) <= (size_t)kWideMaxLds;
+    };
+    if (!a.all_single && a.T >= 512 && fits(4)) return launch_wide_rows<4>(a, stream);
+    if (fits(1)) return launch_wide_rows<1>(a, stream);
+    return launch_wide<bf16, 8>(a, stream);
+  }
   return launch_wide<bf16, 1>(a, stream);
 }
