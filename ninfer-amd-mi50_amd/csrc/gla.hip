@@ -236,11 +236,19 @@ extern "C" int ninfer_gated_linear_attention(const void* qkv, int stride, int q_
 // a sum's terms is free), and a chunk costs it dim / 4 + 4 products for the outputs and
 // dim / 4 for the state, with the operands of the next chunk on their way meanwhile. Nothing
 // is rounded to a shorter type.
+//
+// A request's chunks in order are a long chain on few blocks when the step has few requests.
+// Then they are cut into segments of kGlaSegment chunks: every segment's state from a zero start
+// and its decays' products (all segments side by side), the states in front of the segments from
+// those (one pass over the segments, S <- E S + S_segment, a number of the state per thread),
+// and the outputs of all segments side by side, each from the state in front of it.
 namespace ninfer {
 
 typedef float gla_f32x4 __attribute__((ext_vector_type(4)));
 constexpr int kGlaChunk = 16;
 constexpr int kGlaChunkMaxDim = 128;
+constexpr int kGlaSegment = 8;                              // chunks of a segment
+constexpr int kGlaSegmentRows = kGlaSegment * kGlaChunk;
 
 struct GlaChunkArgs {
   GlaArgs g;
@@ -248,18 +256,21 @@ struct GlaChunkArgs {
   float* ke;     // [H, T, dim]  k e^(b_last - b)
   float* eb;     // [H, T, dim]  e^b
   float* A;      // [H, T, 16]
+  float* seg;    // [segments, H, dim, vdim]: a segment's state from zero, then the state in front of it
+  float* seg_e;  // [segments, H, dim]: the products of a segment's decays
   int T, S;
 };
 
-// The request and the first row of chunk `c` of the step (chunks are counted request after
-// request); false if the step has fewer chunks.
+// The request and the first row of chunk `c` of the step (chunks of `rows` rows are counted
+// request after request); false if the step has fewer chunks.
 __device__ __forceinline__ bool gla_find_chunk(const int* seq_row_start, int S, int c, int* r0,
-                                               int* i0, int* n) {
+                                               int* i0, int* n, int* seq = nullptr, int rows = kGlaChunk) {
   for (int s = 0; s < S; ++s) {
     const int a = seq_row_start[s], len = seq_row_start[s + 1] - a;
-    const int chunks = (len + kGlaChunk - 1) / kGlaChunk;
+    const int chunks = (len + rows - 1) / rows;
     if (c < chunks) {
-      *r0 = a, *i0 = c * kGlaChunk, *n = len;
+      *r0 = a, *i0 = c * rows, *n = len;
+      if (seq) *seq = s;
       return true;
     }
     c -= chunks;
@@ -356,15 +367,31 @@ struct GlaChunkRegs {
   float v[4];         // v[row 4 g + x][column c of the wave]
 };
 
-template <typename T, int DT>
+// What a block of the scan walks: a request's rows of the step; a segment of them from a zero
+// state, for the state it leaves only; a segment from the state in front of it, for its outputs.
+enum GlaScan : int { kGlaWhole, kGlaSegmentState, kGlaSegmentOut };
+
+template <typename T, int DT, int MODE>
 __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunkArgs a) {
-  const int s = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  int s = blockIdx.x;
+  const int h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int c = lane & 15, g = lane >> 4;
   const int col = (blockIdx.z * kGlaWaves + wave) * kGlaCols + c;
   const int dim = a.g.dim, vdim = a.g.vdim, H = a.g.H;
   const bool has_col = col < vdim;
-  const int r0 = a.g.seq_row_start[s], n = a.g.seq_row_start[s + 1] - r0;
-  float* st = a.g.state + (int64_t)a.g.seq_slots[s] * a.g.state_stride + (int64_t)h * dim * vdim;
+  int r0, n;
+  bool ends = true;   // the last piece of its request: the state after it goes to the request's slot
+  if constexpr (MODE == kGlaWhole) {
+    r0 = a.g.seq_row_start[s], n = a.g.seq_row_start[s + 1] - r0;
+  } else {
+    int i0;
+    if (!gla_find_chunk(a.g.seq_row_start, a.S, blockIdx.x, &r0, &i0, &n, &s, kGlaSegmentRows)) return;
+    ends = i0 + kGlaSegmentRows >= n;
+    r0 += i0, n = min(kGlaSegmentRows, n - i0);
+    if (MODE == kGlaSegmentState && ends) return;   // nobody starts from its state
+  }
+  float* slot = a.g.state + (int64_t)a.g.seq_slots[s] * a.g.state_stride + (int64_t)h * dim * vdim;
+  float* st = MODE == kGlaWhole ? slot : a.seg + ((int64_t)blockIdx.x * H + h) * dim * vdim;
   const int64_t head_row0 = (int64_t)h * a.T;   // the head's first row in the workspace
   // the state: S[16 dt + 4 g + x][col] in Sreg[dt][x]
   gla_f32x4 Sreg[DT];
@@ -373,8 +400,11 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
       const int d = 16 * dt + 4 * g + x;
-      Sreg[dt][x] = has_col && d < dim ? st[(int64_t)d * vdim + col] : 0.f;
+      Sreg[dt][x] = MODE != kGlaSegmentState && has_col && d < dim ? st[(int64_t)d * vdim + col] : 0.f;
     }
+  gla_f32x4 Ereg[DT];   // the products of the decays so far
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) Ereg[dt] = gla_f32x4{1.f, 1.f, 1.f, 1.f};
   const gla_f32x4 zero4 = {0.f, 0.f, 0.f, 0.f};
   // The loads of a chunk's operands, every one of them unconditional (a load inside a branch is
   // waited for where the branch ends): rows, channels and columns beyond the last are fetched
@@ -389,7 +419,7 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       const int d = min(16 * dt + 4 * g, dim - 4);   // (dim is a multiple of 4)
-      R.q[dt] = *(const gla_f32x4*)(qrow + d);
+      if constexpr (MODE != kGlaSegmentState) R.q[dt] = *(const gla_f32x4*)(qrow + d);
       R.e[dt] = *(const gla_f32x4*)(erow + d);
     }
 #pragma unroll
@@ -400,7 +430,8 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
       for (int dt = 0; dt < DT; ++dt) R.k[x][dt] = krow[min(16 * dt + c, dim - 1)];
       R.v[x] = to_f32(((const T*)a.g.qkv)[row * a.g.stride + a.g.v_off + h * vdim + col_c]);
     }
-    R.A = *(const gla_f32x4*)(a.A + (head_row0 + base + min(c, L - 1)) * kGlaChunk + 4 * g);
+    if constexpr (MODE != kGlaSegmentState)
+      R.A = *(const gla_f32x4*)(a.A + (head_row0 + base + min(c, L - 1)) * kGlaChunk + 4 * g);
   };
   // a chunk: its outputs from the state before it, then the state after it; the operands of the
   // chunk after the next one set out first (three sets of registers take turns)
@@ -410,7 +441,10 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
     // zeros where a sum runs over rows or channels that are not there
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      if (16 * dt + 4 * g >= dim) cur.q[dt] = zero4, cur.e[dt] = zero4;
+      if (16 * dt + 4 * g >= dim) {
+        if constexpr (MODE != kGlaSegmentState) cur.q[dt] = zero4;
+        cur.e[dt] = zero4;
+      }
 #pragma unroll
       for (int x = 0; x < 4; ++x)
         if (4 * g + x >= L || 16 * dt + c >= dim) cur.k[x][dt] = 0.f;
@@ -419,6 +453,7 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
     for (int x = 0; x < 4; ++x)
       if (4 * g + x >= L) cur.v[x] = 0.f;
     // the outputs: rows 4 g + x of column c in o[x] + o2[x]
+    if constexpr (MODE != kGlaSegmentState) {
     gla_f32x4 o = zero4, o2 = zero4;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -438,11 +473,15 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
         if (t < L) a.g.out[((int64_t)(r0 + i0 + t) * H + h) * vdim + col] = o[x] + o2[x];
       }
     }
+    }
     // the state after the chunk
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
 #pragma unroll
-      for (int x = 0; x < 4; ++x) Sreg[dt][x] *= cur.e[dt][x];
+      for (int x = 0; x < 4; ++x) {
+        Sreg[dt][x] *= cur.e[dt][x];
+        if constexpr (MODE == kGlaSegmentState) Ereg[dt][x] *= cur.e[dt][x];
+      }
 #pragma unroll
       for (int x = 0; x < 4; ++x)
         Sreg[dt] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.k[x][dt], cur.v[x], Sreg[dt], 0, 0, 0);
@@ -459,14 +498,48 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
     if (i0 + 2 * kGlaChunk >= n) break;
     chunk(R2, i0 + 2 * kGlaChunk, R1);
   }
+  if (MODE == kGlaSegmentOut && !ends) return;
+  float* to = MODE == kGlaSegmentState ? st : slot;
   if (has_col) {
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
       for (int x = 0; x < 4; ++x) {
         const int d = 16 * dt + 4 * g + x;
-        if (d < dim) st[(int64_t)d * vdim + col] = Sreg[dt][x];
+        if (d < dim) to[(int64_t)d * vdim + col] = Sreg[dt][x];
       }
+  }
+  if (MODE == kGlaSegmentState && blockIdx.z == 0 && wave == 0 && c == 0) {
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const int d = 16 * dt + 4 * g + x;
+        if (d < dim) a.seg_e[((int64_t)blockIdx.x * H + h) * dim + d] = Ereg[dt][x];
+      }
+  }
+}
+
+// The states in front of a request's segments, in place of the states the segments leave from
+// zero: a number of the state per thread.
+__global__ __launch_bounds__(256) void gla_segment_states_kernel(GlaChunkArgs a) {
+  const int s = blockIdx.y, dim = a.g.dim, vdim = a.g.vdim, H = a.g.H;
+  const int n = H * dim * vdim, e = blockIdx.x * 256 + threadIdx.x;
+  if (e >= n) return;
+  int first = 0;
+  for (int i = 0; i < s; ++i)
+    first += (a.g.seq_row_start[i + 1] - a.g.seq_row_start[i] + kGlaSegmentRows - 1) / kGlaSegmentRows;
+  const int count = (a.g.seq_row_start[s + 1] - a.g.seq_row_start[s] + kGlaSegmentRows - 1) / kGlaSegmentRows;
+  float S = a.g.state[(int64_t)a.g.seq_slots[s] * a.g.state_stride + e];
+  const int hd = e / vdim;
+#pragma unroll 8
+  for (int i = 0; i < count; ++i) {
+    float* at = a.seg + (int64_t)(first + i) * n + e;
+    // (the last segment has left neither a state nor decays: nothing comes after it)
+    const bool more = i + 1 < count;
+    const float left = more ? *at : 0.f, keep = more ? a.seg_e[(int64_t)(first + i) * H * dim + hd] : 0.f;
+    *at = S;
+    S = fmaf(keep, S, left);
   }
 }
 
@@ -474,7 +547,8 @@ __global__ __launch_bounds__(64 * kGlaWaves) void gla_chunk_scan_kernel(GlaChunk
 
 // The same as ninfer_gated_linear_attention for bfloat16 rows, in chunks of 16 rows on the
 // matrix cores: for steps that bring prompt portions. `work` holds T * (3 heads dim + 16 heads)
-// floats. Returns 1 (nothing launched) when the sizes do not fit.
+// floats. `segments` (or null): as many floats as ninfer_gla_segment_floats asks for, and the
+// step runs in segments. Returns 1 (nothing launched) when the sizes do not fit.
 extern "C" int ninfer_gated_linear_attention_chunks(const void* qkv, int stride, int q_off, int k_off,
                                                     int v_off, const float* z, float tau,
                                                     float q_scale, float* state,
@@ -482,7 +556,8 @@ extern "C" int ninfer_gated_linear_attention_chunks(const void* qkv, int stride,
                                                     const int* seq_row_start, const int* seq_slots,
                                                     float* work, int T, int S, int H, int dim,
                                                     int vdim, int dtype, int f_off, const float* f_bias,
-                                                    const float* lower, hipStream_t stream) {
+                                                    const float* lower, float* segments,
+                                                    hipStream_t stream) {
   NINFER_REQUIRE(T > 0 && S > 0 && H > 0 && dim > 0 && vdim > 0,
                  "gated_linear_attention: T=%d S=%d heads=%d dim=%d vdim=%d must be positive", T,
                  S, H, dim, vdim);
@@ -506,11 +581,33 @@ extern "C" int ninfer_gated_linear_attention_chunks(const void* qkv, int stride,
   if (lower) gla_chunk_prepare_kernel<bf16, true><<<dim3(chunks, H), 256, 0, stream>>>(a);
   else gla_chunk_prepare_kernel<bf16, false><<<dim3(chunks, H), 256, 0, stream>>>(a);
   const int cols = kGlaCols * kGlaWaves;
-  const dim3 grid(S, H, (vdim + cols - 1) / cols);
-  if (dim <= 16) gla_chunk_scan_kernel<bf16, 1><<<grid, 64 * kGlaWaves, 0, stream>>>(a);
-  else if (dim <= 32) gla_chunk_scan_kernel<bf16, 2><<<grid, 64 * kGlaWaves, 0, stream>>>(a);
-  else if (dim <= 64) gla_chunk_scan_kernel<bf16, 4><<<grid, 64 * kGlaWaves, 0, stream>>>(a);
-  else gla_chunk_scan_kernel<bf16, 8><<<grid, 64 * kGlaWaves, 0, stream>>>(a);
+  dim3 grid(S, H, (vdim + cols - 1) / cols);
+#define NINFER_GLA_SCAN(MODE)                                                                              \
+  do {                                                                                                     \
+    if (dim <= 16) gla_chunk_scan_kernel<bf16, 1, MODE><<<grid, 64 * kGlaWaves, 0, stream>>>(a);           \
+    else if (dim <= 32) gla_chunk_scan_kernel<bf16, 2, MODE><<<grid, 64 * kGlaWaves, 0, stream>>>(a);      \
+    else if (dim <= 64) gla_chunk_scan_kernel<bf16, 4, MODE><<<grid, 64 * kGlaWaves, 0, stream>>>(a);      \
+    else gla_chunk_scan_kernel<bf16, 8, MODE><<<grid, 64 * kGlaWaves, 0, stream>>>(a);                     \
+  } while (0)
+  if (segments) {
+    const int n_seg = T / kGlaSegmentRows + S;   // no step has more
+    a.seg = segments, a.seg_e = segments + (int64_t)n_seg * H * dim * vdim;
+    grid.x = n_seg;
+    NINFER_GLA_SCAN(kGlaSegmentState);
+    gla_segment_states_kernel<<<dim3((H * dim * vdim + 255) / 256, S), 256, 0, stream>>>(a);
+    NINFER_GLA_SCAN(kGlaSegmentOut);
+  } else {
+    NINFER_GLA_SCAN(kGlaWhole);
+  }
+#undef NINFER_GLA_SCAN
   NINFER_LAUNCH_CHECK();
   return 0;
+}
+
+// Floats of workspace with which a step of this shape runs in segments; 0 when it does not pay:
+// few rows, or requests enough to fill the device with one block per request, head and columns.
+extern "C" long long ninfer_gla_segment_floats(int T, int S, int H, int dim, int vdim) {
+  const int cols = kGlaCols * kGlaWaves;
+  if (T < 2 * kGlaSegmentRows * S || (long long)S * H * ((vdim + cols - 1) / cols) >= 2LL * device_cu_count()) return 0;
+  return (long long)(T / kGlaSegmentRows + S) * H * dim * (vdim + 1);
 }

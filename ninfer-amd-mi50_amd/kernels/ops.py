@@ -302,6 +302,7 @@ class HipOps:
         self.lib.ninfer_stream_after.argtypes = [ctypes.c_void_p] * 3
         self.lib.ninfer_sample_few_places.restype = ctypes.c_longlong
         self.lib.ninfer_latent_attention_workspace_floats.restype = ctypes.c_longlong
+        self.lib.ninfer_gla_segment_floats.restype = ctypes.c_longlong
         self.lib.ninfer_diff_attention_workspace_floats.restype = ctypes.c_longlong
         self.lib.ninfer_sigmoid_attention_workspace_floats.restype = ctypes.c_longlong
         self.force_generic = False  # tests: run the plain kernels whatever the shape
@@ -1592,7 +1593,8 @@ class HipOps:
         (heads x vdim) of `qkv`; z: [T, heads * dim] 32-bit. `state` ([slots, >= heads * dim *
         vdim] 32-bit view) holds every request's S between steps. out: [T, heads * vdim] 32-bit.
         `work` ([T, gla_work_floats(..)] 32-bit, or None): with it a bfloat16 step that brings
-        prompt portions runs in chunks of 16 rows on the matrix cores (the sums of a chunk are
+        prompt portions runs in chunks of 16 rows on the matrix cores, and long portions of few
+        requests in segments of such chunks side by side (the sums of a chunk are
         ordered otherwise than token by token, so the 32-bit path, whose logits do not depend
         on the cut to the bit, stays on the token-by-token kernel). `forget` (f_off, bias,
         lower): the form with a forget gate f = lower + (1 - lower) sigmoid(w + bias), w the
@@ -1625,13 +1627,16 @@ class HipOps:
             _need(work.is_contiguous() and work.shape[0] == t
                   and work.shape[1] >= 3 * heads * dim + 16 * heads,
                   "gated_linear_attention: the workspace is too small")
+            floats = int(self.lib.ninfer_gla_segment_floats(t, ctx.S, heads, dim, vdim))
+            seg = torch.empty(floats, dtype=torch.float32, device=qkv.device) if floats else None
             rc = self.lib.ninfer_gated_linear_attention_chunks(
                 ctypes.c_void_p(qkv.data_ptr()), row, q_off, k_off, v_off,
                 ctypes.c_void_p(_ptr(z)), ctypes.c_float(tau), ctypes.c_float(q_scale),
                 ctypes.c_void_p(state.data_ptr()), ctypes.c_longlong(state.stride(0)),
                 ctypes.c_void_p(out.data_ptr()), ctypes.c_void_p(ctx.seq_row_start.data_ptr()),
                 ctypes.c_void_p(ctx.seq_slots.data_ptr()), ctypes.c_void_p(work.data_ptr()),
-                t, ctx.S, heads, dim, vdim, _DT[qkv.dtype], *gate_args, self._stream())
+                t, ctx.S, heads, dim, vdim, _DT[qkv.dtype], *gate_args,
+                ctypes.c_void_p(_ptr(seg)), self._stream())
             if rc == 0:
                 return
             if rc < 0:
