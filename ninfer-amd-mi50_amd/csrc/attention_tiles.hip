@@ -240,7 +240,9 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_kernel(AttnArgs a, int
   const int blocks_last = a.kblk ? attention_blocks_seen(pos_last, a.window, a.block) : 0;
   const int n_bt = (blocks_last + 63) / 64;
 
-  // zeros everywhere once: the padding columns stay zero, the rest is overwritten
+  // zeros everywhere once where heads are shorter than the tile's rows: the padding columns stay
+  // zero, the rest is overwritten
+  if (dim < 16 * KS || vdim < 32 * DB)
   for (int i = tid; i < 2 * TILE / 8; i += 256) ((at_u32x4*)lds)[i] = at_u32x4{0u, 0u, 0u, 0u};
 
   Mover mv;
@@ -354,7 +356,7 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
   const int c = lane & 31, hi = lane >> 5;
   const int hpg = a.Hq / a.Hkv;
   const int t = blockIdx.x, g = blockIdx.y, ch = blockIdx.z;
-  const int pos = a.positions[t];
+  const int pos = a.positions[t], seq = a.row_seq[t];
   const int first = a.window > 0 ? max(0, pos - a.window + 1) : 0;
   const int dim = a.D, vdim = a.Dv;
   const bool q_valid = c < hpg;
@@ -378,11 +380,18 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
     }
     return;
   }
-  const int seq = a.row_seq[t];
-
-  for (int i = tid; i < TILE / 8; i += 128) ((at_u32x4*)lds)[i] = at_u32x4{0u, 0u, 0u, 0u};
   Mover mv;
   mv.init(tid, dim, vdim);
+  auto fetch = [&](int it) {
+    const bool is_b = it < n_bt;
+    const TileSource src = tile_source(a, seq, is_b);
+    mv.load(src.k, src.v, src.bt, src.ps_shift, src.page_size - 1, src.page_size, a.Hkv, g, dim, vdim,
+            (is_b ? it : kt0 + it - n_bt) * 64, is_b ? 0 : first, is_b ? n_blocks - 1 : pos);
+  };
+  fetch(it0);
+  // zeros in the padding of short heads (heads that fill the tile's rows leave none)
+  if (dim < 16 * KS || vdim < 32 * DB)
+    for (int i = tid; i < TILE / 8; i += 128) ((at_u32x4*)lds)[i] = at_u32x4{0u, 0u, 0u, 0u};
 
   at_bf16x8 qf[KS];
   {
@@ -407,13 +416,6 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
   const int s16 = lane & 15, q4 = lane >> 4;
   const int v_lane = (4 * hi + s16 / 4) * VROW + 16 * (q4 & 1) + 4 * (s16 & 3);
 
-  auto fetch = [&](int it) {
-    const bool is_b = it < n_bt;
-    const TileSource src = tile_source(a, seq, is_b);
-    mv.load(src.k, src.v, src.bt, src.ps_shift, src.page_size - 1, src.page_size, a.Hkv, g, dim, vdim,
-            (is_b ? it : kt0 + it - n_bt) * 64, is_b ? 0 : first, is_b ? n_blocks - 1 : pos);
-  };
-  fetch(it0);
   __syncthreads();
   for (int it = it0; it < it1; ++it) {
     const bool is_b = it < n_bt;

@@ -418,6 +418,41 @@ def test_recurrence_with_a_forget_gate(ops, dtype, plain_kernel, heads, dim, vdi
     assert (state[:, :4] == 7).all() and (state[:, 4 + floats:] == 7).all() and (state[1, 4:4 + floats] == 0).all()
 
 
+@pytest.mark.parametrize("lens,first", [([300, 129, 700], 0), ([128, 1, 640], 5), ([513], 2), ([256, 257], 16)])
+def test_recurrence_in_long_portions_of_several_requests(ops, lens, first):
+    """Long portions side by side, each after `first` rows in a step before: pieces of a request
+    that the kernels work on side by side, whole ones and short last ones, a request that is
+    shorter than a piece; the state they leave, and one more row after it."""
+    heads, dim, vdim = 2, 20, 24
+    g = torch.Generator().manual_seed(sum(lens))
+    n = heads * dim
+    total = [first + ln + 1 for ln in lens]
+    u_all = [torch.randn(t, 2 * n + heads * vdim, generator=g).to(torch.bfloat16) for t in total]
+    bias, lower = torch.randn(n, generator=g) + 2, torch.rand(n, generator=g)
+    state = torch.zeros(len(lens), heads * dim * vdim, device=DEV)
+    got = [torch.zeros(t, heads * vdim) for t in total]
+    cuts = [([first] if first else []) + [ln, 1] for ln in lens]
+    slots = list(range(len(lens)))[::-1]
+    for ctx, who, starts, counts in _steps(ops, torch.bfloat16, cuts, slots):
+        u = torch.cat([u_all[r][s:s + c] for r, s, c in zip(who, starts, counts)]).to(DEV)
+        out = torch.empty(ctx.T, heads * vdim, device=DEV)
+        wf = ops.gla_work_floats(torch.bfloat16, ctx, heads, dim)
+        work = torch.empty(ctx.T, wf, device=DEV) if wf else None
+        ops.gated_linear_attention(u, 0, 0, 2 * n, None, heads, dim, vdim, 1.0, 1.0, state, ctx, out, work=work,
+                                   forget=(n, bias.to(DEV), lower.to(DEV)))
+        o = 0
+        for r, s, c in zip(who, starts, counts):
+            got[r][s:s + c] = out[o:o + c].cpu()
+            o += c
+    assert ops.lib.ninfer_gla_segment_floats(sum(lens), len(lens), heads, dim, vdim) > 0
+    for r, t in enumerate(total):
+        u = u_all[r].double()
+        f = plain.forget_gates(u[:, n:2 * n] + bias.double(), lower).view(t, heads, dim)
+        o, last = plain.gated_recurrence(plain.silu(u[:, :n]).view(t, heads, dim), f, u[:, 2 * n:].reshape(t, heads, vdim))
+        assert rel_err(got[r], o.reshape(t, -1)) < 1e-5
+        assert rel_err(state[slots[r]], last.reshape(-1)) < 1e-5
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_recurrence_remembers_and_forgets(ops, dtype):
     """A loud token hundreds of rows back: a channel whose gate is all but open keeps it to the
