@@ -104,7 +104,7 @@ __device__ __forceinline__ void wide_block_mean(const QkvWideArgs& a, const int*
 #pragma unroll
   for (int e = 0; e < VEC; ++e) sum[e] = 0.f;
   const int upto = a.block - (last ? 1 : 0);
-#pragma unroll 4
+#pragma unroll 8
   for (int j = 0; j < upto; ++j) {
     const int p = first + j;
     float v[VEC];
@@ -488,7 +488,7 @@ extern "C" int ninfer_qkv_wide(const QkvWideArgs* args, hipStream_t stream) {
       return aligned && n <= 8 * kWideRowsMaxThreads &&
              (size_t)rows * (a.rot_dim + (a.interleaved ? 0 : n)) * sizeof(float) <= (size_t)kWideMaxLds;
     };
-    if (!a.all_single && a.T >= 512 && fits(4)) return launch_wide_rows<4>(a, stream);
+    if (!a.all_single && a.T >= 512 && fits(2)) return launch_wide_rows<2>(a, stream);
     if (fits(1)) return launch_wide_rows<1>(a, stream);
     return launch_wide<bf16, 8>(a, stream);
   }

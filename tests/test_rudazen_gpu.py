@@ -134,8 +134,8 @@ def _rows(tables, who, width):
 @pytest.mark.parametrize("heads,kv,dim,vdim,rot,pairing,pool,temp,rows", [
     (6, 3, 20, 20, 10, "interleaved", 3, False, 1), (4, 2, 64, 64, 64, "interleaved", 8, False, 1),
     (8, 2, 64, 32, 32, "half", None, True, 1), (2, 1, 88, 72, 40, "half", None, True, 1), (3, 1, 36, 36, 36, "interleaved", 7, True, 1),
-    (2, 2, 16, 16, 0, "half", 1, False, 1), (1, 1, 8, 40, 8, "half", 5, True, 1), (16, 4, 128, 128, 128, "interleaved", 16, False, 8),
-    (16, 4, 128, 128, 64, "half", 16, True, 8), (40, 8, 256, 256, 32, "half", None, False, 3), (5, 1, 128, 128, 12, "interleaved", 4, False, 9)])
+    (2, 2, 16, 16, 0, "half", 1, False, 1), (1, 1, 8, 40, 8, "half", 5, True, 1), (16, 4, 128, 128, 128, "interleaved", 16, False, 16),
+    (16, 4, 128, 128, 64, "half", 16, True, 16), (40, 8, 256, 256, 32, "half", None, False, 16), (5, 1, 128, 128, 12, "interleaved", 4, False, 16)])
 def test_projected_rows_on_their_way_to_attention(ops, dtype, plain_kernel, heads, kv, dim, vdim, rot, pairing, pool, temp, rows):
     """Whole-projection norms, a rotation with a magnitude, the factor per head, the cache write
     (values of their own or the keys' own columns) and the means of completed blocks: three
@@ -162,7 +162,7 @@ def test_projected_rows_on_their_way_to_attention(ops, dtype, plain_kernel, head
         blk = {"k_block": torch.full((bpages, kv, bps, dim), float("nan"), dtype=dtype, device=DEV),
                "v_block": torch.full((bpages, kv, bps, vdim), float("nan"), dtype=dtype, device=DEV)}
     got_q = [torch.zeros(n, nq) for n in lens]
-    cuts = [_cut(lens[0], [13, 2, 9 * rows, 3], 6), _cut(7, [3, 2], 2), _cut(lens[2], [2, 11 * rows, 1, 8], 4)]
+    cuts = [_cut(lens[0], [13, 2, (9 if rows == 1 else 36 * rows + 1), 3], 6), _cut(7, [3, 2], 2), _cut(lens[2], [2, 11 * rows, 1, 8], 4)]
     for ctx, who, starts, counts in _steps(ops, dtype, cuts, [0, 1, 2]):
         wide = torch.zeros(ctx.T, ch + 24, dtype=dtype, device=DEV)
         wide[:, 8:8 + ch] = torch.cat([u_all[i][s:s + n] for i, s, n in zip(who, starts, counts)]).to(DEV)
@@ -179,7 +179,8 @@ def test_projected_rows_on_their_way_to_attention(ops, dtype, plain_kernel, head
         for i, s, n in zip(who, starts, counts):
             got_q[i][s:s + n] = q[o:o + n].float().cpu()
             o += n
-    tol = 3e-6 if dtype == torch.float32 else 6e-3
+    # (a 32-bit angle of hundreds of radians is off by some 1e-5)
+    tol = (3e-6 if rows == 1 else 1e-5) if dtype == torch.float32 else 6e-3
     for i, n in enumerate(lens):
         x, pos = u_all[i].double(), torch.arange(n)
         q = plain.rotate(plain.rms_norm(x[:, :nq], qn, eps).reshape(n, heads, dim), pos, r if rot else None, pairing)
