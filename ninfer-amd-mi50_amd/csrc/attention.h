@@ -39,6 +39,7 @@ struct AttnArgs {
                             // [T, Hq*Dv] (0: the same as D)
   int sink;                 // != 0: the softmax's denominator has one more term, exp(0), that
                             // belongs to no key (a sink with score 0 and no value)
+                            // (with `sinks`, below, exp(sinks[h]): a sink of a learned score)
   // Beside the keys of its window a row may see one key and value per block of `block` tokens
   // that lies wholly before the window: block b (positions b block .. b block + block - 1) where
   // b block + block - 1 <= position - window. Keys and blocks share one softmax.
@@ -51,7 +52,11 @@ struct AttnArgs {
   // a gate on the output: out[t, c] times sigmoid(gate[t * gate_stride + c]), c < Hq * Dv
   const void* gate;         // of the activation dtype, or null
   int gate_stride;
+  const float* sinks;       // [Hq] or null (0): the score of head h's sink, not scaled
 };
+
+// The score of head h's sink.
+__device__ __forceinline__ float attention_sink(const AttnArgs& a, int h) { return a.sinks ? a.sinks[h] : 0.f; }
 
 // How many blocks a row at this position sees (they are the first ones of its request).
 __host__ __device__ inline int attention_blocks_seen(int pos, int window, int block) {

@@ -30,6 +30,7 @@ int attention_check(const AttnArgs& args) {
   NINFER_REQUIRE(!a->kblk || !a->slopes, "paged_attention: a position bias beside blocks is not built");
   NINFER_REQUIRE(!a->gate || a->gate_stride >= a->Hq * (a->Dv > 0 ? a->Dv : a->D),
                  "paged_attention: the gate's rows of %d are too short", a->gate_stride);
+  NINFER_REQUIRE(!a->sinks || a->sink, "paged_attention: scores of sinks without a sink");
   return 0;
 }
 }  // namespace ninfer
@@ -65,7 +66,7 @@ extern "C" int ninfer_paged_attention(const AttnArgs* a, int force_generic, hipS
   const int n = a->max_qlen == 1 ? a->S : a->single_rows;
   const bool tiles = !force_generic && attention_tiles_takes(*a);
   const bool apart = tiles && n > 0 && attention_tiles_heads_takes(*a) &&
-                     (!attention_prefill_takes(*a) || a->kblk || a->gate);
+                     (!attention_prefill_takes(*a) || a->kblk || a->gate || a->sink);
   if (apart) {
     AttnArgs d = *a;
     d.T = n;

@@ -37,8 +37,8 @@ __global__ __launch_bounds__(64) void paged_attention_generic_kernel(AttnArgs a)
   for (int d = lane; d < D; d += 64) q_s[d] = to_f32(qr[d]);
   __syncthreads();
 
-  // (a sink is a key with score 0 and no value: the running maximum starts at 0, the sum at 1)
-  float m = a.sink ? 0.f : -INFINITY, l = a.sink ? 1.f : 0.f;
+  // (a sink is a key without a value: the running maximum starts at its score, the sum at 1)
+  float m = a.sink ? attention_sink(a, h) : -INFINITY, l = a.sink ? 1.f : 0.f;
   float acc[kMaxDPerLane];
 #pragma unroll
   for (int i = 0; i < kMaxDPerLane; ++i) acc[i] = 0.f;

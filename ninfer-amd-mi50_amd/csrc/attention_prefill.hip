@@ -33,7 +33,7 @@
 // the tiles of the blocks that the rows see come in front of the keys' tiles: in the kernel
 // they lie at "keys" before t_first, and a tile there takes its rows from the blocks' pools
 // and pages and its bounds from how many blocks a row sees. The output may be gated, element by
-// element, where it is written.
+// element, where it is written. A softmax with a sink starts from the sink's score.
 //
 // The same kernel serves decoding for models whose kv heads are shared by three
 // or more query heads (HEADS): the 32 "rows" of a block are then the query
@@ -211,7 +211,10 @@ __global__ __launch_bounds__(NQ * 128, 2) void attn_prefill_kernel(AttnArgs a, i
   // scale is applied to score + bias together)
   const bool biased = a.slopes != nullptr;
   const float slope_raw = biased ? a.slopes[h + (HEADS ? (q_valid ? q_local : 0) : 0)] / a.scale : 0.f;
-  float m = -1e30f, l = 0.f;
+  // a sink is a key without a value: the running maximum starts at its score; it counts once in
+  // the row's sum, in one of the row's two lanes of the wave that meets the first key half
+  const bool with_sink = !HEADS && a.sink && kh == 0;
+  float m = with_sink ? attention_sink(a, h) * 1.44269504088896f : -1e30f, l = with_sink && j == 0 ? 1.f : 0.f;
 
   // Loads. Load i of wave w fills piece i NW + w of a tile's keys (and the same piece of its
   // values): RPP rows, lane l at row l / CPR, position l % CPR, which takes the row's chunk
@@ -602,7 +605,7 @@ int attention_decode_heads(const AttnArgs& a, int chunk, int n_chunks, hipStream
 
 bool attention_prefill_takes(const AttnArgs& a) {
   return a.dtype == kBF16 && (a.D == 64 || a.D == 128) && a.q_stride % 8 == 0 &&
-         prefill_page_ok(a) && a.seq_row_start != nullptr && (a.Dv == 0 || a.Dv == a.D) && !a.sink &&
+         prefill_page_ok(a) && a.seq_row_start != nullptr && (a.Dv == 0 || a.Dv == a.D) &&
          (!a.kblk || (a.blk_page_size == a.page_size && !a.slopes)) &&
          (!a.gate || (a.gate_stride % 4 == 0 && (uintptr_t)a.gate % 8 == 0));
 }

@@ -18,8 +18,8 @@
 // are the B operand of
 //   O^T[value column][row] += V^T P^T   (A = V^T: the transposing LDS read hands a lane four
 //                                        consecutive keys of one value column)
-// with the contraction index numbered as the lanes hold it. A sink is a key with score 0 and
-// no value: the running maximum starts at 0 and the running sum at 1.
+// with the contraction index numbered as the lanes hold it. A sink is a key without
+// a value: the running maximum starts at its score and the running sum at 1.
 //
 // Single rows (decode steps): a block of two waves owns one row and one kv head, the query heads
 // of the kv head (at most 32) are the tile's rows, so that the keys and values of the kv head
@@ -276,7 +276,7 @@ __global__ __launch_bounds__(256, 2) void attention_tiles_kernel(AttnArgs a, int
   for (int db = 0; db < DB; ++db)
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[db][v] = 0.f;
-  float m = a.sink ? 0.f : -1e30f, l = a.sink ? 1.f : 0.f;
+  float m = a.sink ? attention_sink(a, h) * kAtLog2e : -1e30f, l = a.sink ? 1.f : 0.f;
 
   // the transposing read's address of this lane inside a value tile: lane s of a group of 16
   // fetches key s / 4 (+ 4 hi), value columns 16 (group % 2) + 4 (s % 4) .. + 3
@@ -412,7 +412,7 @@ __global__ __launch_bounds__(128, 2) void attention_tiles_heads_kernel(AttnArgs 
     for (int v = 0; v < 16; ++v) o[db][v] = 0.f;
   // the sink counts once: in the first wave's sum of the first chunk
   const bool with_sink = a.sink && kb == 0 && ch == 0;
-  float m = with_sink ? 0.f : -1e30f, l = with_sink ? 1.f : 0.f;
+  float m = with_sink ? attention_sink(a, h) * kAtLog2e : -1e30f, l = with_sink ? 1.f : 0.f;
   const int s16 = lane & 15, q4 = lane >> 4;
   const int v_lane = (4 * hi + s16 / 4) * VROW + 16 * (q4 & 1) + 4 * (s16 & 3);
 

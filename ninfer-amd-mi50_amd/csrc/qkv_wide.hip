@@ -7,6 +7,9 @@
 //        `magnitude`: pair i is (i, i + rot_dim / 2), or the neighbours (2i, 2i + 1) when
 //        `interleaved`; a query head is multiplied by head_scale[h] where that is given (a
 //        factor on the head's scores);
+//   with `unit_heads` every query and key head is divided by its root mean square instead (over
+//        its dim numbers, eps inside the root, no gain): before or after it turns is the same, a
+//        rotation keeps the sum of the squares (`magnitude` is 1 then);
 //   queries go to q_out [T, Hq * dim]; keys and values to the request's pages. Values are columns
 //        of the projected row from v_col on: columns of their own, or the keys' own columns
 //        (values that are the keys as projected, before norm and rotation).
@@ -60,6 +63,7 @@ struct QkvWideArgs {
   float magnitude;
   int all_single;           // every request of the step brings one row
   int force_plain;          // tests: 1 the kernel of single numbers, 2 the kernel of whole pieces
+  int unit_heads;           // every query and key head divided by its root mean square
 };
 
 constexpr int kWideThreads = 256;
@@ -140,6 +144,7 @@ __global__ __launch_bounds__(kWideThreads) void qkv_wide_kernel(QkvWideArgs a) {
   const int nq = a.Hq * a.dim, nk = a.Hkv * a.dim, nv = a.Hkv * a.vdim;
   float* row_s = smem;                 // [nq + nk]
   float* trig = row_s + nq + nk;       // [rot_dim]: cos, then sin
+  float* inv_s = trig + a.rot_dim;     // [Hq + Hkv] 1 / root mean square of each head, with unit_heads
   const int t = blockIdx.x, tid = threadIdx.x;
   const int s = a.row_seq[t], pos = a.positions[t];
   const int half = a.rot_dim / 2;
@@ -173,6 +178,15 @@ __global__ __launch_bounds__(kWideThreads) void qkv_wide_kernel(QkvWideArgs a) {
   for (int i = 0; i < kWideThreads / 64; ++i) sq += red[0][i], sk += red[1][i];
   const float inv_q = a.q_gain ? 1.f / sqrtf(sq / (float)nq + a.eps) : 1.f;
   const float inv_k = a.k_gain ? 1.f / sqrtf(sk / (float)nk + a.eps) : 1.f;
+  if (a.unit_heads) {   // a wave per head
+    for (int hd = tid >> 6; hd < a.Hq + a.Hkv; hd += kWideThreads / 64) {
+      float ss = 0.f;
+      for (int d = tid & 63; d < a.dim; d += 64) ss = fmaf(row_s[hd * a.dim + d], row_s[hd * a.dim + d], ss);
+      ss = wave_sum(ss);
+      if ((tid & 63) == 0) inv_s[hd] = 1.f / sqrtf(ss / (float)a.dim + a.eps);
+    }
+    __syncthreads();
+  }
   const int64_t page = bt[pos / a.page_size];
   const int slot = pos % a.page_size;
   // the block that this row's token completes, when the row itself forms its means
@@ -186,10 +200,11 @@ __global__ __launch_bounds__(kWideThreads) void qkv_wide_kernel(QkvWideArgs a) {
     const float* head = row_s + i - d0;
     const float* gain = is_q ? a.q_gain : a.k_gain;
     const float* hg = gain ? gain + j0 - d0 : nullptr;
-    const float inv = is_q ? inv_q : inv_k;
+    const float inv = a.unit_heads ? inv_s[is_q ? hd : a.Hq + hd] : is_q ? inv_q : inv_k;
+    const float plain = a.unit_heads ? inv : 1.f;   // the factor where there are no gains
     float x[VEC];
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) x[e] = head[d0 + e] * (hg ? inv * hg[d0 + e] : 1.f);
+    for (int e = 0; e < VEC; ++e) x[e] = head[d0 + e] * (hg ? inv * hg[d0 + e] : plain);
     if constexpr (VEC == 8) {
       if (a.interleaved) {
 #pragma unroll
@@ -206,7 +221,7 @@ __global__ __launch_bounds__(kWideThreads) void qkv_wide_kernel(QkvWideArgs a) {
         const int o0 = first ? d0 + half : d0 - half, p0 = first ? d0 : d0 - half;
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
-          const float y = head[o0 + e] * (hg ? inv * hg[o0 + e] : 1.f);
+          const float y = head[o0 + e] * (hg ? inv * hg[o0 + e] : plain);
           const float cs = trig[p0 + e], sn = trig[half + p0 + e];
           x[e] = first ? x[e] * cs - y * sn : x[e] * cs + y * sn;
         }
@@ -215,7 +230,7 @@ __global__ __launch_bounds__(kWideThreads) void qkv_wide_kernel(QkvWideArgs a) {
       const bool first = a.interleaved ? !(d0 & 1) : d0 < half;
       const int o = a.interleaved ? d0 ^ 1 : first ? d0 + half : d0 - half;
       const int p = a.interleaved ? d0 >> 1 : first ? d0 : d0 - half;
-      const float y = head[o] * (hg ? inv * hg[o] : 1.f);
+      const float y = head[o] * (hg ? inv * hg[o] : plain);
       x[0] = first ? x[0] * trig[p] - y * trig[half + p] : x[0] * trig[p] + y * trig[half + p];
     }
     if (is_q) {
@@ -263,6 +278,8 @@ __global__ __launch_bounds__(kWideRowsMaxThreads) void qkv_wide_rows_kernel(QkvW
   const int half = a.rot_dim / 2, t0 = blockIdx.x * ROWS;
   float* trig = smem;                          // [ROWS][rot_dim]: cos, then sin
   float* x_s = smem + ROWS * a.rot_dim;        // [ROWS][nq + nk], for half-split pairs
+  // [ROWS][pieces] the squares' sums of the pieces, with unit_heads
+  float* piece_s = x_s + (a.interleaved ? 0 : ROWS * (nq + nk));
   const int i = 8 * tid;
   const bool live = i < nq + nk, is_q = i < nq;
   const int j0 = is_q ? i : i - nq;
@@ -305,6 +322,10 @@ __global__ __launch_bounds__(kWideRowsMaxThreads) void qkv_wide_rows_kernel(QkvW
       *(float4*)dst = make_float4(f[0] * g[0], f[1] * g[1], f[2] * g[2], f[3] * g[3]);
       *(float4*)(dst + 4) = make_float4(f[4] * g[4], f[5] * g[5], f[6] * g[6], f[7] * g[7]);
     }
+    if (a.unit_heads) {
+      if (live) piece_s[r * ((nq + nk) / 8) + tid] = ss;
+      continue;
+    }
     const float sq = has_q ? wave_sum(is_q ? ss : 0.f) : 0.f;
     const float sk = has_k ? wave_sum(is_q ? 0.f : ss) : 0.f;
     if ((tid & 63) == 0) red[r][wave][0] = sq, red[r][wave][1] = sk;
@@ -314,9 +335,15 @@ __global__ __launch_bounds__(kWideRowsMaxThreads) void qkv_wide_rows_kernel(QkvW
   for (int r = 0; r < ROWS; ++r) {
     const int t = t0 + r;
     if (t >= a.T) break;
-    float sum = 0.f;
-    for (int w = 0; w < nt / 64; ++w) sum += red[r][w][is_q ? 0 : 1];
-    const float inv = gain ? 1.f / sqrtf(sum / (float)(is_q ? nq : nk) + a.eps) : 1.f;
+    float sum = 0.f, over = (float)(is_q ? nq : nk);
+    if (a.unit_heads) {   // (heads of whole pieces: the piece's head begins d0 / 8 pieces before it)
+      const float* p = piece_s + r * ((nq + nk) / 8) + (live ? tid - d0 / 8 : 0);
+      for (int i = 0; i < a.dim / 8; ++i) sum += p[i];
+      over = (float)a.dim;
+    } else {
+      for (int w = 0; w < nt / 64; ++w) sum += red[r][w][is_q ? 0 : 1];
+    }
+    const float inv = gain || a.unit_heads ? 1.f / sqrtf(sum / over + a.eps) : 1.f;
     const int* bt = a.block_table + (int64_t)seq[r] * a.bt_stride;
     const int64_t page = bt[pos[r] / a.page_size];
     const int slot = pos[r] % a.page_size;
@@ -435,7 +462,7 @@ static int launch_means(const QkvWideArgs& a, hipStream_t stream) {
 template <int ROWS>
 static int launch_wide_rows(const QkvWideArgs& a, hipStream_t stream) {
   const int n = (a.Hq + a.Hkv) * a.dim;
-  const size_t lds = (size_t)ROWS * (a.rot_dim + (a.interleaved ? 0 : n)) * sizeof(float);
+  const size_t lds = (size_t)ROWS * (a.rot_dim + (a.interleaved ? 0 : n) + (a.unit_heads ? n / 8 : 0)) * sizeof(float);
   static bool raised = false;
   if (int rc = wide_lds(qkv_wide_rows_kernel<ROWS>, lds, &raised)) return rc;
   qkv_wide_rows_kernel<ROWS><<<(a.T + ROWS - 1) / ROWS, (n / 8 + 63) / 64 * 64, lds, stream>>>(a);
@@ -445,7 +472,7 @@ static int launch_wide_rows(const QkvWideArgs& a, hipStream_t stream) {
 
 template <typename T, int VEC>
 static int launch_wide(const QkvWideArgs& a, hipStream_t stream) {
-  const size_t lds = (size_t)((a.Hq + a.Hkv) * a.dim + a.rot_dim) * sizeof(float);
+  const size_t lds = (size_t)((a.Hq + a.Hkv) * (a.dim + (a.unit_heads ? 1 : 0)) + a.rot_dim) * sizeof(float);
   NINFER_REQUIRE(lds <= (size_t)kWideMaxLds, "qkv_wide: rows of %d queries' and keys' numbers exceed LDS",
                  (a.Hq + a.Hkv) * a.dim);
   static bool raised = false;
@@ -470,6 +497,8 @@ extern "C" int ninfer_qkv_wide(const QkvWideArgs* args, hipStream_t stream) {
                  "qkv_wide: columns outside rows of %d", a.stride);
   NINFER_REQUIRE(a.rot_dim >= 0 && a.rot_dim % 2 == 0 && a.rot_dim <= a.dim && (a.rot_dim == 0 || a.inv_freq),
                  "qkv_wide: %d turning numbers of %d", a.rot_dim, a.dim);
+  NINFER_REQUIRE(!a.unit_heads || (!a.q_gain && !a.k_gain && a.magnitude == 1.f),
+                 "qkv_wide: heads of unit size beside gains or a scaled rotation");
   NINFER_REQUIRE(a.kpool && a.vpool && a.block_table && a.page_size > 0 && a.bt_stride > 0,
                  "qkv_wide: keys and values without pages");
   NINFER_REQUIRE(a.block >= 0 && (a.block == 0 || (a.kblk && a.vblk && a.blk_table && a.blk_page_size > 0 &&
@@ -486,7 +515,8 @@ extern "C" int ninfer_qkv_wide(const QkvWideArgs* args, hipStream_t stream) {
     const bool aligned = (uintptr_t)a.q_gain % 16 == 0 && (uintptr_t)a.k_gain % 16 == 0;
     auto fits = [&](int rows) {
       return aligned && n <= 8 * kWideRowsMaxThreads &&
-             (size_t)rows * (a.rot_dim + (a.interleaved ? 0 : n)) * sizeof(float) <= (size_t)kWideMaxLds;
+             (size_t)rows * (a.rot_dim + (a.interleaved ? 0 : n) + (a.unit_heads ? n / 8 : 0)) * sizeof(float) <=
+                 (size_t)kWideMaxLds;
     };
     if (!a.all_single && a.T >= 512 && fits(2)) return launch_wide_rows<2>(a, stream);
     if (fits(1)) return launch_wide_rows<1>(a, stream);

@@ -9,7 +9,8 @@
 //                  sum of rows.
 //   gated_rmsnorm  out = o rsqrt(mean(o^2) + eps) w sigmoid(g) (or w g sigmoid(g)), the norm
 //                  over the whole row or over every group of columns (a head's) by itself;
-//                  without a gate the last factor is 1.
+//                  without a gate the last factor is 1. Or with the gate in front of the norm,
+//                  o <- o act(g) first; with a divisor per group, o <- o / den first.
 //   post_norm      x <- z rsqrt(mean(z^2) + eps) g with z = alpha x + y, written in 32-bit and
 //                  once more in the activation dtype for whoever reads x next; y a row, a
 //                  weighted sum of rows, or half-and-half of two normed rows.
@@ -300,43 +301,84 @@ __global__ void post_norm_kernel(PostNormArgs a) {
   }
 }
 
+struct GatedNormArgs {
+  const float* o;       // [T, N]
+  const void* gate;     // [T, gate_stride] or null
+  const float* w;       // [w_n]: a number per column of the row (w_n = N) or of a group
+  const float* den;     // [T, N / group] or null: what a group's numbers are divided by first
+  void* out;            // [T, N]
+  int gate_stride, T, N, group, w_n, silu, gate_first, dtype;
+  float eps;
+};
+
+// A number of the row as the norm takes it, and the factor that follows the norm.
 template <typename T>
-__global__ void gated_rmsnorm_kernel(const float* __restrict__ o, const T* __restrict__ gate,
-                                     int gate_stride, const float* __restrict__ w,
-                                     T* __restrict__ out, int N, float eps, int silu) {
+__device__ __forceinline__ float gated_norm_in(const GatedNormArgs& a, int64_t r, int i, float inv_den, float* after) {
+  float v = a.o[r * a.N + i] * inv_den;
+  float sg = 1.f;
+  if (a.gate) {
+    const float z = to_f32(((const T*)a.gate)[r * a.gate_stride + i]);
+    sg = (a.silu ? z : 1.f) / (1.f + expf(-z));
+  }
+  if (a.gate_first) v *= sg, sg = 1.f;
+  *after = sg;
+  return v;
+}
+
+// A block per (row, group); a thread keeps its (at most 16) numbers in registers.
+constexpr int kGatedPerThread = 16;
+template <typename T>
+__global__ void gated_rmsnorm_kernel(GatedNormArgs a) {
   __shared__ float red[16];
   const int64_t r = blockIdx.x;
-  const float* orow = o + r * N;
+  const int g0 = blockIdx.y * a.group;
+  const float inv_den = a.den ? 1.f / a.den[r * gridDim.y + blockIdx.y] : 1.f;
+  const float* w = a.w + (a.w_n == a.N ? g0 : 0);
+  float v[kGatedPerThread], sg[kGatedPerThread];
   float ss = 0.f;
-  for (int i = threadIdx.x; i < N; i += blockDim.x) ss = fmaf(orow[i], orow[i], ss);
+#pragma unroll
+  for (int c = 0; c < kGatedPerThread; ++c) {
+    const int i = threadIdx.x + c * blockDim.x;
+    v[c] = sg[c] = 0.f;
+    if (i < a.group) v[c] = gated_norm_in<T>(a, r, g0 + i, inv_den, &sg[c]);
+    ss = fmaf(v[c], v[c], ss);
+  }
   ss = block_sum(ss, red);
-  const float inv = 1.f / sqrtf(ss / (float)N + eps);
-  const T* g = gate ? gate + r * gate_stride : nullptr;
-  for (int i = threadIdx.x; i < N; i += blockDim.x) {
-    const float z = g ? to_f32(g[i]) : 0.f;
-    const float sg = g ? (silu ? z : 1.f) / (1.f + expf(-z)) : 1.f;
-    out[r * N + i] = from_f32<T>(orow[i] * inv * w[i] * sg);
+  const float inv = 1.f / sqrtf(ss / (float)a.group + a.eps);
+#pragma unroll
+  for (int c = 0; c < kGatedPerThread; ++c) {
+    const int i = threadIdx.x + c * blockDim.x;
+    if (i < a.group) ((T*)a.out)[r * a.N + g0 + i] = from_f32<T>(v[c] * inv * w[i] * sg[c]);
   }
 }
 
-// The same with the norm over every group of `group` neighbouring columns by itself (a head's
-// values) and a weight of `group` numbers that all groups share: one wave per (row, group).
+// The same for groups of few columns (a head's values): one wave per (row, group), four groups
+// to a block.
+constexpr int kGatedWaveMax = 512;
 template <typename T>
-__global__ __launch_bounds__(64) void gated_group_rmsnorm_kernel(
-    const float* __restrict__ o, const T* __restrict__ gate, int gate_stride,
-    const float* __restrict__ w, T* __restrict__ out, int N, int group, float eps, int silu) {
+__global__ __launch_bounds__(256) void gated_group_rmsnorm_kernel(GatedNormArgs a) {
   const int64_t r = blockIdx.x;
-  const int g0 = blockIdx.y * group, lane = threadIdx.x;
-  const float* orow = o + r * N + g0;
+  const int g = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int g0 = g * a.group;
+  if (g0 >= a.N) return;
+  const float inv_den = a.den ? 1.f / a.den[r * (a.N / a.group) + g] : 1.f;
+  const float* w = a.w + (a.w_n == a.N ? g0 : 0);
+  constexpr int PER = kGatedWaveMax / 64;
+  float v[PER], sg[PER];
   float ss = 0.f;
-  for (int i = lane; i < group; i += 64) ss = fmaf(orow[i], orow[i], ss);
+#pragma unroll
+  for (int c = 0; c < PER; ++c) {
+    const int i = lane + 64 * c;
+    v[c] = sg[c] = 0.f;
+    if (i < a.group) v[c] = gated_norm_in<T>(a, r, g0 + i, inv_den, &sg[c]);
+    ss = fmaf(v[c], v[c], ss);
+  }
   ss = wave_sum(ss);
-  const float inv = 1.f / sqrtf(ss / (float)group + eps);
-  const T* g = gate ? gate + r * gate_stride + g0 : nullptr;
-  for (int i = lane; i < group; i += 64) {
-    const float z = g ? to_f32(g[i]) : 0.f;
-    const float sg = g ? (silu ? z : 1.f) / (1.f + expf(-z)) : 1.f;
-    out[r * N + g0 + i] = from_f32<T>(orow[i] * inv * w[i] * sg);
+  const float inv = 1.f / sqrtf(ss / (float)a.group + a.eps);
+#pragma unroll
+  for (int c = 0; c < PER; ++c) {
+    const int i = lane + 64 * c;
+    if (i < a.group) ((T*)a.out)[r * a.N + g0 + i] = from_f32<T>(v[c] * inv * w[i] * sg[c]);
   }
 }
 
@@ -429,35 +471,30 @@ extern "C" int ninfer_post_norm(const PostNormArgs* args, hipStream_t stream) {
   return 0;
 }
 
-// group 0 (or N): the norm over the whole row with a weight of N numbers; else over every
-// group of `group` columns with a weight of `group` numbers. silu: the gate's factor is
-// g sigmoid(g) instead of sigmoid(g).
-extern "C" int ninfer_gated_rmsnorm(const float* o, const void* gate, int gate_stride,
-                                    const float* w, void* out, int T, int N, float eps, int dtype,
-                                    int group, int silu, hipStream_t stream) {
-  NINFER_REQUIRE(T > 0 && N > 0 && (!gate || gate_stride >= N), "gated_rmsnorm: T=%d N=%d gate stride %d", T,
-                 N, gate_stride);
-  NINFER_REQUIRE(dtype == kF32 || dtype == kBF16, "gated_rmsnorm: unknown dtype %d", dtype);
-  NINFER_REQUIRE(group >= 0 && (group == 0 || N % group == 0),
-                 "gated_rmsnorm: groups of %d columns do not fill rows of %d", group, N);
-  if (group > 0 && group < N) {
-    const dim3 grid(T, N / group);
-    if (dtype == kF32)
-      gated_group_rmsnorm_kernel<float><<<grid, 64, 0, stream>>>(o, (const float*)gate, gate_stride,
-                                                                 w, (float*)out, N, group, eps, silu);
-    else
-      gated_group_rmsnorm_kernel<bf16><<<grid, 64, 0, stream>>>(o, (const bf16*)gate, gate_stride,
-                                                                w, (bf16*)out, N, group, eps, silu);
-    NINFER_LAUNCH_CHECK();
-    return 0;
+// group 0 (or N): the norm over the whole row; else over every group of `group` columns by
+// itself, with a weight of `group` numbers that the groups share or of N.
+extern "C" int ninfer_gated_rmsnorm(const GatedNormArgs* args, hipStream_t stream) {
+  GatedNormArgs a = *args;
+  NINFER_REQUIRE(a.T > 0 && a.N > 0 && (!a.gate || a.gate_stride >= a.N), "gated_rmsnorm: T=%d N=%d gate stride %d", a.T,
+                 a.N, a.gate_stride);
+  NINFER_REQUIRE(a.dtype == kF32 || a.dtype == kBF16, "gated_rmsnorm: unknown dtype %d", a.dtype);
+  if (a.group == 0) a.group = a.N;
+  NINFER_REQUIRE(a.group > 0 && a.N % a.group == 0, "gated_rmsnorm: groups of %d columns do not fill rows of %d",
+                 a.group, a.N);
+  NINFER_REQUIRE(a.w_n == a.N || a.w_n == a.group, "gated_rmsnorm: %d weights for groups of %d columns", a.w_n, a.group);
+  NINFER_REQUIRE(a.group <= 1024 * kGatedPerThread, "gated_rmsnorm: %d columns exceed %d", a.group, 1024 * kGatedPerThread);
+  NINFER_REQUIRE(!a.gate_first || a.gate, "gated_rmsnorm: no gate to apply first");
+  const int groups = a.N / a.group;
+  if (a.group <= kGatedWaveMax && groups > 1) {
+    const dim3 grid(a.T, (groups + 3) / 4);
+    if (a.dtype == kF32) gated_group_rmsnorm_kernel<float><<<grid, 256, 0, stream>>>(a);
+    else gated_group_rmsnorm_kernel<bf16><<<grid, 256, 0, stream>>>(a);
+  } else {
+    const int block = a.group >= 1024 ? 1024 : (a.group + 63) / 64 * 64;
+    const dim3 grid(a.T, groups);
+    if (a.dtype == kF32) gated_rmsnorm_kernel<float><<<grid, block, 0, stream>>>(a);
+    else gated_rmsnorm_kernel<bf16><<<grid, block, 0, stream>>>(a);
   }
-  const int block = N >= 1024 ? 1024 : (N + 63) / 64 * 64;
-  if (dtype == kF32)
-    gated_rmsnorm_kernel<float><<<T, block, 0, stream>>>(o, (const float*)gate, gate_stride, w,
-                                                         (float*)out, N, eps, silu);
-  else
-    gated_rmsnorm_kernel<bf16><<<T, block, 0, stream>>>(o, (const bf16*)gate, gate_stride, w,
-                                                        (bf16*)out, N, eps, silu);
   NINFER_LAUNCH_CHECK();
   return 0;
 }

@@ -83,7 +83,8 @@ class _AttnArgs(ctypes.Structure):
                 ("slopes", ctypes.c_void_p), ("Dv", ctypes.c_int), ("sink", ctypes.c_int),
                 ("kblk", ctypes.c_void_p), ("vblk", ctypes.c_void_p), ("blk_table", ctypes.c_void_p),
                 ("blk_bt_stride", ctypes.c_int), ("blk_page_size", ctypes.c_int),
-                ("block", ctypes.c_int), ("gate", ctypes.c_void_p), ("gate_stride", ctypes.c_int)]
+                ("block", ctypes.c_int), ("gate", ctypes.c_void_p), ("gate_stride", ctypes.c_int),
+                ("sinks", ctypes.c_void_p)]
 
 
 class _QkvWideArgs(ctypes.Structure):
@@ -101,7 +102,7 @@ class _QkvWideArgs(ctypes.Structure):
                 ("interleaved", ctypes.c_int), ("page_size", ctypes.c_int),
                 ("blk_page_size", ctypes.c_int), ("block", ctypes.c_int), ("dtype", ctypes.c_int),
                 ("eps", ctypes.c_float), ("magnitude", ctypes.c_float), ("all_single", ctypes.c_int),
-                ("force_plain", ctypes.c_int)]
+                ("force_plain", ctypes.c_int), ("unit_heads", ctypes.c_int)]
 
 
 class _PostNormArgs(ctypes.Structure):
@@ -110,6 +111,45 @@ class _PostNormArgs(ctypes.Structure):
                 ("gain", ctypes.c_void_p), ("out", ctypes.c_void_p), ("T", ctypes.c_int),
                 ("H", ctypes.c_int), ("k", ctypes.c_int), ("dtype", ctypes.c_int),
                 ("alpha", ctypes.c_float), ("eps", ctypes.c_float), ("factor", ctypes.c_float)]
+
+
+class _GatedNormArgs(ctypes.Structure):
+    _fields_ = [("o", ctypes.c_void_p), ("gate", ctypes.c_void_p), ("w", ctypes.c_void_p),
+                ("den", ctypes.c_void_p), ("out", ctypes.c_void_p), ("gate_stride", ctypes.c_int),
+                ("T", ctypes.c_int), ("N", ctypes.c_int), ("group", ctypes.c_int), ("w_n", ctypes.c_int),
+                ("silu", ctypes.c_int), ("gate_first", ctypes.c_int), ("dtype", ctypes.c_int),
+                ("eps", ctypes.c_float)]
+
+
+class _StreamNormArgs(ctypes.Structure):
+    _fields_ = [("x", ctypes.c_void_p), ("y1", ctypes.c_void_p), ("y2", ctypes.c_void_p),
+                ("bias", ctypes.c_void_p), ("gain1", ctypes.c_void_p), ("gain", ctypes.c_void_p),
+                ("out", ctypes.c_void_p), ("rows", ctypes.c_void_p), ("n_rows", ctypes.c_int),
+                ("H", ctypes.c_int), ("dtype", ctypes.c_int), ("f1", ctypes.c_float),
+                ("f2", ctypes.c_float), ("eps1", ctypes.c_float), ("eps", ctypes.c_float)]
+
+
+class _ConvSiluArgs(ctypes.Structure):
+    _fields_ = [("u", ctypes.c_void_p), ("w", ctypes.c_void_p), ("b", ctypes.c_void_p),
+                ("state", ctypes.c_void_p), ("out", ctypes.c_void_p), ("row_seq", ctypes.c_void_p),
+                ("seq_row_start", ctypes.c_void_p), ("seq_slots", ctypes.c_void_p),
+                ("state_stride", ctypes.c_int64), ("stride", ctypes.c_int), ("T", ctypes.c_int),
+                ("S", ctypes.c_int), ("C", ctypes.c_int), ("taps", ctypes.c_int),
+                ("all_single", ctypes.c_int), ("dtype", ctypes.c_int)]
+
+
+class _ScanArgs(ctypes.Structure):
+    _fields_ = [("rows", ctypes.c_void_p), ("z", ctypes.c_void_p), ("z_bias", ctypes.c_void_p),
+                ("rate", ctypes.c_void_p), ("skip", ctypes.c_void_p), ("state", ctypes.c_void_p),
+                ("out", ctypes.c_void_p), ("den", ctypes.c_void_p), ("work", ctypes.c_void_p),
+                ("seq_row_start", ctypes.c_void_p), ("seq_slots", ctypes.c_void_p),
+                ("state_stride", ctypes.c_int64), ("gate", ctypes.c_void_p), ("norm_w", ctypes.c_void_p),
+                ("normed", ctypes.c_void_p), ("gate_stride", ctypes.c_int), ("stride", ctypes.c_int),
+                ("q_off", ctypes.c_int), ("k_off", ctypes.c_int), ("v_off", ctypes.c_int),
+                ("H", ctypes.c_int), ("G", ctypes.c_int), ("dim", ctypes.c_int), ("vdim", ctypes.c_int),
+                ("T", ctypes.c_int), ("S", ctypes.c_int), ("first_seq", ctypes.c_int),
+                ("form", ctypes.c_int), ("dtype", ctypes.c_int), ("cap", ctypes.c_float),
+                ("q_scale", ctypes.c_float), ("eps", ctypes.c_float)]
 
 
 class _QkvConvArgs(ctypes.Structure):
@@ -303,6 +343,7 @@ class HipOps:
         self.lib.ninfer_sample_few_places.restype = ctypes.c_longlong
         self.lib.ninfer_latent_attention_workspace_floats.restype = ctypes.c_longlong
         self.lib.ninfer_gla_segment_floats.restype = ctypes.c_longlong
+        self.lib.ninfer_decay_scan_chunk_floats.restype = ctypes.c_longlong
         self.lib.ninfer_diff_attention_workspace_floats.restype = ctypes.c_longlong
         self.lib.ninfer_sigmoid_attention_workspace_floats.restype = ctypes.c_longlong
         self.force_generic = False  # tests: run the plain kernels whatever the shape
@@ -329,6 +370,7 @@ class HipOps:
         self.beside_heavy_bytes = 256 << 20
         self.conv_pieces_always = False     # tests: qkv_conv's kernel of whole pieces at every row count
         self.gla_chunk_min_rows = 8         # the same for gated linear attention
+        self.scan_chunk_min_rows = 8        # ... and for the scans with one decay per head and token
         self.lightning_chunk_min_rows = 8   # a step's longest portion from which lightning attention runs in chunks
         self.library_min_rows = 32  # dense bf16 products with more rows go to the library
         self.rows_kernel_max = 64   # ... unless the kernel for 33 to 64 rows takes them
@@ -926,14 +968,14 @@ class HipOps:
     # ---- attention ------------------------------------------------------------------
     def paged_attention(self, qkv, k_pool, v_pool, block_table, ctx, n_q, n_kv, head_dim,
                         page_size, window, scale, out, plan_only=False, slopes=None, vdim=None,
-                        sink=False, blocks=None, gate=None):
+                        sink=False, blocks=None, gate=None, sinks=None):
         """Attention of the rows' query heads (the first n_q * head_dim columns
         of `qkv`) over their requests' cached keys and values. `slopes` [n_q] (32-bit): head
         h's scores get slopes[h] * (key's position - row's position) added before the softmax
         (a distance-based position bias; negative distances, so a positive slope favours near
         keys). `vdim`: numbers of a value head when they differ from a key head's (`v_pool` and
         `out` are that wide). `sink`: the softmax's denominator has one more term, exp(0), that
-        belongs to no key. `blocks` (a CacheView's `blocks` with pools 'k_block' and 'v_block'
+        belongs to no key; `sinks` [n_q] (32-bit): exp(sinks[h]) in its place. `blocks` (a CacheView's `blocks` with pools 'k_block' and 'v_block'
         [.., n_kv, its page size, head_dim or vdim]): one more key and value for every block of
         `blocks.stride` tokens that lies wholly before the window, in the same softmax. `gate`
         ([T, n_q * vdim] columns of a wider row-major tensor, a view): the output is multiplied
@@ -985,6 +1027,10 @@ class HipOps:
             args.kblk, args.vblk = blocks["k_block"].data_ptr(), blocks["v_block"].data_ptr()
             args.blk_table, args.blk_bt_stride = blocks.block_table.data_ptr(), blocks.block_table.shape[1]
             args.blk_page_size, args.block = blocks.page_size, blocks.stride
+        if sinks is not None:
+            _dev(sinks, "sinks", torch.float32, 1)
+            _need(sink and sinks.shape[0] == n_q, "paged_attention: one sink's score per query head")
+            args.sinks = sinks.data_ptr()
         if gate is not None:
             _need(gate.is_cuda and gate.dtype == qkv.dtype and gate.shape == out.shape
                   and gate.stride(1) == 1, "paged_attention: the gate must be [T, n_q * vdim] columns of rows")
@@ -1013,15 +1059,17 @@ class HipOps:
 
     def qkv_wide(self, u, ctx, q_out, heads, kv_heads, dim, vdim, k_pool, v_pool, block_table,
                  page_size, v_col=None, q_norm=None, k_norm=None, norm_eps=0.0, inv_freq=None,
-                 rot_dim=0, interleaved=False, magnitude=1.0, head_scale=None, blocks=None):
+                 rot_dim=0, interleaved=False, magnitude=1.0, head_scale=None, blocks=None,
+                 unit_heads=False):
         """Projected rows u ([T, C] columns of a wider row-major tensor: heads x dim queries,
         kv_heads x dim keys, and from column `v_col` on kv_heads x vdim values; None: behind the
         keys; the keys' own first column: values that are the keys as projected) on their way to
         attention: queries and keys normed over their whole projections (gains `q_norm`
         [heads * dim], `k_norm` [kv_heads * dim], None: no norm), turned by their position with
         cosine and sine times `magnitude`, query heads times `head_scale` [heads] (32-bit);
-        queries to `q_out`, keys and values to the requests' pages. `blocks` (see
-        `paged_attention`): the means of the cached keys and values of every block of tokens
+        queries to `q_out`, keys and values to the requests' pages. `unit_heads`: every query and
+        key head divided by its root mean square over its dim numbers (eps `norm_eps`), no gains
+        and a magnitude of 1. `blocks` (see `paged_attention`): the means of the cached keys and values of every block of tokens
         that this step completes go to its pools."""
         _need(u.is_cuda and u.dim() == 2 and u.stride(1) == 1 and u.dtype in _DT,
               "qkv_wide: u must be columns of rows")
@@ -1060,7 +1108,7 @@ class HipOps:
         a.rot_dim, a.interleaved, a.page_size = rot_dim, 1 if interleaved else 0, page_size
         a.dtype, a.eps, a.magnitude = _DT[u.dtype], norm_eps, magnitude
         a.all_single = 1 if ctx.max_qlen == 1 else 0
-        a.force_plain = 1 if self.force_generic else 0
+        a.force_plain, a.unit_heads = 1 if self.force_generic else 0, 1 if unit_heads else 0
         self._ok(self.lib.ninfer_qkv_wide(ctypes.byref(a), self._stream()))
 
     def qkv_conv(self, u, w_conv, state, ctx, q_out, heads, kv_heads, dim, vdim, k_pool, v_pool,
@@ -1220,11 +1268,14 @@ class HipOps:
         a.T, a.H, a.dtype, a.alpha, a.eps = t, h, _DT[first.dtype], float(alpha), float(eps)
         self._ok(self.lib.ninfer_post_norm(ctypes.byref(a), self._stream()))
 
-    def gated_rmsnorm(self, o, gate, weight, eps, out, group=0, gate_act="sigmoid"):
+    def gated_rmsnorm(self, o, gate, weight, eps, out, group=0, gate_act="sigmoid", gate_first=False,
+                      den=None):
         """out = o rsqrt(mean(o^2) + eps) weight sigmoid(gate), the mean over the whole row, or
         with `group` over every group of so many neighbouring columns by itself (`weight` then
-        has `group` numbers, shared by the groups). `gate_act` 'silu': gate sigmoid(gate) in
-        place of sigmoid(gate). o: [T, N] 32-bit; gate: [T, N] columns of a wider row-major
+        has `group` numbers, shared by the groups, or one per column of the row). `gate_act`
+        'silu': gate sigmoid(gate) in place of sigmoid(gate). `gate_first`: o is multiplied by the
+        gate's factor before the norm, not after. `den` [T, groups] (32-bit): o is divided by its
+        group's number first. o: [T, N] 32-bit; gate: [T, N] columns of a wider row-major
         tensor (a view), or None for no gate (factor 1)."""
         _dev(o, "o", torch.float32, 2)
         _dev(weight, "weight", torch.float32, 1)
@@ -1232,16 +1283,207 @@ class HipOps:
         t, n = o.shape
         _need(gate_act in ("sigmoid", "silu"), f"gated_rmsnorm: gate activation {gate_act!r}")
         _need(group >= 0 and (group == 0 or n % group == 0), "gated_rmsnorm: groups do not fill the rows")
-        _need(out.shape == (t, n) and weight.shape[0] == (group or n) and out.dtype in _DT,
+        _need(out.shape == (t, n) and weight.shape[0] in (group or n, n) and out.dtype in _DT,
               "gated_rmsnorm: shapes")
         _need(gate is None or (gate.is_cuda and gate.dtype == out.dtype and gate.shape == (t, n)
               and gate.stride(1) == 1), "gated_rmsnorm: the gate must be [T, N] columns of rows")
-        self._ok(self.lib.ninfer_gated_rmsnorm(
-            ctypes.c_void_p(o.data_ptr()), ctypes.c_void_p(_ptr(gate)),
-            0 if gate is None else gate.stride(0) if t > 1 else max(n, gate.stride(0)),
-            ctypes.c_void_p(weight.data_ptr()), ctypes.c_void_p(out.data_ptr()), t, n,
-            ctypes.c_float(eps), _DT[out.dtype], int(group), 1 if gate_act == "silu" else 0,
-            self._stream()))
+        a = _GatedNormArgs()
+        a.o, a.gate, a.w, a.out = o.data_ptr(), _ptr(gate), weight.data_ptr(), out.data_ptr()
+        if den is not None:
+            _dev(den, "den", torch.float32, 2)
+            _need(den.shape == (t, n // (group or n)), "gated_rmsnorm: one divisor per row and group")
+            a.den = den.data_ptr()
+        a.gate_stride = 0 if gate is None else gate.stride(0) if t > 1 else max(n, gate.stride(0))
+        a.T, a.N, a.group, a.w_n, a.silu = t, n, int(group), weight.shape[0], 1 if gate_act == "silu" else 0
+        a.gate_first, a.dtype, a.eps = 1 if gate_first else 0, _DT[out.dtype], eps
+        self._ok(self.lib.ninfer_gated_rmsnorm(ctypes.byref(a), self._stream()))
+
+    def stream_norm(self, residual, pending=None, gain=None, eps=0.0, out=None, rows=None):
+        """residual += what `pending` stands for (rows [T, H]; an object with y, gain and eps: rows
+        normed by themselves; an object with a, factor_a, b, factor_b and bias: a weighted sum of
+        rows and a bias; None: nothing), all in 32-bit; then, when `out` is given, out =
+        residual rsqrt(mean(residual^2) + eps) gain, or the residual itself where `gain` is None.
+        `rows`: only those rows are formed, and the residual is left as it is."""
+        _dev(residual, "residual", torch.float32, 2)
+        t, h = residual.shape
+        a = _StreamNormArgs()
+        a.f1 = 1.0
+        dtype = out.dtype if out is not None else None
+        normed = hasattr(pending, "y")
+        y1 = pending.y if normed else getattr(pending, "a", pending)
+        y2 = getattr(pending, "b", None) if not normed else None
+        for v in (y1, y2):
+            if v is not None:
+                dtype = dtype or v.dtype
+                _dev(v, "rows", dtype, 2)
+                _need(v.shape == (t, h), "stream_norm: the rows do not fit the residual")
+        if normed:
+            _dev(pending.gain, "gain", torch.float32, 1)
+            _need(pending.gain.shape[0] == h, "stream_norm: one gain per column")
+            a.gain1, a.eps1 = pending.gain.data_ptr(), pending.eps
+        elif hasattr(pending, "factor_a"):
+            a.f1, a.f2 = pending.factor_a, pending.factor_b
+            if pending.bias is not None:
+                _dev(pending.bias, "bias", torch.float32, 1)
+                _need(pending.bias.shape[0] == h, "stream_norm: one bias per column")
+                a.bias = pending.bias.data_ptr()
+        _need(dtype in _DT, "stream_norm: rows' dtype")
+        n = t
+        if rows is not None:
+            _dev(rows, "rows", torch.int32, 1)
+            _need(out is not None, "stream_norm: selected rows need an output")
+            n = rows.shape[0]
+            a.rows = rows.data_ptr()
+        if out is not None:
+            _dev(out, "out", dtype, 2)
+            _need(out.shape == (n, h), "stream_norm: out has the wrong shape")
+            a.out = out.data_ptr()
+        if gain is not None:
+            _dev(gain, "gain", torch.float32, 1)
+            _need(gain.shape[0] == h, "stream_norm: one gain per column")
+            a.gain = gain.data_ptr()
+        a.x, a.y1, a.y2 = residual.data_ptr(), _ptr(y1), _ptr(y2)
+        a.n_rows, a.H, a.dtype, a.eps = n, h, _DT[dtype], eps
+        self._ok(self.lib.ninfer_stream_norm(ctypes.byref(a), self._stream()))
+
+    def token_gate(self, z, table, tokens, column0, out):
+        """out[t] = gelu(z[t]) table[tokens[t], column0 : column0 + d], the tanh form of gelu;
+        z, out: [T, d], table: [vocab, width] of the same dtype."""
+        _dev(z, "z", dims=2)
+        _dev(table, "table", z.dtype, 2)
+        _dev(out, "out", z.dtype, 2)
+        _dev(tokens, "tokens", torch.int32, 1)
+        t, d = z.shape
+        _need(z.dtype in _DT and out.shape == (t, d) and tokens.shape[0] == t, "token_gate: shapes")
+        _need(0 <= column0 and column0 + d <= table.shape[1], "token_gate: columns outside the table")
+        self._ok(self.lib.ninfer_token_gate(
+            ctypes.c_void_p(z.data_ptr()), ctypes.c_void_p(table.data_ptr()), ctypes.c_void_p(tokens.data_ptr()),
+            ctypes.c_void_p(out.data_ptr()), t, d, table.shape[1], int(column0), _DT[z.dtype], self._stream()))
+
+    # ---- linear attention with one decay per head and token ---------------------------
+    @staticmethod
+    def _columns(x, width, who):
+        """The row stride of [T, >= width] columns of a row-major tensor."""
+        _need(x.is_cuda and x.dim() == 2 and x.stride(1) == 1 and x.dtype in _DT and x.shape[1] >= width,
+              f"{who} must be columns of rows")
+        return x.stride(0) if x.shape[0] > 1 else max(x.shape[1], x.stride(0))
+
+    @staticmethod
+    def _state_rows(state, floats, who):
+        _need(state is not None and state.is_cuda and state.dtype == torch.float32 and state.dim() == 2
+              and state.stride(1) == 1 and state.shape[1] >= floats,
+              f"{who}: the state must be 32-bit rows of at least {floats} numbers")
+
+    def conv_silu(self, u, w, bias, state, ctx, out):
+        """out = silu(bias + sum_j w[j] u_(t - taps + 1 + j)) per channel over the rows of each
+        request: u [T, C] columns of a wider row-major tensor, w [taps, C], bias [C] (32-bit). The
+        taps - 1 inputs before a step's first row come from `state` ([slots, >= (taps - 1) C] 32-bit
+        view), which is moved on."""
+        _dev(w, "w", torch.float32, 2)
+        _dev(bias, "bias", torch.float32, 1)
+        _dev(out, "out", u.dtype, 2)
+        taps, c = w.shape
+        a = _ConvSiluArgs()
+        a.stride = self._columns(u, c, "conv_silu: u")
+        _need(u.shape == (ctx.T, c) and out.shape == (ctx.T, c) and bias.shape[0] == c, "conv_silu: shapes")
+        if taps > 1:
+            self._state_rows(state, (taps - 1) * c, "conv_silu")
+            a.state, a.state_stride = state.data_ptr(), state.stride(0)
+        a.u, a.w, a.b, a.out = u.data_ptr(), w.data_ptr(), bias.data_ptr(), out.data_ptr()
+        a.row_seq, a.seq_row_start, a.seq_slots = ctx.row_seq.data_ptr(), ctx.seq_row_start.data_ptr(), ctx.seq_slots.data_ptr()
+        a.T, a.S, a.C, a.taps, a.all_single, a.dtype = ctx.T, ctx.S, c, taps, 1 if ctx.max_qlen == 1 else 0, _DT[u.dtype]
+        self._ok(self.lib.ninfer_conv_silu(ctypes.byref(a), self._stream()))
+
+    def _scan_args(self, rows, q_off, k_off, v_off, z, z_bias, heads, groups, dim, vdim, state, ctx, form):
+        exp = form == 1
+        a = _ScanArgs()
+        a.stride = self._columns(rows, 0, "decay scan: rows")
+        t = ctx.T
+        for off, n in ((q_off, groups * dim), (k_off, groups * dim), (v_off, heads * vdim)):
+            _need(0 <= off and off + n <= rows.shape[1], "decay scan: columns outside the rows")
+        _dev(z, "z", torch.float32, 2)
+        _dev(z_bias, "z_bias", torch.float32, 1)
+        n_z = heads * (2 if exp else 1)
+        _need(rows.shape[0] == t and z.shape == (t, n_z) and z_bias.shape[0] == n_z, "decay scan: shapes")
+        self._state_rows(state, heads * dim * vdim + (heads * (dim + 1) if exp else 0), "decay scan")
+        a.rows, a.z, a.z_bias, a.state = rows.data_ptr(), z.data_ptr(), z_bias.data_ptr(), state.data_ptr()
+        a.state_stride = state.stride(0)
+        a.seq_row_start, a.seq_slots = ctx.seq_row_start.data_ptr(), ctx.seq_slots.data_ptr()
+        a.q_off, a.k_off, a.v_off = q_off, k_off, v_off
+        a.H, a.G, a.dim, a.vdim, a.T, a.S, a.form, a.dtype = heads, groups, dim, vdim, t, ctx.S, form, _DT[rows.dtype]
+        a.cap = a.q_scale = 1.0
+        return a
+
+    def _scan_run(self, a, ctx, device):
+        """Runs a decay scan: how many of the step's first rows the kernel of single rows has
+        taken (and, in the exponential form, finished). The 32-bit path walks every request row by
+        row, so that its logits do not depend on the cut to the bit; bfloat16 prompt portions run
+        in chunks on the matrix cores where the sizes fit."""
+        single = ctx.S if ctx.max_qlen == 1 else int(getattr(ctx, "single_rows", 0))
+        if a.dtype != _DT[torch.bfloat16] or self.force_generic:
+            single = 0
+        if single:
+            rc = self.lib.ninfer_decay_scan_single(ctypes.byref(a), single, self._stream())
+            if rc < 0:
+                self._ok(rc)
+            if rc == 1:
+                single = 0
+            elif single == ctx.S:
+                return single
+        a.first_seq = single
+        if ctx.max_qlen >= self.scan_chunk_min_rows and not self.force_generic:
+            floats = int(self.lib.ninfer_decay_scan_chunk_floats(ctypes.byref(a)))
+            if floats:
+                work = torch.empty(floats, dtype=torch.float32, device=device)
+                a.work = work.data_ptr()
+                self._ok(self.lib.ninfer_decay_scan_chunks(ctypes.byref(a), self._stream()))
+                return single
+        work = torch.empty(a.T * a.H * 3, dtype=torch.float32, device=device)
+        a.work = work.data_ptr()
+        self._ok(self.lib.ninfer_decay_scan(ctypes.byref(a), self._stream()))
+        return single
+
+    def state_space(self, xbc, heads, vdim, dim, groups, dt, dt_bias, rate, skip, state, ctx, out):
+        """A state-space recurrence per head over the rows of each request: with dt = softplus(dt +
+        dt_bias), S <- exp(-rate dt) S + dt B x^T, out = S^T C + skip x. xbc: [T, heads * vdim + 2
+        groups * dim] rows (x, then B, then C; head h reads group h // (heads / groups)); dt
+        [T, heads] 32-bit; dt_bias, rate, skip [heads] (32-bit). `state` ([slots, >= heads * dim *
+        vdim] 32-bit view) holds every request's S between steps. out: [T, heads * vdim] 32-bit."""
+        inner = heads * vdim
+        a = self._scan_args(xbc, inner + groups * dim, inner, 0, dt, dt_bias, heads, groups, dim, vdim, state, ctx, 0)
+        for g, name in ((rate, "rate"), (skip, "skip")):
+            _dev(g, name, torch.float32, 1)
+            _need(g.shape[0] == heads, f"state_space: one {name} per head")
+        _dev(out, "out", torch.float32, 2)
+        _need(out.shape == (ctx.T, inner), "state_space: out has the wrong shape")
+        a.rate, a.skip, a.out = rate.data_ptr(), skip.data_ptr(), out.data_ptr()
+        self._scan_run(a, ctx, xbc.device)
+
+    def matrix_memory(self, u, q_off, k_off, v_off, z, z_bias, heads, dim, vdim, cap, q_scale, state, ctx,
+                      gate, norm_w, eps, out):
+        """A matrix memory with exponential gates per head over the rows of each request (z
+        [T, 2 heads] 32-bit: the write gates' logits, then the forget gates'; z_bias [2 heads]):
+        with c(x) = cap tanh(x / cap), i = c(z_i + b_i), f = log_sigmoid(c(z_f + b_f)) and m' =
+        max(f + m, i), S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone, o = S^T q
+        / (max(|n . q|, exp(-m')) + 1e-6), q times `q_scale`; then out = rms(o) per head (eps) *
+        norm_w [heads * vdim] * sigmoid(gate) in u's dtype. u: columns of rows; `state` ([slots, >=
+        heads * (dim * vdim + dim + 1)] 32-bit view): S, n and m between steps."""
+        a = self._scan_args(u, q_off, k_off, v_off, z, z_bias, heads, heads, dim, vdim, state, ctx, 1)
+        t, n = ctx.T, heads * vdim
+        _dev(norm_w, "norm_w", torch.float32, 1)
+        _dev(out, "out", u.dtype, 2)
+        _need(norm_w.shape[0] == n and out.shape == (t, n) and gate.dtype == u.dtype and gate.shape == (t, n),
+              "matrix_memory: shapes")
+        a.gate, a.gate_stride = gate.data_ptr(), self._columns(gate, n, "matrix_memory: the gate")
+        a.norm_w, a.normed, a.eps, a.cap, a.q_scale = norm_w.data_ptr(), out.data_ptr(), eps, cap, q_scale
+        o = den = None
+        if ctx.max_qlen > 1 or u.dtype != torch.bfloat16 or self.force_generic or vdim > 1024:
+            o = torch.empty((t, n), dtype=torch.float32, device=u.device)
+            den = torch.empty((t, heads), dtype=torch.float32, device=u.device)
+            a.out, a.den = o.data_ptr(), den.data_ptr()
+        done = self._scan_run(a, ctx, u.device)
+        if done < ctx.S:   # (single rows come first: rows 0 .. done - 1 are finished)
+            self.gated_rmsnorm(o[done:], gate[done:], norm_w, eps, out[done:], group=vdim, den=den[done:])
 
     def lightning_attention(self, qkv, q_off, k_off, v_off, heads, dim, vdim, decay, state, ctx,
                             out):

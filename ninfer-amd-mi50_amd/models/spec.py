@@ -31,12 +31,15 @@ class ModelSpec:
     def __init__(self, embedding: TokenEmbedding, blocks: List[Block], final_norm: Norm,
                  head: LMHead, plan: Optional[List[LayerCall]] = None,
                  vocab_size: Optional[int] = None, eos_token_ids=(),
-                 joins: Optional[List[Part]] = None):
+                 joins: Optional[List[Part]] = None, shared: Optional[List[Part]] = None):
         self.embedding = embedding
         self.blocks = blocks
         # parts that plan entries name in `before`: forward(ctx, residual, pending, first)
         # -> the new residual, `first` being the embedding's output
         self.joins: List[Part] = list(joins or [])
+        # parts that several blocks hold and read (a table with a piece for every layer): bound
+        # once, here, and not by the blocks
+        self.shared: List[Part] = list(shared or [])
         self.final_norm = final_norm
         self.head = head
         self.vocab_size = vocab_size if vocab_size is not None else head.vocab
@@ -65,7 +68,7 @@ class ModelSpec:
         self.plan = list(plan)
 
     def parts(self) -> List[Part]:
-        return [self.embedding, *self.joins, *self.blocks, self.final_norm, self.head]
+        return [self.embedding, *self.shared, *self.joins, *self.blocks, self.final_norm, self.head]
 
     def max_positions(self) -> Optional[int]:
         """The longest request the parts allow (None: no part limits it)."""

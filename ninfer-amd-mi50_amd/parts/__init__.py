@@ -1,7 +1,7 @@
 from .attention import Attention
 from .base import (Block, CacheNeed, CacheView, CallInfo, FeedForward, Mixer, Norm, Part,
-                   NormedSum, PendingRows, PoolSpec, PositionEncoding, ReadyRows, StepContext,
-                   WeightBinder, plain_rows, settle)
+                   NormedRows, NormedSum, PendingRows, PoolSpec, PositionEncoding, ReadyRows, StepContext,
+                   SumRows, WeightBinder, plain_rows, settle)
 from .block import OutputNormBlock, ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock
 from .diff_attention import DifferentialAttention
 from .embedding import LMHead, TokenEmbedding
@@ -9,6 +9,7 @@ from .forget_gate import ForgetGateAttention
 from .gla import GatedLinearAttention
 from .latent_attention import LatentAttention
 from .lightning import LightningAttention
+from .matrix_memory import MatrixMemory
 from .mlp import MLP, SwiGLU
 from .moe import RoutedExperts, Routing, SoftmaxTopKRouter, SparseMoE, TopKRouter
 from .norm import LayerNorm, OutputLayerNorm, OutputRMSNorm, ResidualRMSNorm, RMSNorm
@@ -17,6 +18,8 @@ from .reentry import StreamReentry
 from .short_conv import ShortConv
 from .side_by_side import SideBySide
 from .sigmoid_attention import SigmoidAttention
+from .state_space import StateSpace
+from .token_side import TokenSide, TokenSideTable
 
 __all__ = ["Attention", "Block", "CacheNeed", "CacheView", "CallInfo", "FeedForward", "Mixer",
            "Norm", "Part", "PendingRows", "PoolSpec", "settle", "PositionEncoding", "StepContext", "WeightBinder", "PreNormBlock",
@@ -26,4 +29,4 @@ __all__ = ["Attention", "Block", "CacheNeed", "CacheView", "CallInfo", "FeedForw
            "DifferentialAttention", "MLP", "StreamReentry", "GatedLinearAttention",
            "SigmoidAttention", "SandwichBlock", "LayerNorm", "OutputLayerNorm", "NormedSum",
            "ReadyRows", "plain_rows", "PostNormBlock", "ForgetGateAttention", "ResidualRMSNorm",
-           "SideBySide"]
+           "SideBySide", "SumRows", "NormedRows", "MatrixMemory", "StateSpace", "TokenSide", "TokenSideTable"]

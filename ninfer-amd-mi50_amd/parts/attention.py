@@ -21,7 +21,9 @@ product): queries and keys normed over their whole projections (`qk_norm="projec
 values that are the keys as projected (`values="keys"`), one more key and value per block of
 tokens before the window, the means of the block's (`pool`), a factor per head on the scores
 (`head_temp`), a position encoding that scales what it turns (its `magnitude`), and an output
-gate computed from the layer's input (`output_gate`). Such a layer reads its input through one
+gate computed from the layer's input (`output_gate`), query and key heads brought to a root mean
+square of 1 after they turn, without a weight (`qk_norm="unit"`), and a sink whose score is a
+learned number per head (`sink="learned"`). Such a layer reads its input through one
 product (`input_width`), which layers side by side may share.
 """
 from __future__ import annotations
@@ -42,7 +44,7 @@ class Attention(Mixer):
                  window: Optional[int] = None, scale: Optional[float] = None,
                  score_slopes: Optional[Sequence[float]] = None,
                  qk_norm_eps: Optional[float] = None, page_size: Optional[int] = None,
-                 vdim: Optional[int] = None, conv_taps: int = 0, sink: bool = False,
+                 vdim: Optional[int] = None, conv_taps: int = 0, sink=False,
                  own_kv: bool = True, names=None, cache_window="same", qk_norm: str = "head",
                  values: str = "own", pool: Optional[int] = None, head_temp: bool = False,
                  output_gate: bool = False):
@@ -68,19 +70,28 @@ class Attention(Mixer):
         of `pool` tokens that lies wholly before the window, the mean of the block's cached keys
         and values, in the same softmax. `head_temp`: a factor per head on the scores (tensor
         `names['temp']` [heads]). `output_gate`: the heads' outputs are multiplied by
-        sigmoid(W_g x), element by element (`names['g']` [heads * vdim, hidden])."""
-        if qk_norm not in ("head", "projection") or values not in ("own", "keys"):
+        sigmoid(W_g x), element by element (`names['g']` [heads * vdim, hidden]). `qk_norm` 'unit':
+        every query and key head is divided by its root mean square after it has turned (eps:
+        `qk_norm_eps`), no weight. `sink` 'learned': the sink's score is not 0 but a number per
+        head (`names['sink']` [heads]), which the scale leaves alone."""
+        if qk_norm not in ("head", "projection", "unit") or values not in ("own", "keys"):
             raise ValueError(f"qk_norm {qk_norm!r} or values {values!r} is not known")
         self.qk_norm, self.values, self.pool = qk_norm, values, pool
         self.head_temp, self.output_gate = bool(head_temp), bool(output_gate)
         self.wide = qk_norm == "projection" or values == "keys" or pool is not None or head_temp \
-            or output_gate or getattr(position, "magnitude", 1.0) != 1.0
+            or output_gate or getattr(position, "magnitude", 1.0) != 1.0 or qk_norm == "unit" \
+            or sink == "learned"
+        if sink not in (False, True, "learned"):
+            raise ValueError(f"sink {sink!r} is not known")
+        if qk_norm == "unit" and (qk_norm_eps is None or getattr(position, "magnitude", 1.0) != 1.0):
+            raise ValueError("heads of unit root mean square need the norm's eps, and a rotation that "
+                             "keeps their size")
         if self.wide:
             if qkv_bias or conv_taps or not own_kv:
                 raise ValueError("biases, a convolution or another layer's cache beside norms over "
                                  "whole projections, values from keys, blocks, head factors, a scaled "
-                                 "rotation or an output gate are not built")
-            if qk_norm_eps is not None and qk_norm != "projection":
+                                 "rotation, an output gate, unit heads or a learned sink are not built")
+            if qk_norm_eps is not None and qk_norm == "head":
                 raise ValueError("a norm per head beside these is not built")
             if values == "keys" and vdim not in (None, head_dim):
                 raise ValueError(f"values that are keys have {head_dim} numbers, not {vdim}")
@@ -94,11 +105,14 @@ class Attention(Mixer):
         self.cache_window = window if cache_window == "same" else cache_window
         self.vdim = head_dim if vdim is None else int(vdim)
         self.conv_taps, self.sink, self.own_kv = int(conv_taps), bool(sink), bool(own_kv)
+        self.learned_sink = sink == "learned"
+        self.sinks: Optional[torch.Tensor] = None      # a learned sink's scores [heads]
         if self.conv_taps < 0:
             raise ValueError(f"conv_taps ({conv_taps}) must be >= 0")
         self.names = dict({"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight",
                            "o": "o_proj.weight", "q_norm": "q_norm.weight",
-                           "k_norm": "k_norm.weight", "conv": ".conv", "temp": "temp", "g": "g_proj.weight"},
+                           "k_norm": "k_norm.weight", "conv": ".conv", "temp": "temp", "g": "g_proj.weight",
+                           "sink": "sink"},
                           **(names or {}))
         # the fused product + rotation + cache write serves the plain layer; everything else
         # (values of their own size, a convolution, another layer's cache) goes the general way
@@ -177,7 +191,9 @@ class Attention(Mixer):
             specs[p + "q_proj.bias"] = TensorSpec((self.heads * d,), "bias")
             specs[p + "k_proj.bias"] = TensorSpec((self.kv_heads * d,), "bias")
             specs[p + "v_proj.bias"] = TensorSpec((self.kv_heads * d,), "bias")
-        if self.qk_norm_eps is not None:
+        if self.learned_sink:
+            specs[p + n["sink"]] = TensorSpec((self.heads,), "bias")
+        if self.qk_norm_eps is not None and self.qk_norm != "unit":
             nq, nk = (self.heads, self.kv_heads) if self.qk_norm == "projection" else (1, 1)
             specs[p + n["q_norm"]] = TensorSpec((nq * d,), "gain")
             if self.own_kv:
@@ -195,9 +211,11 @@ class Attention(Mixer):
         nq, nk = self.heads * d, self.kv_heads * d
         if self.score_slopes is not None:
             self.slopes = torch.tensor(self.score_slopes, dtype=torch.float32, device=w.device)
-        if self.qk_norm_eps is not None:
+        if self.qk_norm_eps is not None and self.qk_norm != "unit":
             self.q_norm = w.float32(p + n["q_norm"])
             self.k_norm = w.float32(p + n["k_norm"]) if self.own_kv else None
+        if self.learned_sink:
+            self.sinks = w.float32(p + n["sink"])
         if self.wide:
             if self.head_temp:
                 self.temp = w.float32(p + n["temp"])
@@ -240,7 +258,7 @@ class Attention(Mixer):
                 w.matrix_into(p + n[key], rows[at:at + width])
                 at += width
 
-    def forward_projected(self, ctx: StepContext, u, call: CallInfo):
+    def mix_projected(self, ctx: StepContext, u, call: CallInfo, extra=None):
         ops, cache, d = ctx.ops, call.cache, self.head_dim
         if not call.writes_cache:
             raise ValueError(f"{self.prefix}: this layer writes a cache of its own")
@@ -252,14 +270,17 @@ class Attention(Mixer):
                      inv_freq=self.position.table(), rot_dim=self.position.rot_dim,
                      interleaved=self.position.pairing == "interleaved",
                      magnitude=getattr(self.position, "magnitude", 1.0), head_scale=self.temp,
-                     blocks=cache.blocks)
+                     blocks=cache.blocks, unit_heads=self.qk_norm == "unit")
         attn = ctx.empty((ctx.T, self.heads * self.vdim))
         ops.paged_attention(q, cache["k"], cache["v"], cache.block_table, ctx, self.heads,
                             self.kv_heads, d, cache.page_size, self.window, self.scale, attn,
                             slopes=self.slopes, vdim=self.vdim, sink=self.sink, blocks=cache.blocks,
-                            gate=u[:, self.qkv_width:] if self.output_gate else None)
+                            gate=u[:, self.qkv_width:] if self.output_gate else None, sinks=self.sinks)
+        return attn
+
+    def output(self, ctx: StepContext, rows):
         out = ctx.empty((ctx.T, self.hidden))
-        ops.linear(attn, self.w_o, out)
+        ctx.ops.linear(rows, self.w_o, out)
         return out
 
     def _forward_general(self, ctx: StepContext, x, call: CallInfo):

@@ -192,10 +192,44 @@ class ReadyRows:
     rows: torch.Tensor
 
 
+@dataclass
+class SumRows:
+    """Rows that a part leaves to be added to the residual by whoever comes next, in 32-bit:
+    factor_a a + factor_b b + bias, from rows a and b [T, hidden] (b may be None) and a bias
+    [hidden] (32-bit, or None)."""
+    a: torch.Tensor
+    factor_a: float = 1.0
+    b: Optional[torch.Tensor] = None
+    factor_b: float = 1.0
+    bias: Optional[torch.Tensor] = None
+
+    def rows(self, ctx: "StepContext") -> torch.Tensor:
+        """The rows themselves, for parts that take only plain ones."""
+        return _formed(ctx, self, self.a)
+
+
+@dataclass
+class NormedRows:
+    """The same for rows that are normed first: y rsqrt(mean(y^2) + eps) gain, gain [hidden]
+    (32-bit)."""
+    y: torch.Tensor
+    gain: torch.Tensor
+    eps: float
+
+    def rows(self, ctx: "StepContext") -> torch.Tensor:
+        return _formed(ctx, self, self.y)
+
+
+def _formed(ctx: "StepContext", pending, like: torch.Tensor) -> torch.Tensor:
+    total = torch.zeros(like.shape, dtype=torch.float32, device=like.device)
+    ctx.ops.stream_norm(total, pending)
+    return total.to(ctx.act_dtype)
+
+
 def plain_rows(ctx: "StepContext", y):
-    """What a part handed on as something that any part takes: a NormedSum becomes rows, a
-    ReadyRows nothing; everything else is handed back unchanged."""
-    if isinstance(y, NormedSum):
+    """What a part handed on as something that any part takes: a NormedSum, a SumRows or a
+    NormedRows becomes rows, a ReadyRows nothing; everything else is handed back unchanged."""
+    if isinstance(y, (NormedSum, SumRows, NormedRows)):
         return y.rows(ctx)
     return None if isinstance(y, ReadyRows) else y
 
@@ -344,10 +378,26 @@ class Mixer(Part):
         """Columns of the one product through which this mixer reads its input, or None when it
         reads it in another way. A mixer that gives a width also has `bind_input(w, rows)`
         (place the product's weights into `rows` [input_width, hidden]) and
-        `forward_projected(ctx, u, call)` (`u`: the product's [T, input_width], columns of a
-        wider row-major tensor), so that mixers which read the same input share one product;
-        its own `bind` then leaves these weights alone once `shares_input` is set."""
+        `mix_projected(ctx, u, call, extra)` (`u`: the product's [T, input_width], columns of a
+        wider row-major tensor; returns what `output` takes), so that mixers which read the same
+        input share one product; its own `bind` then leaves these weights alone once
+        `shares_input` is set."""
         return None
+
+    def input_extra(self, ctx: StepContext, x: torch.Tensor):
+        """Small products of the input that stay beside the shared one (numbers wanted in
+        32-bit): called inside `together()`, handed to `mix_projected` as `extra`."""
+        return None
+
+    def mix_projected(self, ctx: StepContext, u: torch.Tensor, call: CallInfo, extra=None) -> torch.Tensor:
+        raise NotImplementedError
+
+    def output(self, ctx: StepContext, rows: torch.Tensor) -> torch.Tensor:
+        """The output product of what `mix_projected` returned."""
+        raise NotImplementedError
+
+    def forward_projected(self, ctx: StepContext, u: torch.Tensor, call: CallInfo, extra=None) -> torch.Tensor:
+        return self.output(ctx, self.mix_projected(ctx, u, call, extra))
 
     def forward(self, ctx: StepContext, x: torch.Tensor, residual: torch.Tensor,
                 call: CallInfo) -> Optional[torch.Tensor]:

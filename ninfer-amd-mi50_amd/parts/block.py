@@ -19,20 +19,35 @@ from .base import (Block, CallInfo, FeedForward, Mixer, Norm, Part, PendingRows,
 
 
 class PreNormBlock(Block):
-    def __init__(self, mixer_norm: Norm, mixer: Mixer, ff_norm: Norm, feed_forward: FeedForward):
+    """`feed_forward` may be None (a norm given all the same is one whose tensors the checkpoint
+    may carry). `after`: a part the stream passes behind the feed-forward, `forward(ctx, residual,
+    pending)` -> what is to be added to the residual next."""
+
+    def __init__(self, mixer_norm: Norm, mixer: Mixer, ff_norm: Optional[Norm] = None,
+                 feed_forward: Optional[FeedForward] = None, after: Optional[Part] = None):
+        if feed_forward is not None and ff_norm is None:
+            raise ValueError("a feed-forward needs the norm in front of it")
         self.mixer_norm = mixer_norm
         self.mixer = mixer
-        self.ff_norm = ff_norm
+        self.ff_norm = ff_norm if feed_forward is not None else None
+        self.spare_norm = ff_norm if feed_forward is None else None
         self.feed_forward = feed_forward
+        self.after = after
+
+    def unused_tensor_specs(self):
+        return self.spare_norm.all_tensor_specs() if self.spare_norm is not None else {}
 
     def children(self) -> List[Part]:
-        return [self.mixer_norm, self.mixer, self.ff_norm, self.feed_forward]
+        return [p for p in (self.mixer_norm, self.mixer, self.ff_norm, self.feed_forward, self.after)
+                if p is not None]
 
     def forward(self, ctx: StepContext, residual, pending, call: CallInfo):
         a = self.mixer_norm.forward(ctx, residual, pending)
         pending = self.mixer.forward(ctx, a, residual, call)
-        m = self.ff_norm.forward(ctx, residual, pending)
-        return self.feed_forward.forward(ctx, m, residual)
+        if self.feed_forward is not None:
+            m = self.ff_norm.forward(ctx, residual, pending)
+            pending = self.feed_forward.forward(ctx, m, residual)
+        return pending if self.after is None else self.after.forward(ctx, residual, pending)
 
 
 register_part("block", "pre_norm", PreNormBlock)

@@ -68,7 +68,7 @@ class ForgetGateAttention(Mixer):
         if not bool(((self.lower >= 0) & (self.lower <= 1)).all()):
             raise ValueError(f"{p + n[5]}: a forget gate's lower bounds lie between 0 and 1")
 
-    def forward_projected(self, ctx: StepContext, u, call: CallInfo):
+    def mix_projected(self, ctx: StepContext, u, call: CallInfo, extra=None):
         ops = ctx.ops
         qk, v = self.heads * self.dim, self.heads * self.vdim
         o = ctx.empty((ctx.T, v), torch.float32)
@@ -80,8 +80,11 @@ class ForgetGateAttention(Mixer):
                                    forget=(qk, self.f_bias, self.lower))
         normed = ctx.empty((ctx.T, v))
         ops.gated_rmsnorm(o, None, self.norm_w, self.eps, normed, group=self.vdim)
+        return normed
+
+    def output(self, ctx: StepContext, rows):
         out = ctx.empty((ctx.T, self.hidden))
-        ops.linear(normed, self.w_o, out)
+        ctx.ops.linear(rows, self.w_o, out)
         return out
 
     def forward(self, ctx: StepContext, x, residual, call: CallInfo):

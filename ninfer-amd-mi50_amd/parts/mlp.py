@@ -14,23 +14,27 @@ import torch
 
 from ..registry import register_part
 from ..weights.source import TensorSpec
-from .base import FeedForward, StepContext, WeightBinder
+from .base import FeedForward, StepContext, SumRows, WeightBinder
 
 
 class SwiGLU(FeedForward):
     def __init__(self, prefix: str, hidden: int, inner: int, act: str = "silu", bias: bool = False,
                  names=("gate_proj.weight", "up_proj.weight", "down_proj.weight"),
-                 act_limit: float = 0.0, act_alpha: float = 1.0):
+                 act_limit: float = 0.0, act_alpha: float = 1.0,
+                 bias_names=("gate_proj.bias", "up_proj.bias", "down_proj.bias"),
+                 hand_on_bias: bool = False):
         """`names`: what follows the prefix in the names of the gate's, the other half's and the
-        down product's weights. `act` 'clamped_swish': g sigmoid(act_alpha g) (u + 1) with g cut
+        down product's weights; `bias_names`: the same of their biases. `hand_on_bias`: the down
+        product's bias is left to whoever adds the rows to the residual (a `SumRows`). `act` 'clamped_swish': g sigmoid(act_alpha g) (u + 1) with g cut
         at act_limit from above and u to [-act_limit, act_limit]."""
         self.act_limit, self.act_alpha = float(act_limit), float(act_alpha)
         self.prefix = prefix
-        self.names = tuple(names)
+        self.names, self.bias_names = tuple(names), tuple(bias_names)
+        self.hand_on_bias = bool(hand_on_bias and bias)
         self.hidden = hidden
         self.inner = inner
         self.act = act   # the gate's activation: 'silu' | 'gelu_pytorch_tanh' | 'clamped_swish'
-        self.bias = bias   # gate_proj.bias, up_proj.bias [inner] and down_proj.bias [hidden] are read
+        self.bias = bias   # biases of the gate, the other half [inner] and the down product [hidden]
         self.w_gate_up: Optional[torch.Tensor] = None
         self.w_down: Optional[torch.Tensor] = None
         self.b_gate_up: Optional[torch.Tensor] = None
@@ -42,9 +46,8 @@ class SwiGLU(FeedForward):
                  p + self.names[1]: TensorSpec((self.inner, self.hidden)),
                  p + self.names[2]: TensorSpec((self.hidden, self.inner))}
         if self.bias:
-            specs[p + "gate_proj.bias"] = TensorSpec((self.inner,), "bias")
-            specs[p + "up_proj.bias"] = TensorSpec((self.inner,), "bias")
-            specs[p + "down_proj.bias"] = TensorSpec((self.hidden,), "bias")
+            for name, n in zip(self.bias_names, (self.inner, self.inner, self.hidden)):
+                specs[p + name] = TensorSpec((n,), "bias")
         return specs
 
     def bind(self, w: WeightBinder) -> None:
@@ -55,10 +58,11 @@ class SwiGLU(FeedForward):
         w.matrix_into(p + self.names[1], self.w_gate_up[self.inner:])
         self.w_down = w.matrix(p + self.names[2])
         if self.bias:
-            self.b_gate_up = torch.cat([w.float32(p + "gate_proj.bias"), w.float32(p + "up_proj.bias")])
-            w.hold(p + "gate_proj.bias", self.b_gate_up[:self.inner])
-            w.hold(p + "up_proj.bias", self.b_gate_up[self.inner:])
-            self.b_down = w.float32(p + "down_proj.bias")
+            gate, up, down = (p + name for name in self.bias_names)
+            self.b_gate_up = torch.cat([w.float32(gate), w.float32(up)])
+            w.hold(gate, self.b_gate_up[:self.inner])
+            w.hold(up, self.b_gate_up[self.inner:])
+            self.b_down = w.float32(down)
 
     def weight_bytes(self) -> int:
         """What one pass over the two weight matrices reads."""
@@ -75,6 +79,9 @@ class SwiGLU(FeedForward):
 
     def down(self, ctx: StepContext, h: torch.Tensor) -> torch.Tensor:
         out = ctx.empty((h.shape[0], self.hidden))
+        if self.hand_on_bias:
+            ctx.ops.linear(h, self.w_down, out)
+            return SumRows(out, bias=self.b_down)
         ctx.ops.linear(h, self.w_down, out, bias=self.b_down)
         return out
 

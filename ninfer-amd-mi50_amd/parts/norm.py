@@ -13,16 +13,19 @@ import torch
 
 from ..registry import register_part
 from ..weights.source import TensorSpec
-from .base import Norm, Part, PendingRows, StepContext, WeightBinder, plain_rows
+from .base import (NormedRows, Norm, Part, PendingRows, StepContext, SumRows, WeightBinder,
+                   plain_rows)
 
 
 class RMSNorm(Norm):
     def __init__(self, prefix: str, size: int, eps: float, leaf: str = "weight",
-                 single_gain: bool = False, center: bool = False):
+                 single_gain: bool = False, center: bool = False, around_zero: bool = False):
         """`leaf`: what follows the prefix in the gain's name ('' when the prefix is the whole
         name). `single_gain`: the checkpoint holds one number (shape []) for all columns.
-        `center`: the row's mean is taken off first (a layer norm without a bias)."""
+        `center`: the row's mean is taken off first (a layer norm without a bias).
+        `around_zero`: the checkpoint holds w and the gain is 1 + w."""
         self.center = bool(center)
+        self.around_zero = bool(around_zero)
         self.prefix = prefix
         self.size = size
         self.eps = eps
@@ -31,15 +34,21 @@ class RMSNorm(Norm):
         self.gain: Optional[torch.Tensor] = None
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
-        return {self.prefix + self.leaf: TensorSpec(() if self.single_gain else (self.size,), "gain")}
+        return {self.prefix + self.leaf: TensorSpec(() if self.single_gain else (self.size,),
+                                                    "bias" if self.around_zero else "gain")}
 
     def bind(self, w: WeightBinder) -> None:
         self.gain = w.float32(self.prefix + self.leaf)
+        if self.around_zero:   # (read-back by name hands out w itself)
+            self.gain = self.gain + 1.0
         if self.single_gain:   # the kernel reads one gain per column
             self.gain = self.gain.reshape(1).expand(self.size).contiguous()
 
     def forward(self, ctx: StepContext, residual, pending):
         out = ctx.empty((residual.shape[0], self.size))
+        if isinstance(pending, (SumRows, NormedRows)) and not self.center:
+            ctx.ops.stream_norm(residual, pending, self.gain, self.eps, out)
+            return out
         pending = plain_rows(ctx, pending)
         if isinstance(pending, PendingRows):
             ctx.ops.rmsnorm(residual, self.gain, self.eps, out, rows_sum=pending, center=self.center)
@@ -49,6 +58,9 @@ class RMSNorm(Norm):
 
     def forward_rows(self, ctx: StepContext, residual, rows, pending=None):
         out = ctx.empty((rows.shape[0], self.size))
+        if isinstance(pending, (SumRows, NormedRows)) and not self.center:
+            ctx.ops.stream_norm(residual, pending, self.gain, self.eps, out, rows=rows)
+            return out
         pending = plain_rows(ctx, pending)
         if isinstance(pending, PendingRows):
             ctx.ops.rmsnorm(residual, self.gain, self.eps, out, rows_sum=pending, rows=rows,

@@ -18,6 +18,8 @@ A `scaling` with the keys {factor, original, low, high} slows pairs down by thei
 l_i = 2 pi / f_i instead: f_i stays where l_i < original / high, becomes f_i / factor where
 l_i > original / low, and between the two, with s = (original / l_i - low) / (high - low),
 (1 - s) f_i / factor + s f_i; cosine and sine keep their size.
+
+A `scaling` with the key {factor} alone divides every f_i by it.
 """
 from __future__ import annotations
 
@@ -37,7 +39,8 @@ class Rotary(PositionEncoding):
         context, and the turns over that context above which a pair is left alone (`fast`)
         and below which it is stretched in full (`slow`); or {'factor', 'original', 'low',
         'high'}: the same bounds given as wavelengths, original / high and original / low, with
-        the blend linear in the turns and cosine and sine left as they are."""
+        the blend linear in the turns and cosine and sine left as they are; or {'factor'}: every
+        frequency divided by it."""
         if rot_dim % 2:
             raise ValueError(f"rotary dimension must be even, got {rot_dim}")
         if pairing not in ("half", "interleaved"):
@@ -48,7 +51,12 @@ class Rotary(PositionEncoding):
         self.scaling = None
         self.magnitude = 1.0   # factor on cosine and sine
         self.bands = None
-        if scaling is not None and "low" in scaling and "high" in scaling:
+        self.divisor = 1.0
+        if scaling is not None and set(scaling) == {"factor"}:
+            self.divisor = float(scaling["factor"])
+            if not self.divisor > 0:
+                raise ValueError("rotary scaling needs factor > 0")
+        elif scaling is not None and "low" in scaling and "high" in scaling:
             missing = [k for k in ("factor", "original") if k not in scaling]
             if missing:
                 raise ValueError(f"rotary scaling lacks {missing}")
@@ -89,7 +97,7 @@ class Rotary(PositionEncoding):
                 else:
                     s = (b["original"] / wave - b["low"]) / (b["high"] - b["low"])
                     vals[i] = (1.0 - s) * f / b["factor"] + s * f
-        return torch.tensor(vals, dtype=torch.float64).to(torch.float32)
+        return (torch.tensor(vals, dtype=torch.float64) / self.divisor).to(torch.float32)
 
     def bind(self, w: WeightBinder) -> None:
         self._table = self.inv_freq().to(w.device)

@@ -336,7 +336,7 @@ class PlainOps:
 
     def paged_attention(self, qkv, k_pool, v_pool, block_table, ctx, n_q, n_kv, head_dim,
                         page_size, window, scale, out, slopes=None, vdim=None, sink=False,
-                        blocks=None, gate=None):
+                        blocks=None, gate=None, sinks=None):
         t = qkv.shape[0]
         vdim = head_dim if vdim is None else vdim
         q = _f(qkv[:, :n_q * head_dim]).view(t, n_q, head_dim)
@@ -362,9 +362,10 @@ class PlainOps:
                 s = (k[:, g, :] @ q[r, h]) * scale
                 if slopes is not None:
                     s = s + float(slopes[h]) * (js - pos[r]).float().to(s.device)
-                top = torch.clamp(s.max(), min=0.0) if sink else s.max()
+                rest = 0.0 if sinks is None else float(sinks[h])     # the sink's score, where there is one
+                top = torch.clamp(s.max(), min=rest) if sink else s.max()
                 p = torch.exp(s - top)
-                p = p / (p.sum() + (torch.exp(-top) if sink else 0.0))
+                p = p / (p.sum() + (torch.exp(rest - top) if sink else 0.0))
                 y = p @ v[:, g, :]
                 if gate is not None:
                     y = y * torch.sigmoid(_f(gate[r, h * vdim:(h + 1) * vdim]))
@@ -372,7 +373,8 @@ class PlainOps:
 
     def qkv_wide(self, u, ctx, q_out, heads, kv_heads, dim, vdim, k_pool, v_pool, block_table,
                  page_size, v_col=None, q_norm=None, k_norm=None, norm_eps=0.0, inv_freq=None,
-                 rot_dim=0, interleaved=False, magnitude=1.0, head_scale=None, blocks=None):
+                 rot_dim=0, interleaved=False, magnitude=1.0, head_scale=None, blocks=None,
+                 unit_heads=False):
         t, nq, nk = ctx.T, heads * dim, kv_heads * dim
         v_col = nq + nk if v_col is None else v_col
         x = _f(u)
@@ -384,6 +386,8 @@ class PlainOps:
             turned = self._turn(y, ctx.positions, inv_freq, rot_dim, interleaved)
             if magnitude != 1.0:
                 turned = torch.cat([turned[..., :rot_dim] * magnitude, y[..., rot_dim:]], -1)
+            if unit_heads:
+                turned = turned * torch.rsqrt((turned * turned).mean(-1, keepdim=True) + norm_eps)
             return turned
         q = ready(x[:, :nq], q_norm, heads)
         if head_scale is not None:
@@ -477,16 +481,106 @@ class PlainOps:
             total += _f(f) * gate(g2, b2)
         residual += mult * total
 
-    def gated_rmsnorm(self, o, gate, weight, eps, out, group=0, gate_act="sigmoid"):
+    def gated_rmsnorm(self, o, gate, weight, eps, out, group=0, gate_act="sigmoid", gate_first=False,
+                      den=None):
         t, n = o.shape
         g = group or n
-        x = o.view(t, n // g, g)
-        x = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * weight
-        f = 1.0
+        x, f = o, 1.0
         if gate is not None:
             z = _f(gate)
             f = torch.sigmoid(z) * (z if gate_act == "silu" else 1.0)
-        out.copy_((x.reshape(t, n) * f).to(out.dtype))
+        if gate_first:
+            x, f = x * f, 1.0
+        x = x.reshape(t, n // g, g)
+        if den is not None:
+            x = x / den[:, :, None]
+        x = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps)
+        x = x.reshape(t, n) * weight if weight.shape[0] == n else (x * weight).reshape(t, n)
+        out.copy_((x * f).to(out.dtype))
+
+    def stream_norm(self, residual, pending=None, gain=None, eps=0.0, out=None, rows=None):
+        add = torch.zeros_like(residual)
+        if hasattr(pending, "y"):
+            y = _f(pending.y)
+            add = y * torch.rsqrt((y * y).mean(-1, keepdim=True) + pending.eps) * pending.gain
+        elif hasattr(pending, "factor_a"):
+            add = pending.factor_a * _f(pending.a)
+            if pending.b is not None:
+                add = add + pending.factor_b * _f(pending.b)
+            if pending.bias is not None:
+                add = add + pending.bias
+        elif pending is not None:
+            add = _f(pending)
+        if rows is None:
+            residual += add
+            z = residual
+        else:
+            z = (residual + add)[rows.long()]
+        if out is None:
+            return
+        if gain is not None:
+            z = z * torch.rsqrt((z * z).mean(-1, keepdim=True) + eps) * gain
+        out.copy_(z.to(out.dtype))
+
+    def token_gate(self, z, table, tokens, column0, out):
+        e = _f(table[tokens.long()])[:, column0:column0 + z.shape[1]]
+        out.copy_((self._act(_f(z), "gelu_pytorch_tanh") * e).to(out.dtype))
+
+    def conv_silu(self, u, w, bias, state, ctx, out):
+        taps, c = w.shape
+        starts, slots = ctx.seq_row_start.tolist(), ctx.seq_slots.tolist()
+        for s in range(ctx.S):
+            lo, hi = starts[s], starts[s + 1]
+            x = _f(u[lo:hi])
+            if taps > 1:
+                st = state[slots[s]]
+                x = torch.cat([st[:(taps - 1) * c].view(taps - 1, c), x])
+                st[:(taps - 1) * c] = x[x.shape[0] - (taps - 1):].reshape(-1)
+            y = bias + sum(w[j] * x[j:j + hi - lo] for j in range(taps))
+            out[lo:hi] = (y * torch.sigmoid(y)).to(out.dtype)
+
+    @staticmethod
+    def _softplus(z):
+        return torch.clamp(z, min=0.0) + torch.log1p(torch.exp(-z.abs()))
+
+    def state_space(self, xbc, heads, vdim, dim, groups, dt, dt_bias, rate, skip, state, ctx, out):
+        inner, gn = heads * vdim, groups * dim
+        starts, slots = ctx.seq_row_start.tolist(), ctx.seq_slots.tolist()
+        step = self._softplus(dt + dt_bias)
+        for s in range(ctx.S):
+            S = state[slots[s], :heads * dim * vdim].view(heads, dim, vdim)
+            for t in range(starts[s], starts[s + 1]):
+                r = _f(xbc[t])
+                x = r[:inner].view(heads, vdim)
+                b = r[inner:inner + gn].view(groups, dim).repeat_interleave(heads // groups, 0)
+                c = r[inner + gn:].view(groups, dim).repeat_interleave(heads // groups, 0)
+                S.mul_(torch.exp(-rate * step[t])[:, None, None])
+                S.add_(step[t][:, None, None] * b[:, :, None] * x[:, None, :])
+                out[t] = ((S * c[:, :, None]).sum(1) + skip[:, None] * x).reshape(-1)
+
+    def matrix_memory(self, u, q_off, k_off, v_off, z, z_bias, heads, dim, vdim, cap, q_scale, state, ctx,
+                      gate, norm_w, eps, out):
+        starts, slots = ctx.seq_row_start.tolist(), ctx.seq_slots.tolist()
+        zc = cap * torch.tanh((z + z_bias) / cap)
+        write, keep = zc[:, :heads], -self._softplus(-zc[:, heads:])
+        n_s, n_n = heads * dim * vdim, heads * dim
+        o, den = torch.zeros(ctx.T, heads * vdim), torch.zeros(ctx.T, heads)
+        for s in range(ctx.S):
+            st = state[slots[s]]
+            S, n = st[:n_s].view(heads, dim, vdim), st[n_s:n_s + n_n].view(heads, dim)
+            m = st[n_s + n_n:n_s + n_n + heads]
+            for t in range(starts[s], starts[s + 1]):
+                q = _f(u[t, q_off:q_off + n_n]).view(heads, dim) * q_scale
+                k = _f(u[t, k_off:k_off + n_n]).view(heads, dim)
+                v = _f(u[t, v_off:v_off + heads * vdim]).view(heads, vdim)
+                top = torch.maximum(keep[t] + m, write[t])
+                a, b = torch.exp(keep[t] + m - top), torch.exp(write[t] - top)
+                S.mul_(a[:, None, None]).add_(b[:, None, None] * k[:, :, None] * v[:, None, :])
+                n.mul_(a[:, None]).add_(b[:, None] * k)
+                m.copy_(top)
+                o[t] = (S * q[:, :, None]).sum(1).reshape(-1)
+                den[t] = torch.maximum((n * q).sum(-1).abs(), torch.exp(-top)) + 1e-6
+        self.gated_rmsnorm(o, gate, norm_w, eps, out, group=vdim, den=den)
 
     def gla_work_floats(self, qkv_dtype, ctx, heads, dim):
         return 0
