@@ -49,6 +49,13 @@ a mean key and value per block of tokens before the window, or gated windowed at
 forget-gate linear attention side by side; a dense feed-forward) beside a dense Qwen2-style
 model of the same width, depth, heads, window and feed-forward size.
 
+    python bench.py --scenario designs --design nosedra [--sizes small,medium] [--only nosedra|rudazen]
+
+the same for Nosedra (attention with unit heads, a learned sink and an output gate beside a
+matrix memory, or a state-space layer; a dense feed-forward with biases and a per-layer token
+input) beside a Rudazen model of the same width, depth, feed-forward, heads and memory sizes,
+every layer with attention and a recurrence side by side.
+
     python bench.py --scenario long [--model 57b-a14b] [--requests 8] [--prompt 32768] [--new 256]
 
 is another measurement with a JSON line of its own: the scheduler serves
@@ -111,7 +118,7 @@ def main() -> int:
     ap.add_argument("--scenario", default="decode", choices=["decode", "long", "designs"])
     ap.add_argument("--sizes", default="small,medium",
                     help="--scenario designs: which of the layer sizes to run (small, medium)")
-    ap.add_argument("--design", default="getodra", choices=["getodra", "sosepel", "fopinex", "tuzapel", "rudazen"],
+    ap.add_argument("--design", default="getodra", choices=["getodra", "sosepel", "fopinex", "tuzapel", "rudazen", "nosedra"],
                     help="--scenario designs: the design to run beside the closest model the engine had")
     ap.add_argument("--only", default="", help="--scenario designs: run this one of the two models only")
     ap.add_argument("--requests", type=int, default=8, help="--scenario long: concurrent requests")
@@ -711,6 +718,47 @@ def dense_for_rudazen_config(z: dict) -> dict:
                 sliding_window=z["window"], max_window_layers=0)
 
 
+NOSEDRA_SIZES = {
+    # width, layers (the second of every four is a state-space layer, the others have attention
+    # and a matrix memory side by side), query and kv heads of a size, the memory's heads and
+    # sizes, the state-space layer's heads, value and state sizes and groups, feed-forward,
+    # numbers of the per-layer token input
+    "small": dict(width=1024, layers=8, heads=8, kv_heads=2, dim=128, mem_heads=4, mem_dim=128, mem_vdim=256,
+                  ssm_heads=32, ssm_vdim=64, ssm_state=128, ssm_groups=4, ff=2816, side=128, vocab=32000,
+                  positions=4096),
+    "medium": dict(width=2048, layers=8, heads=16, kv_heads=4, dim=128, mem_heads=8, mem_dim=128, mem_vdim=256,
+                   ssm_heads=64, ssm_vdim=64, ssm_state=128, ssm_groups=8, ff=5632, side=256, vocab=32000,
+                   positions=4096),
+}
+
+
+def nosedra_config(z: dict) -> dict:
+    left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"],
+            "scale": z["dim"] ** -0.5, "rot": {"base": 500000.0, "dims": z["dim"] // 2, "scaling": {"factor": 4.0}}}
+    parallel = {"type": "parallel", "mlp": {"kind": "dense", "ff": z["ff"]},
+                "mixer": {"left": left, "left_scale": 0.7, "right_scale": 0.7,
+                          "right": {"heads": z["mem_heads"], "dim": z["mem_dim"], "vdim": z["mem_vdim"],
+                                    "gate_cap": 15.0}}}
+    ssm = {"type": "mamba2", "mlp": {"kind": "dense", "ff": z["ff"]},
+           "mixer": {"heads": z["ssm_heads"], "vdim": z["ssm_vdim"], "state": z["ssm_state"],
+                     "groups": z["ssm_groups"], "conv": 4, "norm_groups": 1}}
+    return {"architecture": "Nosedra", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "logit_softcap": 30.0, "token_side": {"dim": z["side"]},
+            "layers": [ssm if i % 4 == 1 else parallel for i in range(z["layers"])]}
+
+
+def rudazen_for_nosedra_config(z: dict) -> dict:
+    """The closest model the engine had: Rudazen with attention (heads of the same number and
+    size over all positions, an output gate) and a recurrence with as large a state side by side
+    in every layer, and a feed-forward of the same size."""
+    left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"],
+            "scale": z["dim"] ** -0.5, "rot": {"base": 500000.0, "dims": z["dim"] // 2}}
+    layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": z["ff"]},
+             "mixer": {"left": left, "right": {"heads": z["mem_heads"], "dim": z["mem_dim"], "vdim": z["mem_vdim"]}}}
+    return {"architecture": "Rudazen", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "postln_alpha": 2.0, "embedding": {"scale": z["width"] ** 0.5}, "layers": [layer] * z["layers"]}
+
+
 def designs_scenario(args) -> int:
     import torch
     from ninfer_amd import Chunk, EngineOptions, random_model
@@ -720,22 +768,25 @@ def designs_scenario(args) -> int:
     gen = torch.Generator().manual_seed(11)
     fopinex = args.design == "fopinex"
     rudazen = args.design == "rudazen"
+    nosedra = args.design == "nosedra"
     out = {"metric": "prefill and decode throughput, " + ("Sosepel beside a Qwen2-MoE model" if sosepel
                      else "Fopinex beside a Qwen2-MoE model" if fopinex
                      else "Tuzapel beside a Qwen2-MoE model" if tuzapel
                      else "Rudazen beside a dense model" if rudazen
+                     else "Nosedra beside a Rudazen model" if nosedra
                      else "Getodra beside a dense model") + " of equal size",
            "unit": "tok/s", "n_gpus": 1, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
            "data": "synthetic", "sizes": {}}
     for size in args.sizes.split(","):
         z = (SOSEPEL_SIZES if sosepel else FOPINEX_SIZES if fopinex else TUZAPEL_SIZES if tuzapel
-             else RUDAZEN_SIZES if rudazen else DESIGN_SIZES)[size]
+             else RUDAZEN_SIZES if rudazen else NOSEDRA_SIZES if nosedra else DESIGN_SIZES)[size]
         ctx = z["positions"]
         row = {"shape": z}
         pairs = (("sosepel", sosepel_config(z)), ("sparse", sparse_config(z))) if sosepel else \
             (("fopinex", fopinex_config(z)), ("sparse", sparse_for_fopinex_config(z))) if fopinex else \
             (("tuzapel", tuzapel_config(z)), ("sparse", sparse_for_tuzapel_config(z))) if tuzapel else \
             (("rudazen", rudazen_config(z)), ("dense", dense_for_rudazen_config(z))) if rudazen else \
+            (("nosedra", nosedra_config(z)), ("rudazen", rudazen_for_nosedra_config(z))) if nosedra else \
             (("getodra", getodra_config(z)), ("dense", dense_config(z)))
         for name, raw in pairs:
             if args.only and name != args.only:

@@ -496,11 +496,16 @@ def check_logits(case, dtype, got, what):
 
 
 def test_layer_by_layer(case):
-    """The 32-bit residual stream after every layer, for a prompt in one step and in portions."""
+    """The 32-bit residual stream after every layer, for a prompt in one step and in portions;
+    bounds from how far the plain streams move when every weight is off by 32-bit rounding (a
+    head whose output all but cancels in front of its norm carries that far)."""
     from ninfer_amd.engine import Chunk
     cfg, w = util.read_folder(case["dirs"]["float32"])
     toks = case["reqs"]["r4"]
     streams = plain.forward(cfg, w, toks)[1]
+    g = torch.Generator().manual_seed(1)
+    off = {k: v.double() * (1 + torch.randn(v.shape, generator=g, dtype=D) * 2.0 ** -24) for k, v in w.items()}
+    moved = [rel_err(a, b) for a, b in zip(plain.forward(cfg, off, toks)[1], streams)]
     runner = make_runner(case, "float32")
     assert len(runner.spec.plan) == len(streams)
     got = []
@@ -521,9 +526,7 @@ def test_layer_by_layer(case):
         runner.close(slot)
         for i, want in enumerate(streams):
             g = torch.cat(got[i]).double()
-            # (a head whose output all but cancels before its norm carries a few rounding errors far)
-            assert rel_err(g, want) < 1e-5, f"layer {i}"
-            assert (g - want).abs().max() <= 1e-4 * max(1.0, want.abs().max().item()), f"layer {i}"
+            assert rel_err(g, want) < max(2e-6, 8 * moved[i]), f"layer {i}"
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
