@@ -106,7 +106,9 @@ __global__ void conv_silu_kernel(ConvSiluArgs a) {
   cs_store<T, VEC>((T*)a.out + (int64_t)t * a.C + c, acc);
 }
 
-// ROWS consecutive rows per thread, TAPS known: every input is read once and kept while it counts
+// ROWS consecutive rows per thread, TAPS known: every input is read once, all reads of a thread
+// under way together (a thread whose rows and their inputs lie in one request; the others take
+// their inputs one by one).
 template <typename T, int VEC, int TAPS, int ROWS>
 __global__ __launch_bounds__(256) void conv_silu_rows_kernel(ConvSiluArgs a) {
   const int pieces = a.C / VEC;
@@ -114,37 +116,43 @@ __global__ __launch_bounds__(256) void conv_silu_rows_kernel(ConvSiluArgs a) {
   const int tile = (int)(idx / pieces), c = (int)(idx - (int64_t)tile * pieces) * VEC;
   const int t0 = tile * ROWS;
   if (t0 >= a.T) return;
-  float w[TAPS][VEC], bias[VEC], win[TAPS][VEC];
+  const int t1 = min(t0 + ROWS, a.T) - 1;
+  const int s0 = a.row_seq[t0], s1 = a.row_seq[t1], r0 = a.seq_row_start[s0];
+  float in[ROWS + TAPS - 1][VEC];
+#pragma unroll
+  for (int k = 0; k < ROWS + TAPS - 1; ++k)
+    cs_load<T, VEC>((const T*)a.u + (int64_t)min(max(t0 + k - (TAPS - 1), 0), a.T - 1) * a.stride + c, in[k]);
+  float w[TAPS][VEC], bias[VEC];
 #pragma unroll
   for (int j = 0; j < TAPS; ++j) cs_load32<VEC>(a.w + (int64_t)j * a.C + c, w[j]);
   cs_load32<VEC>(a.b + c, bias);
-  int seq = -1;
+  const bool plain = s0 == s1 && t0 - (TAPS - 1) >= r0;
 #pragma unroll
   for (int k = 0; k < ROWS; ++k) {
     const int t = t0 + k;
     if (t >= a.T) break;
-    const int s = a.row_seq[t];
-    const int r0 = a.seq_row_start[s], i = t - r0;
-    if (s != seq) {   // the thread's first row, or another request: all of the window anew
-      seq = s;
-      const float* st = a.state ? a.state + (int64_t)a.seq_slots[s] * a.state_stride : nullptr;
-#pragma unroll
-      for (int j = 0; j + 1 < TAPS; ++j) cs_input<T, VEC>(a, st, r0, i - (TAPS - 1 - j), c, win[j]);
-    }
-    cs_load<T, VEC>((const T*)a.u + (int64_t)t * a.stride + c, win[TAPS - 1]);
     float acc[VEC];
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      acc[e] = bias[e];
+    for (int e = 0; e < VEC; ++e) acc[e] = bias[e];
+    if (plain) {
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) acc[e] = fmaf(w[j][e], win[j][e], acc[e]);
-      acc[e] = acc[e] / (1.f + expf(-acc[e]));
+      for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) acc[e] = fmaf(w[j][e], in[k + j][e], acc[e]);
+    } else {
+      const int s = a.row_seq[t], first = a.seq_row_start[s];
+      const float* st = a.state ? a.state + (int64_t)a.seq_slots[s] * a.state_stride : nullptr;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        float v[VEC];
+        cs_input<T, VEC>(a, st, first, t - first - (TAPS - 1 - j), c, v);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) acc[e] = fmaf(w[j][e], v[e], acc[e]);
+      }
     }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) acc[e] = acc[e] / (1.f + expf(-acc[e]));
     cs_store<T, VEC>((T*)a.out + (int64_t)t * a.C + c, acc);
-#pragma unroll
-    for (int j = 0; j + 1 < TAPS; ++j)
-#pragma unroll
-      for (int e = 0; e < VEC; ++e) win[j][e] = win[j + 1][e];
   }
 }
 

@@ -164,10 +164,9 @@ __global__ __launch_bounds__(64 * kSeqWaves) void scan_seq_kernel(ScanArgs a) {
 
 // ---- requests that bring one row each -------------------------------------------------------------
 //
-// A block owns one (request, head) and, in the form kScanStep, up to 64 value columns of it; thread
-// (row, col) moves VEC neighbouring columns of every (threads / 16)th key channel, all loads of a
-// group of 64 columns under way together.
-constexpr int kStepThreads = 512, kStepRows = kStepThreads / 16;
+// A block of NT threads owns one (request, head) and, in the form kScanStep, TX * VEC value columns
+// of it. Thread (row, col) moves VEC neighbouring columns of every (NT / TX)th key channel; all
+// loads of a group of TX * VEC columns are under way together, before anything else is asked for.
 constexpr int kStepMaxDim = 512, kStepMaxV = 1024;
 
 template <int VEC>
@@ -185,11 +184,12 @@ __device__ __forceinline__ void step_store(float* p, const float* f) {
   else p[0] = f[0];
 }
 
-template <typename T, int VEC, int PASSES, int FORM>
-__global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
-  constexpr int COLS = 16 * VEC;
+template <typename T, int NT, int VEC, int TX, int PASSES, int FORM>
+__global__ __launch_bounds__(NT) void scan_step_kernel(ScanArgs a) {
+  constexpr int COLS = TX * VEC, ROWS = NT / TX, WAVES = NT / 64;
+  static_assert(COLS <= NT, "a thread adds up one column");
   __shared__ float q_s[kStepMaxDim], k_s[kStepMaxDim];
-  __shared__ __attribute__((aligned(16))) float part_s[kStepRows / 4][COLS];
+  __shared__ __attribute__((aligned(16))) float part_s[WAVES][COLS];
   __shared__ float o_s[FORM == kScanExp ? kStepMaxV : 1];
   __shared__ float red[16];
   const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -198,23 +198,19 @@ __global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
   const T* r = (const T*)a.rows + row * a.stride;
   float* slot = a.state + (int64_t)a.seq_slots[s] * a.state_stride;
   float* st = slot + (int64_t)h * dim * vdim;
-  const int ty = tid >> 4, tx = tid & 15;
+  const int ty = tid / TX, tx = tid % TX;
   const int c_begin = FORM == kScanExp ? 0 : blockIdx.z * COLS;
   const int c_end = FORM == kScanExp ? vdim : min(vdim, c_begin + COLS);
-  // the first columns' state sets out before anything else
   float S[PASSES][VEC];
+  // (channels and columns beyond the last are fetched from the last: loads inside branches would
+  // be waited for one by one)
   auto fetch = [&](int c0) {
-    const int col = c0 + tx * VEC;
+    const int col = min(c0 + tx * VEC, vdim - VEC);
 #pragma unroll
-    for (int p = 0; p < PASSES; ++p) {
-      const int d = p * kStepRows + ty;
-#pragma unroll
-      for (int e = 0; e < VEC; ++e) S[p][e] = 0.f;
-      if (d < dim && col < vdim) step_load<VEC>(st + (int64_t)d * vdim + col, S[p]);
-    }
+    for (int p = 0; p < PASSES; ++p) step_load<VEC>(st + (int64_t)min(p * ROWS + ty, dim - 1) * vdim + col, S[p]);
   };
   fetch(c_begin);
-  for (int d = tid; d < dim; d += kStepThreads) {
+  for (int d = tid; d < dim; d += NT) {
     q_s[d] = to_f32(r[a.q_off + g * dim + d]) * a.q_scale;
     k_s[d] = to_f32(r[a.k_off + g * dim + d]);
   }
@@ -236,7 +232,7 @@ __global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
   if constexpr (FORM == kScanExp) {
     float* n = slot + (int64_t)H * dim * vdim + (int64_t)h * dim;
     float nq = 0.f;
-    for (int d = tid; d < dim; d += kStepThreads) {
+    for (int d = tid; d < dim; d += NT) {
       const float nn = fmaf(keep, n[d], write * k_s[d]);
       n[d] = nn;
       nq = fmaf(nn, q_s[d], nq);
@@ -256,7 +252,7 @@ __global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
     }
 #pragma unroll
     for (int p = 0; p < PASSES; ++p) {
-      const int d = p * kStepRows + ty;
+      const int d = p * ROWS + ty;
       if (d < dim && col < vdim) {
         const float k = k_s[d], q = q_s[d];
 #pragma unroll
@@ -267,18 +263,17 @@ __global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
         step_store<VEC>(st + (int64_t)d * vdim + col, S[p]);
       }
     }
-    // the four rows of a wave, then the waves
+    // the rows of a wave, then the waves
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      acc[e] += __shfl_xor(acc[e], 16, 64);
-      acc[e] += __shfl_xor(acc[e], 32, 64);
-    }
-    if (lane < 16) step_store<VEC>(&part_s[wave][tx * VEC], acc);
+    for (int off = TX; off < 64; off <<= 1)
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) acc[e] += __shfl_xor(acc[e], off, 64);
+    if (lane < TX) step_store<VEC>(&part_s[wave][tx * VEC], acc);
     __syncthreads();
     if (tid < COLS && c0 + tid < vdim) {
       float o = 0.f;
 #pragma unroll
-      for (int w = 0; w < kStepThreads / 64; ++w) o += part_s[w][tid];
+      for (int w = 0; w < WAVES; ++w) o += part_s[w][tid];
       if constexpr (FORM == kScanStep)
         a.out[(row * H + h) * vdim + c0 + tid] =
             fmaf(a.skip[h], to_f32(r[a.v_off + h * vdim + c0 + tid]), o);
@@ -289,10 +284,10 @@ __global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
   }
   if constexpr (FORM == kScanExp) {   // the head's norm and gate
     float ss = 0.f;
-    for (int c = tid; c < vdim; c += kStepThreads) ss = fmaf(o_s[c], o_s[c], ss);
+    for (int c = tid; c < vdim; c += NT) ss = fmaf(o_s[c], o_s[c], ss);
     ss = block_sum(ss, red);
     const float inv = 1.f / sqrtf(ss / (float)vdim + a.eps);
-    for (int c = tid; c < vdim; c += kStepThreads) {
+    for (int c = tid; c < vdim; c += NT) {
       const float zg = to_f32(((const T*)a.gate)[row * a.gate_stride + h * vdim + c]);
       ((T*)a.normed)[(row * H + h) * vdim + c] =
           from_f32<T>(o_s[c] * inv * a.norm_w[h * vdim + c] / (1.f + expf(-zg)));
@@ -300,17 +295,32 @@ __global__ __launch_bounds__(kStepThreads) void scan_step_kernel(ScanArgs a) {
   }
 }
 
-template <typename T, int VEC, int FORM>
-static int launch_step(const ScanArgs& a, int n, hipStream_t stream) {
-  const dim3 grid(n, a.H, FORM == kScanExp ? 1 : (a.vdim + 16 * VEC - 1) / (16 * VEC));
-  const int passes = (a.dim + kStepRows - 1) / kStepRows;
-  if (passes <= 1) scan_step_kernel<T, VEC, 1, FORM><<<grid, kStepThreads, 0, stream>>>(a);
-  else if (passes <= 2) scan_step_kernel<T, VEC, 2, FORM><<<grid, kStepThreads, 0, stream>>>(a);
-  else if (passes <= 4) scan_step_kernel<T, VEC, 4, FORM><<<grid, kStepThreads, 0, stream>>>(a);
-  else if (passes <= 8) scan_step_kernel<T, VEC, 8, FORM><<<grid, kStepThreads, 0, stream>>>(a);
-  else scan_step_kernel<T, VEC, 16, FORM><<<grid, kStepThreads, 0, stream>>>(a);
+template <typename T, int NT, int VEC, int TX, int FORM>
+static int launch_step_tx(const ScanArgs& a, int n, hipStream_t stream) {
+  const dim3 grid(n, a.H, FORM == kScanExp ? 1 : (a.vdim + TX * VEC - 1) / (TX * VEC));
+  const int passes = (a.dim + NT / TX - 1) / (NT / TX);
+  if (passes <= 1) scan_step_kernel<T, NT, VEC, TX, 1, FORM><<<grid, NT, 0, stream>>>(a);
+  else if (passes <= 2) scan_step_kernel<T, NT, VEC, TX, 2, FORM><<<grid, NT, 0, stream>>>(a);
+  else if (passes <= 4) scan_step_kernel<T, NT, VEC, TX, 4, FORM><<<grid, NT, 0, stream>>>(a);
+  else if (passes <= 8) scan_step_kernel<T, NT, VEC, TX, 8, FORM><<<grid, NT, 0, stream>>>(a);
+  else if constexpr (NT == 512) scan_step_kernel<T, NT, VEC, TX, 16, FORM><<<grid, NT, 0, stream>>>(a);
+  else return set_error(-1, "decay_scan: %d key channels in more passes than there are kernels for", a.dim);
   NINFER_LAUNCH_CHECK();
   return 0;
+}
+
+template <typename T, int VEC, int FORM>
+static int launch_step(const ScanArgs& a, int n, hipStream_t stream) {
+  if constexpr (FORM == kScanStep) {
+    return launch_step_tx<T, 512, VEC, 16, FORM>(a, n, stream);
+  } else {
+    // as many columns at a time as a head has, while a thread's share of the channels is at most 8
+    if constexpr (VEC == 4) {
+      if (a.vdim > 128 && a.dim <= 128) return launch_step_tx<T, 1024, VEC, 64, FORM>(a, n, stream);
+      if (a.vdim > 64 && a.dim <= 256) return launch_step_tx<T, 1024, VEC, 32, FORM>(a, n, stream);
+    }
+    return launch_step_tx<T, 1024, VEC, 16, FORM>(a, n, stream);
+  }
 }
 
 template <typename T, int FORM>

@@ -198,61 +198,72 @@ __device__ __forceinline__ sc_bf16x8 tr_read(const unsigned short* p, int gap_el
 }
 
 // A block: the sum of one (chunk, head) in 64 value columns. Wave w owns the key channels' tiles
-// of 16 w, w + 4, ..
+// of 16 w, w + 4, .. (at most 64 NPW channels). Every load is unconditional and under way before the
+// first result is used: rows, channels and columns beyond the last are fetched from the last.
 template <int NPW>
 __global__ __launch_bounds__(256) void scan_chunk_states_kernel(ScanChunkArgs a) {
+  constexpr int DP = 64 * NPW, KROW = DP + 8, KPC = DP / 8, KP = kScRows * KPC / 256;
+  constexpr int VP = kScRows * 2 * kScCt / 256;
   extern __shared__ __attribute__((aligned(16))) unsigned short lds[];
   int row0, L;
   if (!scan_find_chunk(a.s, blockIdx.x, &row0, &L)) return;
   const int h = blockIdx.y, col0 = blockIdx.z * kScCols, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int dim = a.s.dim, vdim = a.s.vdim, H = a.s.H, g_head = h / (H / a.s.G);
-  const int n_tiles = (dim + 15) / 16, krow = 16 * n_tiles + 8;
-  const int rows32 = (L + 31) / 32 * 32;
   const int64_t chunk_head = (int64_t)blockIdx.x * H + h;
-  unsigned short* k_s = lds;                        // [128][krow]
-  unsigned short* v_s = k_s + kScRows * krow;       // [3][128][kScVRow]
+  unsigned short* k_s = lds;                        // [128][KROW]
+  unsigned short* v_s = k_s + kScRows * KROW;       // [3][128][kScVRow]
   float* e_s = (float*)(v_s + 3 * kScRows * kScVRow);   // [128]
-  const unsigned short* rows = (const unsigned short*)a.s.rows;
-  if (tid < kScRows) {
-    float e = 0.f;
-    if (tid < L) {
-      const int64_t at = (int64_t)h * a.s.T + row0 + tid;
-      const bool step = a.s.form == kScanStep;
-      const float2 r = step ? a.b_last[chunk_head] : sc_minus_max(a.m_in[chunk_head], a.c_max[chunk_head]);
-      const float2 cj = a.c[at];
-      e = sc_exp((r.x + cj.x) + (r.y + cj.y)) * (step ? a.w[at].x : 1.f);
-    }
-    e_s[tid] = e;
+  const unsigned short* rows = (const unsigned short*)a.s.rows + (int64_t)row0 * a.s.stride;
+  const sc_u32x4 zero4 = {0u, 0u, 0u, 0u};
+  sc_u32x4 kreg[KP], vreg[VP];
+#pragma unroll
+  for (int i = 0; i < VP; ++i) {
+    const int p = i * 256 + tid, r = p / (2 * kScCt), d = 8 * (p % (2 * kScCt));
+    vreg[i] = *(const sc_u32x4*)(rows + (int64_t)min(r, L - 1) * a.s.stride + a.s.v_off + h * vdim + min(col0 + d, vdim - 8));
   }
-  for (int p = tid; p < rows32 * 2 * n_tiles; p += 256) {
-    const int r = p / (2 * n_tiles), d = 8 * (p - r * 2 * n_tiles);
-    sc_u32x4 v = {0u, 0u, 0u, 0u};
-    if (r < L && d < dim) v = *(const sc_u32x4*)(rows + (int64_t)(row0 + r) * a.s.stride + a.s.k_off + g_head * dim + d);
-    *(sc_u32x4*)(k_s + r * krow + d) = v;
+#pragma unroll
+  for (int i = 0; i < KP; ++i) {
+    const int p = i * 256 + tid, r = p / KPC, d = 8 * (p % KPC);
+    kreg[i] = *(const sc_u32x4*)(rows + (int64_t)min(r, L - 1) * a.s.stride + a.s.k_off + g_head * dim + min(d, dim - 8));
+  }
+  if (tid < kScRows) {
+    const int64_t at = (int64_t)h * a.s.T + row0 + min(tid, L - 1);
+    const bool step = a.s.form == kScanStep;
+    const float2 r = step ? a.b_last[chunk_head] : sc_minus_max(a.m_in[chunk_head], a.c_max[chunk_head]);
+    const float2 cj = a.c[at];
+    const float e = sc_exp((r.x + cj.x) + (r.y + cj.y)) * (step ? a.w[at].x : 1.f);
+    e_s[tid] = tid < L ? e : 0.f;
+  }
+#pragma unroll
+  for (int i = 0; i < KP; ++i) {
+    const int p = i * 256 + tid, r = p / KPC, d = 8 * (p % KPC);
+    *(sc_u32x4*)(k_s + r * KROW + d) = r < L && d < dim ? kreg[i] : zero4;
   }
   __syncthreads();
-  for (int p = tid; p < rows32 * 2 * kScCt; p += 256) {
-    const int r = p / (2 * kScCt), d = 8 * (p - r * 2 * kScCt);
+#pragma unroll
+  for (int i = 0; i < VP; ++i) {
+    const int p = i * 256 + tid, r = p / (2 * kScCt), d = 8 * (p % (2 * kScCt));
     union { __bf16 b[8]; sc_u32x4 v; } o[3];
-    sc_u32x4 v = {0u, 0u, 0u, 0u};
-    if (r < L && col0 + d < vdim)
-      v = *(const sc_u32x4*)(rows + (int64_t)(row0 + r) * a.s.stride + a.s.v_off + h * vdim + col0 + d);
-    const float e = e_s[r];
+    const float e = col0 + d < vdim ? e_s[r] : 0.f;   // (0 for rows beyond the last)
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
-      split3(__uint_as_float(v[x] << 16) * e, o[0].b[2 * x], o[1].b[2 * x], o[2].b[2 * x]);
-      split3(__uint_as_float(v[x] & 0xffff0000u) * e, o[0].b[2 * x + 1], o[1].b[2 * x + 1], o[2].b[2 * x + 1]);
+      split3(__uint_as_float(vreg[i][x] << 16) * e, o[0].b[2 * x], o[1].b[2 * x], o[2].b[2 * x]);
+      split3(__uint_as_float(vreg[i][x] & 0xffff0000u) * e, o[0].b[2 * x + 1], o[1].b[2 * x + 1], o[2].b[2 * x + 1]);
     }
 #pragma unroll
     for (int sp = 0; sp < 3; ++sp) *(sc_u32x4*)(v_s + (sp * kScRows + r) * kScVRow + d) = o[sp].v;
   }
   if (a.s.form == kScanExp && blockIdx.z == 0 && tid < dim) {   // (dim <= 256)
-    float n = 0.f;
-    for (int j = 0; j < L; ++j) n = fmaf(e_s[j], __uint_as_float((unsigned)k_s[j * krow + tid] << 16), n);
-    a.keys[chunk_head * dim + tid] = n;
+    float n[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int j = 0; j < kScRows; j += 4)
+#pragma unroll
+      for (int x = 0; x < 4; ++x)
+        n[x] = fmaf(e_s[j + x], __uint_as_float((unsigned)k_s[(j + x) * KROW + tid] << 16), n[x]);
+    a.keys[chunk_head * dim + tid] = (n[0] + n[1]) + (n[2] + n[3]);
   }
   __syncthreads();
-  const int c = lane & 15, g = lane >> 4;
+  const int c = lane & 15, g = lane >> 4, n_tiles = (dim + 15) / 16, rows32 = (L + 31) / 32 * 32;
   sc_f32x4 acc[NPW][kScCt];
 #pragma unroll
   for (int i = 0; i < NPW; ++i)
@@ -260,7 +271,9 @@ __global__ __launch_bounds__(256) void scan_chunk_states_kernel(ScanChunkArgs a)
     for (int ct = 0; ct < kScCt; ++ct) acc[i][ct] = sc_f32x4{0.f, 0.f, 0.f, 0.f};
   for (int j0 = 0; j0 < rows32; j0 += 32) {
     const int r = j0 + 8 * g + (c >> 2);
-    sc_bf16x8 va[kScCt][3];
+    sc_bf16x8 va[kScCt][3], kb[NPW];
+#pragma unroll
+    for (int i = 0; i < NPW; ++i) kb[i] = tr_read(k_s + r * KROW + 16 * (wave + 4 * i) + 4 * (c & 3), 4 * KROW);
 #pragma unroll
     for (int ct = 0; ct < kScCt; ++ct)
 #pragma unroll
@@ -268,14 +281,12 @@ __global__ __launch_bounds__(256) void scan_chunk_states_kernel(ScanChunkArgs a)
         va[ct][sp] = tr_read(v_s + (sp * kScRows + r) * kScVRow + 16 * ct + 4 * (c & 3), 4 * kScVRow);
 #pragma unroll
     for (int i = 0; i < NPW; ++i) {
-      const int nt = wave + 4 * i;
-      if (nt < n_tiles) {
-        const sc_bf16x8 kb = tr_read(k_s + r * krow + 16 * nt + 4 * (c & 3), 4 * krow);
+      if (wave + 4 * i < n_tiles) {
 #pragma unroll
         for (int sp = 2; sp >= 0; --sp)
 #pragma unroll
           for (int ct = 0; ct < kScCt; ++ct)
-            acc[i][ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[ct][sp], kb, acc[i][ct], 0, 0, 0);
+            acc[i][ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va[ct][sp], kb[i], acc[i][ct], 0, 0, 0);
       }
     }
   }
@@ -323,7 +334,7 @@ __global__ __launch_bounds__(256) void scan_chunk_carry_kernel(ScanChunkArgs a) 
 // A block: the outputs of one (chunk, head) in 64 value columns; wave w owns rows 32 w .. + 31, in
 // two tiles of 16. In the accumulators lane (c, g) holds row c of a tile and value columns 4 g ..
 template <int KS, int FORM>
-__global__ __launch_bounds__(256) void scan_chunk_outputs_kernel(ScanChunkArgs a) {
+__global__ __launch_bounds__(256, KS <= 4 ? 3 : 1) void scan_chunk_outputs_kernel(ScanChunkArgs a) {
   constexpr int DP = 32 * KS, KROW = DP + 8;
   extern __shared__ __attribute__((aligned(16))) unsigned short lds[];
   __shared__ __attribute__((aligned(16))) float c_s[kScRows], cl_s[kScRows], w_s[kScRows];
@@ -334,7 +345,20 @@ __global__ __launch_bounds__(256) void scan_chunk_outputs_kernel(ScanChunkArgs a
   const int dim = a.s.dim, vdim = a.s.vdim, H = a.s.H, g_head = h / (H / a.s.G);
   const int c = lane & 15, g = lane >> 4;
   const int64_t chunk_head = (int64_t)blockIdx.x * H + h, gates0 = (int64_t)h * a.s.T + row0;
-  const unsigned short* rows = (const unsigned short*)a.s.rows;
+  const unsigned short* rows = (const unsigned short*)a.s.rows + (int64_t)row0 * a.s.stride;
+  const sc_u32x4 zero4 = {0u, 0u, 0u, 0u};
+  // All loads set out here, every one unconditional: rows, channels and columns beyond the last are
+  // fetched from the last. First the state, then queries and gates, then keys and values, which
+  // are not wanted before the state's part is done.
+  constexpr int SP = DP * 4 * kScCt / 256, KPC = DP / 8, KP = kScRows * KPC / 256, VP = kScRows * 2 * kScCt / 256;
+  sc_f32x4 sreg[SP];
+  sc_u32x4 kreg[KP], vreg[VP];
+  const float* S = a.sums + chunk_head * dim * vdim;
+#pragma unroll
+  for (int i = 0; i < SP; ++i) {
+    const int p = i * 256 + tid, d = p / (4 * kScCt), col = 4 * (p % (4 * kScCt));
+    sreg[i] = *(const sc_f32x4*)(S + (int64_t)min(d, dim - 1) * vdim + min(col0 + col, vdim - 4));
+  }
   // this lane's queries (operand of both products)
   sc_bf16x8 qf[2][KS];
   float2 r_t[2];
@@ -343,32 +367,44 @@ __global__ __launch_bounds__(256) void scan_chunk_outputs_kernel(ScanChunkArgs a
 #pragma unroll
   for (int tt = 0; tt < 2; ++tt) {
     const int t = min(32 * wave + 16 * tt + c, L - 1);
-    const unsigned short* qr = rows + (int64_t)(row0 + t) * a.s.stride + a.s.q_off + g_head * dim;
+    const unsigned short* qr = rows + (int64_t)t * a.s.stride + a.s.q_off + g_head * dim;
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      const int d = 32 * ks + 8 * g;
-      sc_u32x4 v = {0u, 0u, 0u, 0u};
-      if (d < dim) v = *(const sc_u32x4*)(qr + d);
-      qf[tt][ks] = __builtin_bit_cast(sc_bf16x8, v);
-    }
-    r_t[tt] = FORM == kScanExp ? sc_minus_max(m_in, a.w[gates0 + t]) : a.b[gates0 + t];
+    for (int ks = 0; ks < KS; ++ks)
+      qf[tt][ks] = __builtin_bit_cast(sc_bf16x8, *(const sc_u32x4*)(qr + min(32 * ks + 8 * g, dim - 8)));
+    r_t[tt] = FORM == kScanExp ? a.w[gates0 + t] : a.b[gates0 + t];
+  }
+  const float2 c_t = a.c[gates0 + min(tid & (kScRows - 1), L - 1)], w_t = a.w[gates0 + min(tid & (kScRows - 1), L - 1)];
+#pragma unroll
+  for (int i = 0; i < KP; ++i) {
+    const int p = i * 256 + tid, r = p / KPC, d = 8 * (p % KPC);
+    kreg[i] = *(const sc_u32x4*)(rows + (int64_t)min(r, L - 1) * a.s.stride + a.s.k_off + g_head * dim + min(d, dim - 8));
+  }
+#pragma unroll
+  for (int i = 0; i < VP; ++i) {
+    const int p = i * 256 + tid, r = p / (2 * kScCt), d = 8 * (p % (2 * kScCt));
+    vreg[i] = *(const sc_u32x4*)(rows + (int64_t)min(r, L - 1) * a.s.stride + a.s.v_off + h * vdim + min(col0 + d, vdim - 8));
+  }
+#pragma unroll
+  for (int tt = 0; tt < 2; ++tt) {
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+      if (32 * ks + 8 * g >= dim) qf[tt][ks] = __builtin_bit_cast(sc_bf16x8, zero4);
+    if (FORM == kScanExp) r_t[tt] = sc_minus_max(m_in, r_t[tt]);
     scale_in[tt] = sc_exp((m_in + r_t[tt].x) + r_t[tt].y);
   }
   if (tid < kScRows) {
-    const float2 cj = tid < L ? a.c[gates0 + tid] : make_float2(0.f, 0.f);
-    c_s[tid] = cj.x;
-    cl_s[tid] = cj.y;
-    w_s[tid] = FORM == kScanExp ? 1.f : tid < L ? a.w[gates0 + tid].x : 0.f;
+    c_s[tid] = tid < L ? c_t.x : 0.f;
+    cl_s[tid] = tid < L ? c_t.y : 0.f;
+    w_s[tid] = FORM == kScanExp ? 1.f : tid < L ? w_t.x : 0.f;
   }
   // 1. the state before the chunk, in three parts: [3][DP][kScVRow]
-  const float* S = a.sums + chunk_head * dim * vdim + col0;
-  for (int p = tid; p < DP * 4 * kScCt; p += 256) {
-    const int d = p / (4 * kScCt), col = 4 * (p - d * 4 * kScCt);
-    sc_f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    if (d < dim && col0 + col < vdim) v = *(const sc_f32x4*)(S + (int64_t)d * vdim + col);
+#pragma unroll
+  for (int i = 0; i < SP; ++i) {
+    const int p = i * 256 + tid, d = p / (4 * kScCt), col = 4 * (p % (4 * kScCt));
+    const bool in = d < dim && col0 + col < vdim;
     union { __bf16 b[4]; uint2 u; } o[3];
 #pragma unroll
-    for (int x = 0; x < 4; ++x) split3(v[x], o[0].b[x], o[1].b[x], o[2].b[x]);
+    for (int x = 0; x < 4; ++x) split3(in ? sreg[i][x] : 0.f, o[0].b[x], o[1].b[x], o[2].b[x]);
 #pragma unroll
     for (int sp = 0; sp < 3; ++sp) *(uint2*)(lds + (sp * DP + d) * kScVRow + col) = o[sp].u;
   }
@@ -414,19 +450,15 @@ __global__ __launch_bounds__(256) void scan_chunk_outputs_kernel(ScanChunkArgs a
   // 2. keys [128][KROW] and values [128][kScVRow]
   unsigned short* k_s = lds;
   unsigned short* v_s = lds + kScRows * KROW;
-  const int rows32 = (L + 31) / 32 * 32;
-  for (int p = tid; p < rows32 * 4 * KS; p += 256) {
-    const int r = p / (4 * KS), d = 8 * (p - r * 4 * KS);
-    sc_u32x4 v = {0u, 0u, 0u, 0u};
-    if (r < L && d < dim) v = *(const sc_u32x4*)(rows + (int64_t)(row0 + r) * a.s.stride + a.s.k_off + g_head * dim + d);
-    *(sc_u32x4*)(k_s + r * KROW + d) = v;
+#pragma unroll
+  for (int i = 0; i < KP; ++i) {
+    const int p = i * 256 + tid, r = p / KPC, d = 8 * (p % KPC);
+    *(sc_u32x4*)(k_s + r * KROW + d) = r < L && d < dim ? kreg[i] : zero4;
   }
-  for (int p = tid; p < rows32 * 2 * kScCt; p += 256) {
-    const int r = p / (2 * kScCt), d = 8 * (p - r * 2 * kScCt);
-    sc_u32x4 v = {0u, 0u, 0u, 0u};
-    if (r < L && col0 + d < vdim)
-      v = *(const sc_u32x4*)(rows + (int64_t)(row0 + r) * a.s.stride + a.s.v_off + h * vdim + col0 + d);
-    *(sc_u32x4*)(v_s + r * kScVRow + d) = v;
+#pragma unroll
+  for (int i = 0; i < VP; ++i) {
+    const int p = i * 256 + tid, r = p / (2 * kScCt), d = 8 * (p % (2 * kScCt));
+    *(sc_u32x4*)(v_s + r * kScVRow + d) = r < L && col0 + d < vdim ? vreg[i] : zero4;
   }
   __syncthreads();
   if (!live) return;
@@ -535,8 +567,7 @@ static int scan_lds(K kern, size_t lds, bool* raised) {
 
 template <int NPW>
 static int launch_states(const ScanChunkArgs& a, dim3 grid, hipStream_t stream) {
-  const int krow = (a.s.dim + 15) / 16 * 16 + 8;
-  const size_t lds = ((size_t)kScRows * krow + 3 * kScRows * kScVRow) * 2 + kScRows * sizeof(float);
+  const size_t lds = ((size_t)kScRows * (64 * NPW + 8) + 3 * kScRows * kScVRow) * 2 + kScRows * sizeof(float);
   static bool raised = false;
   if (int rc = scan_lds(scan_chunk_states_kernel<NPW>, lds, &raised)) return rc;
   scan_chunk_states_kernel<NPW><<<grid, 256, lds, stream>>>(a);

@@ -52,6 +52,8 @@ extern "C" int ninfer_gemm_pair(const GemmArgs* a, const GemmArgs* b, int force_
   if (rc) return rc;
   if (!force_generic && !many_rows(*a) && !many_rows(*b) && gemm_skinny_pair_takes(*a, *b))
     return gemm_skinny_pair(*a, *b, stream);
+  if (!force_generic && !many_rows(*a) && !many_rows(*b) && gemm_skinny_pair_takes(*b, *a))
+    return gemm_skinny_pair(*b, *a, stream);
   rc = ninfer_gemm(a, force_generic, stream);
   if (rc) return rc;
   return ninfer_gemm(b, force_generic, stream);

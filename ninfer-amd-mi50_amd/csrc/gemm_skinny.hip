@@ -496,7 +496,9 @@ int gemm_skinny(const GemmArgs& a, hipStream_t stream) {
 
 // The pairs that have a kernel: (dense, 32-bit out) beside (dense SwiGLU), as a router's
 // logits beside a shared expert's gate and up; (grouped) beside (dense), as the experts'
-// down products beside the shared expert's. Both bf16 in, the second bf16 out.
+// down products beside the shared expert's; (dense, any out) beside (dense), as a few numbers
+// wanted in 32-bit beside the wide product of the same rows, or two output products. All bf16 in,
+// the second bf16 out.
 bool gemm_skinny_pair_takes(const GemmArgs& a, const GemmArgs& b) {
   if (!gemm_skinny_takes(a) || !gemm_skinny_takes(b) || a.bias || b.bias) return false;
   const bool dense_b = !b.offsets && b.out_dtype == kBF16;
@@ -504,7 +506,8 @@ bool gemm_skinny_pair_takes(const GemmArgs& a, const GemmArgs& b) {
                      dense_b && epilogue_gated(b.epilogue);
   const bool second = a.offsets && a.out_dtype == kBF16 && a.epilogue == kEpilogueNone &&
                       dense_b && b.epilogue == kEpilogueNone;
-  return first || second;
+  const bool third = !a.offsets && a.epilogue == kEpilogueNone && dense_b && b.epilogue == kEpilogueNone;
+  return first || second || third;
 }
 
 int gemm_skinny_pair(const GemmArgs& a, const GemmArgs& b, hipStream_t stream) {
@@ -527,7 +530,13 @@ int gemm_skinny_pair(const GemmArgs& a, const GemmArgs& b, hipStream_t stream) {
   const long blocks = (long)pa.grid_x * pa.grid_y +
                       (pb.grid_y > 1 ? (long)line_ids(pb.grid_x, pb.grid_y) : (long)pb.grid_x);
   NINFER_REQUIRE(blocks < (1L << 31), "gemm pair: %ld blocks are too many", blocks);
-  if (!a.offsets)
+  if (!a.offsets && b.epilogue == kEpilogueNone && a.out_dtype == kF32)
+    gemm_skinny_pair_kernel<false, false, float, false, false, bf16>
+        <<<(unsigned)blocks, threads, lds, stream>>>(a, pa, b, pb);
+  else if (!a.offsets && b.epilogue == kEpilogueNone)
+    gemm_skinny_pair_kernel<false, false, bf16, false, false, bf16>
+        <<<(unsigned)blocks, threads, lds, stream>>>(a, pa, b, pb);
+  else if (!a.offsets)
     gemm_skinny_pair_kernel<false, false, float, false, true, bf16>
         <<<(unsigned)blocks, threads, lds, stream>>>(a, pa, b, pb);
   else if (pa.two)

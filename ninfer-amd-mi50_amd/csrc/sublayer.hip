@@ -311,74 +311,110 @@ struct GatedNormArgs {
   float eps;
 };
 
-// A number of the row as the norm takes it, and the factor that follows the norm.
-template <typename T>
-__device__ __forceinline__ float gated_norm_in(const GatedNormArgs& a, int64_t r, int i, float inv_den, float* after) {
-  float v = a.o[r * a.N + i] * inv_den;
-  float sg = 1.f;
-  if (a.gate) {
-    const float z = to_f32(((const T*)a.gate)[r * a.gate_stride + i]);
-    sg = (a.silu ? z : 1.f) / (1.f + expf(-z));
+// VEC numbers of the row as the norm takes them, and the factors that follow the norm.
+template <typename T, int VEC>
+__device__ __forceinline__ void gated_norm_in(const GatedNormArgs& a, int64_t r, int i, float inv_den, float* v, float* after) {
+  na_load<VEC>(a.o + r * a.N + i, v);
+  float z[VEC];
+  if (a.gate) na_load<VEC>((const T*)a.gate + r * a.gate_stride + i, z);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) {
+    v[e] *= inv_den;
+    after[e] = a.gate ? (a.silu ? z[e] : 1.f) / (1.f + expf(-z[e])) : 1.f;
+    if (a.gate_first) v[e] *= after[e], after[e] = 1.f;
   }
-  if (a.gate_first) v *= sg, sg = 1.f;
-  *after = sg;
-  return v;
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void gated_norm_out(const GatedNormArgs& a, int64_t r, int i, const float* w, float inv,
+                                               const float* v, const float* after) {
+  T* out = (T*)a.out + r * a.N + i;
+  float g[VEC], y[VEC];
+  na_load<VEC>(w, g);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) y[e] = v[e] * inv * g[e] * after[e];
+  if constexpr (VEC == 4 && sizeof(T) == 4) {
+    *(float4*)out = make_float4(y[0], y[1], y[2], y[3]);
+  } else if constexpr (VEC == 4) {
+    union { __bf16 b[4]; uint2 u; } p;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) p.b[e] = (__bf16)y[e];
+    *(uint2*)out = p.u;
+  } else {
+    out[0] = from_f32<T>(y[0]);
+  }
 }
 
-// A block per (row, group); a thread keeps its (at most 16) numbers in registers.
+// A block per (row, group); a thread keeps its (at most 16) numbers in registers, in groups of VEC
+// consecutive ones.
 constexpr int kGatedPerThread = 16;
-template <typename T>
+template <typename T, int VEC>
 __global__ void gated_rmsnorm_kernel(GatedNormArgs a) {
+  constexpr int G = kGatedPerThread / VEC;
   __shared__ float red[16];
   const int64_t r = blockIdx.x;
   const int g0 = blockIdx.y * a.group;
   const float inv_den = a.den ? 1.f / a.den[r * gridDim.y + blockIdx.y] : 1.f;
   const float* w = a.w + (a.w_n == a.N ? g0 : 0);
-  float v[kGatedPerThread], sg[kGatedPerThread];
+  float v[G][VEC], sg[G][VEC];
   float ss = 0.f;
 #pragma unroll
-  for (int c = 0; c < kGatedPerThread; ++c) {
-    const int i = threadIdx.x + c * blockDim.x;
-    v[c] = sg[c] = 0.f;
-    if (i < a.group) v[c] = gated_norm_in<T>(a, r, g0 + i, inv_den, &sg[c]);
-    ss = fmaf(v[c], v[c], ss);
+  for (int c = 0; c < G; ++c) {
+    const int i = VEC * (threadIdx.x + c * blockDim.x);
+    if (i < a.group) {
+      gated_norm_in<T, VEC>(a, r, g0 + i, inv_den, v[c], sg[c]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss = fmaf(v[c][e], v[c][e], ss);
+    }
   }
   ss = block_sum(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)a.group + a.eps);
 #pragma unroll
-  for (int c = 0; c < kGatedPerThread; ++c) {
-    const int i = threadIdx.x + c * blockDim.x;
-    if (i < a.group) ((T*)a.out)[r * a.N + g0 + i] = from_f32<T>(v[c] * inv * w[i] * sg[c]);
+  for (int c = 0; c < G; ++c) {
+    const int i = VEC * (threadIdx.x + c * blockDim.x);
+    if (i < a.group) gated_norm_out<T, VEC>(a, r, g0 + i, w + i, inv, v[c], sg[c]);
   }
 }
 
 // The same for groups of few columns (a head's values): one wave per (row, group), four groups
 // to a block.
 constexpr int kGatedWaveMax = 512;
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void gated_group_rmsnorm_kernel(GatedNormArgs a) {
+  constexpr int PER = kGatedWaveMax / 64 / VEC;
   const int64_t r = blockIdx.x;
   const int g = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int g0 = g * a.group;
   if (g0 >= a.N) return;
   const float inv_den = a.den ? 1.f / a.den[r * (a.N / a.group) + g] : 1.f;
   const float* w = a.w + (a.w_n == a.N ? g0 : 0);
-  constexpr int PER = kGatedWaveMax / 64;
-  float v[PER], sg[PER];
+  float v[PER][VEC], sg[PER][VEC];
   float ss = 0.f;
 #pragma unroll
   for (int c = 0; c < PER; ++c) {
-    const int i = lane + 64 * c;
-    v[c] = sg[c] = 0.f;
-    if (i < a.group) v[c] = gated_norm_in<T>(a, r, g0 + i, inv_den, &sg[c]);
-    ss = fmaf(v[c], v[c], ss);
+    const int i = VEC * (lane + 64 * c);
+    if (i < a.group) {
+      gated_norm_in<T, VEC>(a, r, g0 + i, inv_den, v[c], sg[c]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss = fmaf(v[c][e], v[c][e], ss);
+    }
   }
   ss = wave_sum(ss);
   const float inv = 1.f / sqrtf(ss / (float)a.group + a.eps);
 #pragma unroll
   for (int c = 0; c < PER; ++c) {
-    const int i = lane + 64 * c;
-    if (i < a.group) ((T*)a.out)[r * a.N + g0 + i] = from_f32<T>(v[c] * inv * w[i] * sg[c]);
+    const int i = VEC * (lane + 64 * c);
+    if (i < a.group) gated_norm_out<T, VEC>(a, r, g0 + i, w + i, inv, v[c], sg[c]);
+  }
+}
+
+template <typename T, int VEC>
+static void launch_gated_norm(const GatedNormArgs& a, hipStream_t stream) {
+  const int groups = a.N / a.group;
+  if (a.group <= kGatedWaveMax && groups > 1) {
+    gated_group_rmsnorm_kernel<T, VEC><<<dim3(a.T, (groups + 3) / 4), 256, 0, stream>>>(a);
+  } else {
+    const int want = ((a.group + VEC - 1) / VEC + 63) / 64 * 64;
+    gated_rmsnorm_kernel<T, VEC><<<dim3(a.T, groups), want > 1024 ? 1024 : want, 0, stream>>>(a);
   }
 }
 
@@ -484,16 +520,15 @@ extern "C" int ninfer_gated_rmsnorm(const GatedNormArgs* args, hipStream_t strea
   NINFER_REQUIRE(a.w_n == a.N || a.w_n == a.group, "gated_rmsnorm: %d weights for groups of %d columns", a.w_n, a.group);
   NINFER_REQUIRE(a.group <= 1024 * kGatedPerThread, "gated_rmsnorm: %d columns exceed %d", a.group, 1024 * kGatedPerThread);
   NINFER_REQUIRE(!a.gate_first || a.gate, "gated_rmsnorm: no gate to apply first");
-  const int groups = a.N / a.group;
-  if (a.group <= kGatedWaveMax && groups > 1) {
-    const dim3 grid(a.T, (groups + 3) / 4);
-    if (a.dtype == kF32) gated_group_rmsnorm_kernel<float><<<grid, 256, 0, stream>>>(a);
-    else gated_group_rmsnorm_kernel<bf16><<<grid, 256, 0, stream>>>(a);
+  auto aligned = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+  const bool vec = a.group % 4 == 0 && (!a.gate || a.gate_stride % 4 == 0) && aligned(a.o) && aligned(a.gate) &&
+                   aligned(a.w) && aligned(a.out);
+  if (a.dtype == kF32) {
+    if (vec) launch_gated_norm<float, 4>(a, stream);
+    else launch_gated_norm<float, 1>(a, stream);
   } else {
-    const int block = a.group >= 1024 ? 1024 : (a.group + 63) / 64 * 64;
-    const dim3 grid(a.T, groups);
-    if (a.dtype == kF32) gated_rmsnorm_kernel<float><<<grid, block, 0, stream>>>(a);
-    else gated_rmsnorm_kernel<bf16><<<grid, block, 0, stream>>>(a);
+    if (vec) launch_gated_norm<bf16, 4>(a, stream);
+    else launch_gated_norm<bf16, 1>(a, stream);
   }
   NINFER_LAUNCH_CHECK();
   return 0;
