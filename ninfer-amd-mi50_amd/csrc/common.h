@@ -21,6 +21,13 @@ template <typename T> __device__ __forceinline__ T from_f32(float v);
 template <> __device__ __forceinline__ float from_f32<float>(float v) { return v; }
 template <> __device__ __forceinline__ bf16 from_f32<bf16>(float v) { return __float2bfloat16(v); }
 
+// 1 / (1 + e^-z) for a result of type T: the hardware's exponential and reciprocal (good to a few
+// units of the 32-bit result's last place) where it is rounded to bfloat16 anyway.
+template <typename T> __device__ __forceinline__ float sigmoid_for(float z) { return 1.f / (1.f + expf(-z)); }
+template <> __device__ __forceinline__ float sigmoid_for<bf16>(float z) {
+  return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.44269504088896f * z));
+}
+
 constexpr int kWave = 64;
 // gfx950 (the one target) has 8 XCDs, each with an L2 of its own; the hardware deals
 // workgroups to them in turn (block id mod 8). Kernels that share operands through L2 map

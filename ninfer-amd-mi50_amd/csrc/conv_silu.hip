@@ -102,7 +102,7 @@ __global__ void conv_silu_kernel(ConvSiluArgs a) {
     cs_store32<VEC>(st + (int64_t)(a.taps - 2) * a.C + c, v);   // (v: the row's own input, the last tap's)
   }
 #pragma unroll
-  for (int e = 0; e < VEC; ++e) acc[e] = acc[e] / (1.f + expf(-acc[e]));
+  for (int e = 0; e < VEC; ++e) acc[e] *= sigmoid_for<T>(acc[e]);
   cs_store<T, VEC>((T*)a.out + (int64_t)t * a.C + c, acc);
 }
 
@@ -151,7 +151,7 @@ __global__ __launch_bounds__(256) void conv_silu_rows_kernel(ConvSiluArgs a) {
       }
     }
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) acc[e] = acc[e] / (1.f + expf(-acc[e]));
+    for (int e = 0; e < VEC; ++e) acc[e] *= sigmoid_for<T>(acc[e]);
     cs_store<T, VEC>((T*)a.out + (int64_t)t * a.C + c, acc);
   }
 }
@@ -175,7 +175,7 @@ __global__ void conv_silu_state_kernel(ConvSiluArgs a) {
 
 template <typename T, int VEC>
 static int launch_conv_silu(const ConvSiluArgs& a, hipStream_t stream) {
-  constexpr int ROWS = 4;
+  constexpr int ROWS = 8;
   const int64_t pieces = a.C / VEC;
   if (!a.all_single && a.taps >= 2 && a.taps <= 4 && a.T >= 256) {
     const int64_t n = (a.T + ROWS - 1) / ROWS * pieces;

@@ -320,7 +320,7 @@ __device__ __forceinline__ void gated_norm_in(const GatedNormArgs& a, int64_t r,
 #pragma unroll
   for (int e = 0; e < VEC; ++e) {
     v[e] *= inv_den;
-    after[e] = a.gate ? (a.silu ? z[e] : 1.f) / (1.f + expf(-z[e])) : 1.f;
+    after[e] = a.gate ? (a.silu ? z[e] : 1.f) * sigmoid_for<T>(z[e]) : 1.f;
     if (a.gate_first) v[e] *= after[e], after[e] = 1.f;
   }
 }

@@ -60,6 +60,15 @@ def config_ones():
 CASES = {"odd": (config_odd, 41), "even": (config_even, 42), "ones": (config_ones, 43)}
 
 
+def alone(kind: str) -> dict:
+    """A model of layers of one kind (a model of state-space layers keeps nothing in pages)."""
+    if kind == "parallel":
+        layers = [layer(parallel(4, 2, 40, 24, 2, 24, 32, factor=2.0), 48), layer(parallel(2, 1, 16, 16, 3, 8, 16), None)]
+    else:
+        layers = [layer(mamba2(4, 24, 40, groups=2), 48), layer(mamba2(2, 8, 16, conv=3), None)]
+    return model(130, 96, 1e-6, 12, 15.0, layers)
+
+
 def random_config(seed: int) -> dict:
     """A seeded random configuration: sizes, head counts, kinds and order of layers, what is
     absent."""

@@ -334,6 +334,19 @@ def test_host_generation_through_the_scheduler(host_case):
     assert [r.output[:len(x)] for r, x in zip(reqs, want)] == want
 
 
+@pytest.mark.parametrize("kind", ["state-space", "parallel"])
+def test_host_models_of_one_kind_of_layer(kind, tmp_path):
+    import ninfer_amd
+    raw = nosedra_cases.alone(kind)
+    ninfer_amd.write_random_model(str(tmp_path), raw, 6, dtype="float32", std=STD)
+    cfg, w = util.read_folder(str(tmp_path))
+    reqs = {f"r{i}": util.random_tokens(n, raw["vocab"], i) for i, n in enumerate([21, 1, 30])}
+    case = {"dir": str(tmp_path), "ref": {k: plain.forward(cfg, w, v)[0] for k, v in reqs.items()}}
+    runner = _host_runner(case, num_sequences=2)
+    assert bool(runner.cache.groups) == (kind == "parallel")
+    _close(case, util.run_schedule(runner, util.schedule_mixed(reqs, seed=5, max_live=2)))
+
+
 def test_host_new_parts_inside_other_blocks():
     """A state-space layer and a pair of mixers without output norms under a block that takes
     plain rows, and a matrix memory by itself, as another design might use them: every layer is

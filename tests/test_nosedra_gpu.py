@@ -184,6 +184,26 @@ def test_gated_norm_in_its_forms(ops, dtype, heads, dim):
                    plain.unit(od / den.double()[:, :, None], eps).reshape(t, n) * w.double() * torch.sigmoid(z)) < tol
 
 
+@pytest.mark.parametrize("rows", [1, 7, 16, 29])
+def test_two_few_row_products_together(ops, rows):
+    """A narrow product wanted in 32-bit beside a wide one of the same rows, in either order, and
+    two products of different rows and widths: what they give held back and launched together is
+    what they give by themselves."""
+    g = torch.Generator().manual_seed(rows)
+    k = 256
+    x, y = (torch.randn(rows, n, generator=g).to(torch.bfloat16).to(DEV) for n in (k, 2 * k))
+    w = [(torch.randn(n, m, generator=g) * 0.1).to(torch.bfloat16).to(DEV) for n, m in ((10, k), (712, k), (96, k), (96, 2 * k))]
+    pairs = [((x, w[0], torch.float32), (x, w[1], torch.bfloat16)), ((x, w[1], torch.bfloat16), (x, w[0], torch.float32)),
+             ((x, w[2], torch.bfloat16), (y, w[3], torch.bfloat16))]
+    for pair in pairs:
+        outs = [torch.full((rows, m.shape[0]), float("nan"), dtype=d, device=DEV) for _, m, d in pair]
+        with ops.together():
+            for (a, m, _), out in zip(pair, outs):
+                ops.linear(a, m, out)
+        for (a, m, d), out in zip(pair, outs):
+            assert rel_err(out, a.double().cpu() @ m.double().cpu().T) < (1e-6 if d == torch.float32 else 4e-3)
+
+
 def _gather(pool, table, n, page_size):
     """Rows 0 .. n - 1 of a request from its pages: [n, heads, numbers]."""
     js = torch.arange(n)
@@ -655,13 +675,15 @@ def test_decoding_from_a_captured_graph(case, dtype):
     check_logits(case, dtype, {k: torch.cat(v) for k, v in got.items()}, "graph replay")
 
 
-@pytest.mark.parametrize("seed", list(range(10)))
+@pytest.mark.parametrize("seed", ["state-space layers alone", "parallel layers alone"] + list(range(10)))
 def test_random_configurations(seed, tmp_path):
     """Configurations drawn at random (sizes, head counts, kinds and order of layers, what is
-    absent), in both precisions: whole, in portions and in a mixed batch."""
+    absent), and models of one kind of layer, in both precisions: whole, in portions and in a
+    mixed batch."""
     import ninfer_amd
     from ninfer_amd import EngineOptions, load_model
-    raw = nosedra_cases.random_config(seed)
+    raw = nosedra_cases.alone(seed.split()[0]) if isinstance(seed, str) else nosedra_cases.random_config(seed)
+    seed = len(seed) if isinstance(seed, str) else seed
     reqs = {f"q{i}": util.random_tokens(n, raw["vocab"], 7 * seed + i) for i, n in enumerate([33, 1, 14, 50])}
     for dtype in ("float32", "bfloat16"):
         d = str(tmp_path / dtype)
