@@ -22,7 +22,7 @@ struct ScanArgs {
   float* state;             // + slot * state_stride: S [H, dim, vdim], then (kScanExp) n [H, dim], m [H]
   float* out;               // [T, H * vdim] 32-bit
   float* den;               // [T, H] (kScanExp) what the outputs are to be divided by
-  float* work;              // gates of the rows and, for chunks, their states: see scan_work_floats
+  float* work;              // gates of the rows and, for chunks, their states: see scan_chunks_work_floats
   const int* seq_row_start; // [S + 1]
   const int* seq_slots;     // [S]
   int64_t state_stride;

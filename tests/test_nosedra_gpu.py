@@ -314,6 +314,43 @@ def test_attention_with_learned_sinks(ops, dtype, plain_kernel, gated, heads, kv
             assert rel_err(got[:, h], ref[:, h]) < tol, (step, h, float(sinks[h]))
 
 
+@pytest.mark.parametrize("dtype,plain_kernel", KERNELS, indirect=["plain_kernel"])
+@pytest.mark.parametrize("dim,vdim,ps", [(32, 32, 8), (96, 40, 16), (128, 128, 16)])
+def test_one_loud_key_anywhere_before_a_sink(ops, dtype, plain_kernel, dim, vdim, ps):
+    """Among hundreds of keys that score 0 one that stands out, with a value no other has: the
+    request's first, at both sides of pages' and tiles' borders, the row's own, and the one after
+    it, which is not seen; for rows inside prompt portions and for decoded ones. A sink as loud as
+    the key halves what is seen of it."""
+    n, heads = 330, 4
+    rows_at = [0, 1, 63, 64, 127, 128, 200, 329]
+    g = torch.Generator().manual_seed(dim)
+    tables, pages = _tables([-(-n // ps)], 2, g)
+    js = torch.arange(n)
+    sinks = torch.tensor([-40.0, 12.0, -40.0, 12.0])
+    q = torch.zeros(n, heads, dim)
+    q[:, :, 0] = 1.0
+    for loud in (0, 1, ps - 1, ps, 63, 64, 127, 128, 200, 201):
+        k, v = torch.zeros(n, 2, dim), torch.zeros(n, 2, vdim)
+        k[loud, :, 0] = 12.0
+        v[loud] = 8.0
+        pools = []
+        for x in (k, v):
+            pool = torch.full((pages, 2, ps, x.shape[2]), float("nan"), dtype=dtype)
+            pool[torch.tensor(tables[0])[js // ps], :, js % ps] = x.to(dtype)
+            pools.append(pool.to(DEV))
+        want = plain.attend(q.double(), k.double(), v.double(), 1.0, sinks)
+        assert want[loud, 0, 0] > 7.9 and abs(want[loud, 1, 0] - 4.0) < 0.1 and (loud == 0 or want[loud - 1, 0, 0] == 0)
+        for first, count in [(0, n), (150, 60)] + [(r, 1) for r in rows_at]:
+            ctx = util.make_context(ops, dtype, [(first, count)])
+            ctx.single_rows = 1 if count == 1 else 0
+            out = torch.full((count, heads * vdim), float("nan"), dtype=dtype, device=DEV)
+            ops.paged_attention(q[first:first + count].reshape(count, -1).to(dtype).to(DEV), pools[0], pools[1],
+                                _rows(tables, [0]), ctx, heads, 2, dim, ps, None, 1.0, out, vdim=vdim, sink=True,
+                                sinks=sinks.to(DEV))
+            diff = (out.double().cpu().view(count, heads, vdim) - want[first:first + count]).abs().max()
+            assert diff < (1e-4 if dtype == torch.float32 else 0.05), (loud, first, count)
+
+
 def _scan_requests(lens):
     """Cuts and slots for three requests whose state lies in a wider tensor's rows."""
     cuts = []
@@ -444,6 +481,42 @@ def test_states_remember_and_forget(ops, dtype):
         got = torch.cat(got).view(n, 2, vdim).double()
         # (a decay this close to 1 is rounded alike in every row)
         assert (got - want).abs().max() < 1e-4 * want.abs().max()
+
+
+@pytest.mark.parametrize("dtype", BOTH)
+def test_memory_keeps_a_loud_row_and_its_maximum(ops, dtype):
+    """The same for the matrix memory: one row writes loudly, hundreds of quiet ones follow, and a
+    head that does not forget hands its value back to the end, one that forgets at once does not.
+    The running maximum falls with the forget gate alone, in the state too."""
+    n, heads, dim, vdim, cap = 500, 2, 8, 16, 15.0
+    u = torch.zeros(n, 2 * heads * dim + 2 * heads * vdim)
+    u[:, :2 * heads * dim] = 1.0
+    v0 = 2 * heads * dim
+    u[:, v0:v0 + heads * vdim] = 0.01 * torch.randn(n, heads * vdim, generator=torch.Generator().manual_seed(2))
+    u[5, v0:v0 + heads * vdim] = torch.arange(heads * vdim) - 10.0
+    u = u.to(dtype)
+    z = torch.tensor([-9.0, -9.0, 60.0, -7.0]).repeat(n, 1)     # write gates, then forget gates
+    z[5, :2] = 8.0
+    zc = plain.capped(z.double(), cap)
+    q = u[:, :heads * dim].double().view(n, heads, dim) * dim ** -0.5
+    k, v = u[:, heads * dim:v0].double().view(n, heads, dim), u[:, v0:v0 + heads * vdim].double().view(n, heads, vdim)
+    o, (S, nn, m) = plain.memory(q, k, v, zc[:, :2], plain.log_sigmoid(zc[:, 2:]))
+    want = plain.unit(o, 1e-6)
+    loud = plain.unit(v[5], 1e-6)
+    assert rel_err(want[-1, 0], loud[0]) < 1e-2 and rel_err(want[-1, 1], loud[1]) > 0.5
+    zero, one = torch.zeros(2 * heads, device=DEV), torch.ones(heads * vdim, device=DEV)
+    for cut in ([n], [130, 2, 368], [128, 128, 244], _cut(n, [490], 10)):
+        state, got = torch.zeros(1, heads * (dim * vdim + dim + 1) + 2, device=DEV), []
+        for ctx, _, starts, counts in _steps(ops, dtype, [cut], [0]):
+            s, c = starts[0], counts[0]
+            part = u[s:s + c].to(DEV)
+            out = torch.empty(ctx.T, heads * vdim, dtype=dtype, device=DEV)
+            ops.matrix_memory(part, 0, heads * dim, v0, z[s:s + c].to(DEV), zero, heads, dim, vdim, cap, dim ** -0.5, state,
+                              ctx, part[:, v0 + heads * vdim:], one, 1e-6, out)
+            got.append(2 * out.float().cpu())       # (the gate's logits are 0: a factor of 1 / 2)
+        got = torch.cat(got).view(n, heads, vdim)
+        assert rel_err(got, want) < (1e-4 if dtype == torch.float32 else 5e-3), cut
+        assert (state[0, heads * dim * (vdim + 1):heads * dim * (vdim + 1) + heads].double().cpu() - m).abs().max() < 1e-3
 
 
 # ---- whole models ----------------------------------------------------------------------------
